@@ -194,9 +194,20 @@ class ModelRunner:
         m = self.model
         if self.cache_layout is not None:
             el = torch.tensor([], dtype=self.kv_dtype).element_size()
-            return max(1, sum(g * (dk + dv) for g, dk, dv in self.cache_layout) * self.bs * el)
+            return max(1, sum(g * (dk + dv) * self._page_rows(pool) * el
+                              for g, dk, dv, pool in map(self._cache_entry, self.cache_layout)))
         return (2 * m.num_local_layers * m.local_kv_heads() * self.mcfg.head_dim * self.bs *
                 torch.tensor([], dtype=self.kv_dtype).element_size())
+
+    @staticmethod
+    def _cache_entry(e) -> tuple:
+        """(kv heads, key size, value size, tokens per pooled row; 0: no pooled rows)."""
+        return tuple(e) if len(e) == 4 else (*e, 0)
+
+    def _page_rows(self, pool: int) -> int:
+        """Rows of one page of a layer's cache: its tokens, then one row for every pooled
+        block whose last token may lie in the page."""
+        return self.bs + (-(-self.bs // pool) if pool else 0)
 
     def profile_num_blocks(self, gpu_mem_util: float) -> int:
         """Run a worst-case eager prefill, measure peak activation memory, and size the
@@ -262,11 +273,12 @@ class ModelRunner:
         self._init_states()
         if self.cache_layout is not None:
             # plain row-major pages per attention layer: k [nb, G, bs, dk], v [nb, G, bs, dv]
-            # (dv = 0: the layer reads its values from columns of the key rows)
-            self.kv = [(torch.zeros(num_blocks, g, self.bs, dk, dtype=self.kv_dtype,
-                                    device=self.device),
-                        torch.zeros(num_blocks, g, self.bs, dv, dtype=self.kv_dtype,
-                                    device=self.device)) for g, dk, dv in self.cache_layout]
+            # (dv = 0: the layer reads its values from columns of the key rows); layers with
+            # pooled blocks keep the blocks' mean rows in the same pages, after the tokens
+            self.kv = [tuple(torch.zeros(num_blocks, g, self._page_rows(pool), d,
+                                         dtype=self.kv_dtype, device=self.device)
+                             for d in (dk, dv))
+                       for g, dk, dv, pool in map(self._cache_entry, self.cache_layout)]
             self.kv_caches = list(self.kv)
             self.num_blocks = num_blocks
             return
@@ -553,7 +565,7 @@ class ModelRunner:
     def _forward(self, T, meta: AttnMetadata, hidden_in=None):
         L = self.L
         ctx = ForwardContext(meta, self.kv_caches, self.cos_sin, *self.kv_scales,
-                             states=self.states)
+                             states=self.states, block_size=self.bs)
         ids = self.d64[L.ids:L.ids + T]
         pos = self.d64[L.pos:L.pos + T]
         if self.model.first:

@@ -18,6 +18,7 @@ import torch
 
 from .configs import PRESETS, ModelConfig, resolve_model
 from .dilavik import DilavikForCausalLM
+from .generax import GeneraxForCausalLM
 from .konovik import KonovikForCausalLM
 from .llama import LlamaForCausalLM
 from .lorenex import LorenexForCausalLM
@@ -36,6 +37,8 @@ def build_model(cfg: ModelConfig, dtype=torch.bfloat16, device=None):
         return NolesunForCausalLM(cfg, dtype, device)
     if cfg.arch == "lorenex":
         return LorenexForCausalLM(cfg, dtype, device)
+    if cfg.arch == "generax":
+        return GeneraxForCausalLM(cfg, dtype, device)
     return LlamaForCausalLM(cfg, dtype, device)
 
 

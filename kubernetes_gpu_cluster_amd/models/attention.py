@@ -51,6 +51,7 @@ class ForwardContext:
     v_scale: float = 1.0
     # per recurrent layer: its state tensors, one slot per running sequence
     states: Optional[list] = None
+    block_size: int = 0                                # tokens per KV page
 
 
 class PagedAttention(nn.Module):
@@ -207,7 +208,14 @@ class AttentionCore(nn.Module):
     (no bias, no activation; the last taps - 1 projected rows are per-sequence state).
     ``spec.qk_unit`` / ``spec.v_unit`` divide each head's q and k / v by its root mean square
     (v is cached so), and ``spec.q_temp`` = (coef, every) multiplies q at position p by
-    1 + coef * ln(floor((p + 1) / every) + 1); these take the place of the rotation."""
+    1 + coef * ln(floor((p + 1) / every) + 1); these take the place of the rotation.
+
+    ``spec.qk_norm`` RMS-norms the whole q and the whole k row (all heads at once) with one
+    weight per column before rotation; a learned factor per query head on the scores
+    (``spec.head_temp``) is part of the q weight.  ``spec.rotary.values`` turns the cached
+    values by their positions and each head's output back by the row's.  With
+    ``spec.window.pool`` the cache pages also hold the mean rows of blocks that have left the
+    window.  ``spec.kv_from``: the layer has q columns only and reads the cache it is given."""
 
     def __init__(self, spec, out_scale: float = 1.0, eps: float = 1e-6, device=None):
         super().__init__()
@@ -215,11 +223,21 @@ class AttentionCore(nn.Module):
         H, G, dk, dv = spec.heads, spec.kv_heads, spec.dim, spec.vdim
         assert H % G == 0, "query heads must be a multiple of key/value heads"
         assert spec.rot_dims % 2 == 0 and spec.rot_dims <= dk
-        self.n_qkv = H * dk + G * dk + G * dv
+        self.own_kv = spec.kv_from is None
+        self.n_qkv = H * dk + (G * dk + G * dv if self.own_kv else 0)
         self.n_in = self.n_qkv + (H * dv if spec.elem_gate else 0)
         self.n_out = H * dv
         self.scale = spec.dim ** -0.5 if spec.scale is None else spec.scale
         self.rope = None            # [max_pos, rot_dims] fp32, set by prepare()
+        self.v_rope = None          # [max_pos, dv] fp32 (rotated values)
+        assert self.own_kv or spec.qk_norm, "shared keys and values: qk_norm layers only"
+        one = lambda n: nn.Parameter(torch.ones(n, dtype=torch.float32, device=device),  # noqa: E731
+                                     requires_grad=False)
+        # the q weight carries the heads' score factors; the k weight only where there are keys
+        self.q_norm = one(H * dk) if spec.qk_norm else None
+        self.k_norm = one(G * dk) if spec.qk_norm and self.own_kv else None
+        self.pool = spec.window.pool if spec.window else 0
+        assert not self.pool or spec.window.size > 0
         self.unit = bool(spec.qk_unit or spec.v_unit or spec.q_temp)
         assert not (self.unit and spec.rot_dims), "unit-RMS inputs take the rotation's place"
         self.conv_w = (nn.Parameter(torch.zeros(self.n_qkv, spec.conv, dtype=torch.float32,
@@ -235,10 +253,25 @@ class AttentionCore(nn.Module):
         sp = self.spec
         if not sp.rot_dims:
             return
+        if sp.qk_norm:
+            def table(dims, base, factor):
+                key = ("linear", dims, base, factor)
+                if key not in tables:
+                    tables[key] = ops.ref.rope_table_linear(dims, max_pos, base, factor).to(device)
+                return tables[key]
+            self.rope = table(sp.rot_dims, sp.rot_base, sp.rotary.factor)
+            if sp.rotary.values:
+                self.v_rope = table(sp.vdim, sp.rot_base, 1.0)
+            return
         key = (sp.rot_dims, sp.rot_base)
         if key not in tables:
             tables[key] = ops.ref.rope_table(sp.rot_dims, max_pos, sp.rot_base).to(device)
         self.rope = tables[key]
+
+    def cache_shape(self) -> tuple:
+        """(kv heads, key size, value size, tokens per pooled row) of the layer's own cache."""
+        sp = self.spec
+        return (sp.kv_heads, sp.dim, sp.vdim, self.pool)
 
     def forward(self, proj: torch.Tensor, col0: int, positions: torch.Tensor,
                 ctx: ForwardContext, cache_idx: int, out: torch.Tensor,
@@ -248,7 +281,14 @@ class AttentionCore(nn.Module):
         qkv = proj[:, col0: col0 + self.n_qkv]
         if self.conv_w is not None:
             qkv = ops.causal_conv(qkv, self.conv_w, None, state[0], ctx.attn, False)
-        if self.unit:
+        rotary, bs = sp.rotary, ctx.block_size if self.pool else 0
+        if sp.qk_norm:
+            q = ops.qk_norm_store(qkv, positions, self.q_norm, self.k_norm, self.eps, self.rope,
+                                  self.v_rope, kc if self.own_kv else None,
+                                  vc if self.own_kv else None, ctx.attn.slot_mapping, sp.heads,
+                                  sp.kv_heads, sp.dim, sp.vdim, bs,
+                                  bool(rotary and rotary.interleaved))
+        elif self.unit:
             q = ops.norm_kv_store(qkv.float(), positions, kc, vc, ctx.attn.slot_mapping, sp.heads,
                                   sp.kv_heads, sp.dim, sp.vdim, self.eps, sp.qk_unit, sp.v_unit,
                                   sp.q_temp, proj.dtype)
@@ -260,4 +300,5 @@ class AttentionCore(nn.Module):
         g = proj[:, col0 + self.n_qkv: col0 + self.n_in] if sp.elem_gate else None
         ops.window_attention(q, kc, vc, positions, ctx.attn, self.scale, w.size if w else 0,
                              w.keep_first if w else 0, None, sp.softcap, self.out_scale, out=out,
-                             elem_gate=g)
+                             elem_gate=g, pool=self.pool, block_size=bs, v_table=self.v_rope,
+                             interleaved=bool(rotary and rotary.interleaved))

@@ -21,9 +21,11 @@ from typing import Optional
 @dataclasses.dataclass(frozen=True)
 class WindowSpec:
     """Sliding-window visibility with kept first tokens: query i sees key j when
-    j <= i and (i - j < size or j < keep_first)."""
+    j <= i and (i - j < size or j < keep_first).  ``pool`` > 0: query i also sees one mean
+    key and value for every block of ``pool`` tokens whose last token j has i - j >= size."""
     size: int
     keep_first: int = 0
+    pool: int = 0
 
 
 @dataclasses.dataclass(frozen=True)
@@ -33,11 +35,16 @@ class RotarySpec:
     (factor, original length, fast turns, slow turns): YaRN frequency interpolation --
     pairs that complete fewer than ``slow`` turns over the original length are slowed by
     ``factor``, pairs above ``fast`` turns keep their frequency, a linear ramp between --
-    and cos / sin are scaled by 0.1 ln(factor) + 1."""
+    and cos / sin are scaled by 0.1 ln(factor) + 1.  ``factor``: every frequency is divided
+    by it (linear scaling).  ``values``: the cached value of position j is turned by j over
+    all its dimensions (same base and pair layout, frequencies undivided), and a head's
+    output at position i is turned back by i."""
     dims: int
     base: float = 10000.0
     interleaved: bool = False
     yarn: Optional[tuple] = None
+    factor: float = 1.0
+    values: bool = False
 
 
 @dataclasses.dataclass(frozen=True)
@@ -96,6 +103,9 @@ class MixerSpec:
     kind "gated_delta": the gated delta rule, ``heads`` value heads over ``kv_heads``
     query / key heads, a [dim, vdim] fp32 state per head, convolutions of ``conv`` taps
     without bias on q, k and v, a per-head RMS norm and a SiLU gate after it.
+    kind "channel_delta": the gated delta rule with one decay per head and key channel,
+    exp(-exp(A_log) softplus(W_a2 W_a1 h + dt_bias)) through a bottleneck of ``decay_rank``,
+    and a per-head RMS norm followed by a sigmoid gate through a bottleneck of ``gate_rank``.
     kind "gla": gated linear attention, per head S = diag(alpha) S + k v^T, o = S^T q with a
     decay per key channel alpha = sigmoid(W_a2 W_a1 h + b)^(1 / decay_tau) through a
     bottleneck of ``decay_rank``; a per-head RMS norm and a SiLU gate after it.
@@ -138,8 +148,16 @@ class MixerSpec:
     q_temp: Optional[tuple] = None
     out_bias: Optional[bool] = None
     decay_tau: float = 1.0       # gla
-    decay_rank: int = 0
+    decay_rank: int = 0          # gla, channel_delta
+    gate_rank: int = 0           # channel_delta
     dt_rank: int = 0             # mamba
+    # attention: an RMS norm over the whole q and the whole k projection (all heads at once,
+    # one weight per column) before rotation; a learned factor per query head on the scores
+    # (``head_temp``); ``kv_from``: the layer reads that layer's cached keys and values and
+    # has none of its own
+    qk_norm: bool = False
+    head_temp: bool = False
+    kv_from: Optional[int] = None
     left: Optional["MixerSpec"] = None      # parallel
     right: Optional["MixerSpec"] = None
     left_scale: float = 1.0
@@ -202,6 +220,9 @@ class ModelConfig:
     # times ``residual_mult``; a learned position vector is added to the scaled embedding;
     # layer i runs with the weights of layer ``weights_of[i]`` (cache and state its own)
     weights_of: Optional[tuple] = None
+    # arch "generax": mixer and feed-forward of a layer read one norm's output and join the
+    # stream together; the logits pass cap * tanh(. / cap) when ``logit_softcap`` > 0
+    logit_softcap: float = 0.0
 
     @property
     def q_size(self) -> int:
@@ -252,10 +273,14 @@ class ModelConfig:
                         n += h * (3 * r.heads * r.vdim + 2 * r.kv_heads * r.dim + r.heads)
                     elif r.kind == "mamba":
                         n += 3 * h * r.width + r.width * (2 * r.dt_rank + 3 * r.dim)
+                    elif r.kind == "channel_delta":
+                        n += h * (2 * r.kv_heads * r.dim + 2 * r.heads * r.vdim + r.heads)
+                        n += r.decay_rank * (h + r.heads * r.dim) + r.gate_rank * (h + r.heads * r.vdim)
                     else:
                         n += h * (2 * r.kv_heads * r.dim + 3 * r.heads * r.vdim + 2 * r.heads)
                 elif sp.kind == "attention":
-                    n += h * (sp.heads * sp.dim + sp.kv_heads * (sp.dim + sp.vdim) + sp.heads)
+                    n += h * (sp.heads * sp.dim + (sp.heads if sp.head_gate else 0))
+                    n += h * sp.kv_heads * (sp.dim + sp.vdim) if sp.kv_from is None else 0
                 elif sp.kind == "gla":
                     n += h * (2 * sp.heads * sp.dim + 3 * sp.heads * sp.vdim)
                     n += sp.decay_rank * (h + sp.heads * sp.dim)
@@ -265,7 +290,7 @@ class ModelConfig:
                     n += sp.heads * sp.vdim * h
                 f = sp.mlp
                 if f is None:
-                    n += 2 * h * sp.ff
+                    n += 2 * h * sp.ff          # (0 when the layer has no feed-forward)
                 elif f.kind == "dense":
                     n += (2 if f.gated is False else 3) * h * f.ff
                 else:
@@ -290,9 +315,12 @@ class ModelConfig:
                 n[i] += 1
             att = [(i, sp.left if sp.kind == "parallel" else sp)
                    for i, sp in enumerate(self.layer_specs) if sp.is_attention or sp.kind == "parallel"]
-            return sum(n[i] * dtype_bytes * (sp.kv_rank + sp.rot_dims if sp.kind == "latent_attention"
-                                             else sp.kv_heads * (sp.dim + sp.vdim))
-                       for i, sp in att)
+            b = sum(n[i] * dtype_bytes * (sp.kv_rank + sp.rot_dims if sp.kind == "latent_attention"
+                                          else sp.kv_heads * (sp.dim + sp.vdim))
+                    for i, sp in att if sp.kv_from is None)
+            # one more row per pooled block
+            return b + sum(n[i] * dtype_bytes * sp.kv_heads * (sp.dim + sp.vdim) // sp.window.pool
+                           for i, sp in att if sp.window is not None and sp.window.pool)
         return 2 * self.num_layers * self.num_kv_heads * self.head_dim * dtype_bytes
 
     def shrink(self, **kw) -> "ModelConfig":
@@ -554,6 +582,54 @@ PRESETS.update({
 })
 
 
+def _generax(name: str, width: int, pattern: str, att: dict, delta: dict, ff: int,
+             vocab: int = 32000, softcap: float = 15.0) -> ModelConfig:
+    """A Generax-architecture preset: ``pattern`` is one letter per layer ("p": windowed
+    attention with pooled blocks beside the channel-wise gated delta rule, "a": rotary
+    windowed attention with rotated values, "s": the same on the keys and values of the
+    nearest "a" layer before it)."""
+    mlp = FeedForwardSpec("dense", ff, act="silu")
+    rs = RotarySpec(att["rot"], att.get("base", 1e4), factor=att.get("factor", 8.0), values=True)
+    specs, src = [], None
+    for i, c in enumerate(pattern):
+        if c == "p":
+            left = MixerSpec("attention", att["heads"], att["dim"], att["vdim"], kv_heads=att["kv"],
+                             scale=att["dim"] ** -0.5, qk_norm=True,
+                             window=WindowSpec(att["window"], pool=att["pool"]))
+            right = MixerSpec("channel_delta", delta["heads"], delta["dim"], delta["vdim"],
+                              kv_heads=delta["kv"], conv=delta.get("conv", 4),
+                              decay_rank=delta["rank"], gate_rank=delta["rank"])
+            specs.append(MixerSpec("parallel", left.heads, left.dim, left.vdim,
+                                   kv_heads=left.kv_heads, ff=ff, mlp=mlp, left=left, right=right,
+                                   left_scale=0.5, right_scale=0.5))
+            continue
+        src = i if c == "a" else src
+        specs.append(MixerSpec("attention", att["heads"], att["dim"], att["vdim"],
+                               kv_heads=att["kv"], scale=att["dim"] ** -0.5, rot_dims=rs.dims,
+                               rot_base=rs.base, rotary=rs, window=WindowSpec(att["window"]),
+                               ff=ff, mlp=mlp, qk_norm=True, head_temp=True,
+                               kv_from=None if c == "a" else src))
+    return ModelConfig(name, "generax", len(specs), width, att["heads"], att["kv"], att["dim"],
+                       ff, vocab, max_position=8192, rms_eps=1e-6, layer_specs=tuple(specs),
+                       logit_softcap=softcap, bos_token_id=1, eos_token_id=2)
+
+
+# Generax presets beside the equal-width hybrid / Llama presets above: the same number of
+# layers, 16 / 32 attention heads of 128, the Llama preset's gated feed-forward.  Every second
+# layer also carries a delta-rule recurrence as wide as the model (heads of 128 x 128).
+PRESETS.update({
+    "generax-w2048": _generax("generax-w2048", 2048, "paps" * 3,
+                              dict(heads=16, kv=4, dim=128, vdim=128, rot=128, window=1024, pool=16),
+                              dict(heads=16, kv=8, dim=128, vdim=128, rank=128), 5504),
+    "generax-w4096": _generax("generax-w4096", 4096, "paps" * 2,
+                              dict(heads=32, kv=8, dim=128, vdim=128, rot=128, window=2048, pool=16),
+                              dict(heads=32, kv=16, dim=128, vdim=128, rank=128), 14336),
+    "tiny-generax": _generax("tiny-generax", 128, "paps",
+                             dict(heads=4, kv=2, dim=32, vdim=16, rot=16, window=24, pool=4),
+                             dict(heads=4, kv=2, dim=16, vdim=16, rank=8, conv=3), 192, vocab=1024),
+})
+
+
 # HF repo basenames (lower-cased) -> preset
 _ALIASES = {
     "meta-llama-3-8b": "llama-3-8b", "meta-llama-3-8b-instruct": "llama-3-8b",
@@ -808,6 +884,98 @@ def lorenex_config(d: dict, name: str, shapes: Optional[dict] = None) -> ModelCo
         bos_token_id=int(d.get("bos_token_id", 0)), eos_token_id=int(d.get("eos_token_id", -1)))
 
 
+def _generax_ff(mlp: Optional[dict]) -> Optional[FeedForwardSpec]:
+    if not mlp:
+        return None
+    kind = mlp.get("kind", "dense")
+    if kind != "dense":
+        raise ValueError(f"unsupported feed-forward kind {kind!r}")
+    return FeedForwardSpec("dense", int(mlp["ff"]), act="silu")
+
+
+def _window_spec(mask: Optional[dict]) -> Optional[WindowSpec]:
+    if not mask:
+        return None
+    return WindowSpec(int(mask["size"]), pool=int(mask.get("pool", 0)))
+
+
+def _generax_spec(i: int, layers: list, shapes: dict) -> MixerSpec:
+    """Entry i of a Generax ``layers`` list.  Type "parallel": attention with a window and
+    pooled blocks beside the channel-wise gated delta rule; type "attention": rotary windowed
+    attention with rotated values, on its own or another layer's keys and values.  The ranks
+    of the delta rule's two bottlenecks come from the tensors' shapes (or mixer entries
+    "decay_rank" / "gate_rank")."""
+    entry = layers[i]
+    kind, m, mlp = entry["type"], entry["mixer"], _generax_ff(entry.get("mlp"))
+    ff = mlp.ff if mlp else 0
+    if kind == "attention":
+        rot, kv_from = m.get("rot"), m.get("kv_from")
+        H = int(m["heads"])
+        rs = None
+        if rot:
+            sc = rot.get("scaling") or {}
+            rs = RotarySpec(int(rot["dims"]), float(rot["base"]),
+                            factor=float(sc.get("factor", 1.0)), values=True)
+        sp = MixerSpec("attention", H, int(m["dim"]), int(m["vdim"]),
+                       kv_heads=int(m.get("kv_heads", H)), scale=float(m["scale"]),
+                       rot_dims=rs.dims if rs else 0, rot_base=rs.base if rs else 10000.0,
+                       rotary=rs, window=_window_spec(m.get("mask")), ff=ff, mlp=mlp,
+                       qk_norm=True, head_temp=True,
+                       kv_from=None if kv_from is None else int(kv_from))
+        if sp.kv_from is not None:
+            j = sp.kv_from
+            if not 0 <= j < i or layers[j]["type"] != "attention":
+                raise ValueError(f"layer {i}: kv_from must name an attention layer before it")
+            src = _generax_spec(j, layers, shapes)
+            if src.kv_from is not None:
+                raise ValueError(f"layer {i}: layer {j} has no keys and values of its own")
+            if (src.kv_heads, src.dim, src.vdim) != (sp.kv_heads, sp.dim, sp.vdim):
+                raise ValueError(f"layer {i}: head sizes differ from layer {j}'s")
+    elif kind == "parallel":
+        l, r = m["left"], m["right"]
+        H, Hr = int(l["heads"]), int(r["heads"])
+
+        def rank(entry_name, tensor):
+            if entry_name in r:
+                return int(r[entry_name])
+            shape = shapes.get(f"l{i}.mix.right.{tensor}")
+            if not shape:
+                raise ValueError(f"layer {i} needs {entry_name}: mixer.right.{entry_name} in the "
+                                 f"config, or the checkpoint whose l{i}.mix.right.{tensor} has "
+                                 f"that many rows")
+            return int(shape[0])
+        left = MixerSpec("attention", H, int(l["dim"]), int(l["vdim"]),
+                         kv_heads=int(l.get("kv_heads", H)), scale=float(l["scale"]),
+                         qk_norm=True, window=_window_spec(l.get("mask")))
+        right = MixerSpec("channel_delta", Hr, int(r["dim"]), int(r["vdim"]),
+                          kv_heads=int(r.get("kv_heads", Hr)), conv=int(r["conv"]),
+                          decay_rank=rank("decay_rank", "a1"), gate_rank=rank("gate_rank", "g1"))
+        if right.heads % right.kv_heads:
+            raise ValueError("heads must be a multiple of the key/value heads")
+        sp = MixerSpec("parallel", H, left.dim, left.vdim, kv_heads=left.kv_heads, ff=ff, mlp=mlp,
+                       left=left, right=right, left_scale=0.5, right_scale=0.5)
+    else:
+        raise ValueError(f"unknown mixer type {kind!r}")
+    if sp.heads % sp.kv_heads:
+        raise ValueError("heads must be a multiple of the key/value heads")
+    return sp
+
+
+def generax_config(d: dict, name: str, shapes: Optional[dict] = None) -> ModelConfig:
+    """A Generax config.json (``architecture``, ``width``, ``vocab``, ``layers``, ``norm``,
+    ``logit_softcap``) -> ModelConfig.  ``shapes``: tensor name -> shape of the checkpoint
+    beside it, for the sizes config.json leaves to the tensors."""
+    specs = tuple(_generax_spec(i, d["layers"], shapes or {}) for i in range(len(d["layers"])))
+    a = specs[0]
+    return ModelConfig(
+        name, "generax", len(specs), int(d["width"]), a.heads, a.kv_heads, a.dim,
+        max((sp.ff for sp in specs), default=0), int(d["vocab"]),
+        max_position=int(d.get("max_position", 8192)), rope_theta=a.rot_base,
+        rms_eps=float(d["norm"]["eps"]), layer_specs=specs,
+        logit_softcap=float(d.get("logit_softcap") or 0.0),
+        bos_token_id=int(d.get("bos_token_id", 0)), eos_token_id=int(d.get("eos_token_id", -1)))
+
+
 def _tensor_shapes(path: str) -> dict:
     """Tensor name -> shape from the headers of the safetensors files in ``path``."""
     import glob
@@ -824,6 +992,8 @@ def _tensor_shapes(path: str) -> dict:
 
 def _from_hf_config(d: dict, name: str, path: Optional[str] = None) -> ModelConfig:
     """Map an HF config.json dict onto ModelConfig."""
+    if d.get("architecture") == "Generax":
+        return generax_config(d, name, _tensor_shapes(path) if path else None)
     if d.get("architecture") == "Lorenex":
         return lorenex_config(d, name, _tensor_shapes(path) if path else None)
     if d.get("architecture") == "Nolesun":

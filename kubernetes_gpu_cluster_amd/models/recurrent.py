@@ -168,6 +168,59 @@ class GatedDeltaCore(nn.Module):
         ops.gated_rms_norm(o, g, self.norm_weight, sp.heads, self.eps, False, out)
 
 
+class ChannelDeltaCore(nn.Module):
+    """The gated delta rule with one decay per head and key channel, between its projections.
+    Its projection columns (``cols``) are q | k (kv_heads * dim each) | v (heads * vdim), one
+    write strength b per head, and the two bottlenecks a1 | g1.  q | k | v pass a causal
+    convolution without bias and SiLU; q and k become unit vectors per head, q times dim^-1/2;
+    with beta = sigmoid(b) and g = exp(-exp(A_log) softplus(W_a2 a1 + dt_bias)) per key channel:
+        S = diag(g) S;  u = beta (v - S^T k);  S = S + k u^T;  o = S^T q
+    (S [dim, vdim], fp32, per-sequence state).  Each head's o over its RMS, times a weight
+    shared by the heads, times sigmoid(W_g2 g1).  Both second projections are one launch
+    (``delta_gates``); the bottlenecks are padded to multiples of 32 columns of zeros, the
+    matrix cores' inner size."""
+
+    def __init__(self, spec, eps: float, device, dtype=torch.bfloat16):
+        super().__init__()
+        self.spec, self.eps = spec, eps
+        H, G, d, dv = spec.heads, spec.kv_heads, spec.dim, spec.vdim
+        assert H % G == 0 and spec.decay_rank >= 1 and spec.gate_rank >= 1
+        up = lambda n, m: -(-n // m) * m                                     # noqa: E731
+        self.n_conv = 2 * G * d + H * dv
+        self.ra, self.rg = up(spec.decay_rank, 32), up(spec.gate_rank, 32)
+        self.b0 = up(self.n_conv, 8)
+        self.low0 = up(self.b0 + H, 8)
+        self.n_in = self.low0 + self.ra + self.rg
+        self.n_out = H * dv
+        self.cols = {"q": (0, G * d), "k": (G * d, G * d), "v": (2 * G * d, H * dv),
+                     "b": (self.b0, H), "a1": (self.low0, spec.decay_rank),
+                     "g1": (self.low0 + self.ra, spec.gate_rank)}
+        f = lambda *s: nn.Parameter(torch.zeros(*s, dtype=torch.float32, device=device),  # noqa: E731
+                                    requires_grad=False)
+        self.conv_w = f(self.n_conv, spec.conv)
+        self.neg_a, self.dt_bias = f(H * d), f(H * d)       # -exp(A_log), per key channel
+        self.norm_weight = f(H * dv)                        # the shared weight per head
+        z = lambda *s: nn.Parameter(torch.zeros(*s, dtype=dtype, device=device),   # noqa: E731
+                                    requires_grad=False)
+        self.a2, self.g2 = z(H * d, self.ra), z(H * dv, self.rg)
+
+    def state_shapes(self) -> tuple:
+        sp = self.spec
+        return ((max(sp.conv - 1, 1), self.n_conv), (sp.heads, sp.dim, sp.vdim))
+
+    def forward(self, proj: torch.Tensor, col0: int, ctx: ForwardContext,
+                state: tuple) -> torch.Tensor:
+        """-> the gated heads [T, heads * vdim] in proj's dtype."""
+        sp = self.spec
+        cut = lambda a, n: proj[:, col0 + a: col0 + a + n]                   # noqa: E731
+        qkv = ops.causal_conv(cut(0, self.n_conv), self.conv_w, None, state[0], ctx.attn)
+        decay, gate = ops.delta_gates(cut(self.low0, self.ra + self.rg), self.a2, self.g2,
+                                      self.neg_a, self.dt_bias)
+        o = ops.channel_delta_scan(qkv, cut(self.b0, sp.heads), decay, state[1], ctx.attn,
+                                   sp.heads, sp.kv_heads, sp.dim, sp.vdim)
+        return ops.head_norm_gate(o, gate, self.norm_weight, sp.heads, self.eps, proj.dtype)
+
+
 class GLAMixer(nn.Module):
     """Gated linear attention: per head a [dim, vdim] fp32 state with one decay per key
     channel.  q = W_q h * dim^-1/2, k = W_k h, v = W_v h;

@@ -115,14 +115,20 @@ def layer_norm(x: torch.Tensor, w: torch.Tensor, b: torch.Tensor, eps: float = 1
 
 
 def silu_mul(x: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """silu(gate) * up of x [..., 2 I] = gate | up; a 2-D x and ``out`` [rows, I] may be column
+    slices of wider matrices."""
     if not _gpu(x):
-        return ref.silu_mul(x)
+        r = ref.silu_mul(x)
+        if out is None:
+            return r
+        out.copy_(r)
+        return out
     I = x.shape[-1] // 2
     x2 = x.view(-1, x.shape[-1])
     if out is None:
         out = torch.empty(x2.shape[0], I, dtype=x.dtype, device=x.device)
     _k().silu_mul(out, x2)
-    return out.view(*x.shape[:-1], I)
+    return out if x.dim() == 2 else out.view(*x.shape[:-1], I)
 
 
 # ------------------------------------------------------------------ rope + kv cache
@@ -715,13 +721,22 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
                      positions: torch.Tensor, meta, scale: float, window: int, keep_first: int,
                      gate: Optional[torch.Tensor] = None, softcap: float = 0.0,
                      out_scale: float = 1.0, out: Optional[torch.Tensor] = None,
-                     elem_gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                     elem_gate: Optional[torch.Tensor] = None, pool: int = 0,
+                     block_size: int = 0, v_table: Optional[torch.Tensor] = None,
+                     interleaved: bool = False) -> torch.Tensor:
     """Prefill chunks and decode rows of one step alike: row t sees the cached keys
     j <= p with p - j < window or j < keep_first (p = positions[t]; window <= 0: plain
     causal).  Decode padding rows (context length 0) give zeros.  ``softcap`` > 0: the
     scaled scores pass softcap * tanh(. / softcap).  The result is multiplied by
     sigmoid(``elem_gate`` [T, H * dv], a column slice of a projection) when given and by
-    ``out_scale``, and may go to ``out`` [T, H * dv], a column slice of a wider buffer."""
+    ``out_scale``, and may go to ``out`` [T, H * dv], a column slice of a wider buffer.
+
+    ``pool`` > 0: row t also sees one mean key and value per block of ``pool`` tokens that
+    lies wholly before its window.  Pages hold ``block_size`` token rows followed by
+    ceil(block_size / pool) pooled rows; the call first writes the rows of the blocks that
+    the step's tokens complete.  ``v_table`` (fp32 [max_pos, dv], cos | sin): the cached
+    values were turned by their positions, each head's output is turned back by the row's
+    (pairs (m, m + dv/2), or (2m, 2m + 1) when ``interleaved``)."""
     T, H, _ = q.shape
     dv = v_cache.shape[3]
     if not _gpu(q):
@@ -729,8 +744,12 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
         if meta.num_decodes:
             tp = meta.num_prefill_tokens
             pos[tp:tp + meta.num_decodes] = meta.decode_ctx_lens[: meta.num_decodes].long() - 1
-        r = ref.window_attention(q, k_cache, v_cache, pos, _row_tables(meta, T), scale,
-                                 window, keep_first, gate, softcap, out_scale, elem_gate)
+        rt = _row_tables(meta, T)
+        if pool > 0:
+            ref.pool_kv_rows(k_cache, v_cache, pos, meta.slot_mapping, rt, pool, block_size)
+        r = ref.window_attention(q, k_cache, v_cache, pos, rt, scale, window, keep_first, gate,
+                                 softcap, out_scale, elem_gate, pool, block_size, v_table,
+                                 interleaved)
         if out is not None:
             out.copy_(r)
             return out
@@ -749,7 +768,9 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
                           meta.decode_ctx_lens, meta.decode_block_tables, ws, wb,
                           meta.num_prefills, meta.num_decodes, meta.num_prefill_tokens,
                           scale, window, keep_first, gate, window_attention_fast(),
-                          float(softcap), float(out_scale), elem_gate)
+                          float(softcap), float(out_scale), elem_gate, int(pool),
+                          int(block_size), v_table, interleaved,
+                          meta.slot_mapping if pool > 0 else None)
     return out
 
 
@@ -1152,3 +1173,76 @@ def moe_route_softmax_all(logits: torch.Tensor, correction: torch.Tensor, k: int
     idw = torch.empty(T, dtype=torch.float32, device=logits.device)
     _k().moe_route_softmax_all(w, ids, idw, logits, correction, int(n_real))
     return w, ids, idw
+
+
+# ------------------------------------------------------------------ Generax-style decoders
+# Norms over the whole q / k projection, rotated values, pooled blocks beside a sliding window
+# (``window_attention`` with ``pool``), the gated delta rule with a decay per key channel, and
+# several sublayer results that join the residual stream in one pass.
+def residual_sum_norm(x: torch.Tensor, adds: list, w: Optional[torch.Tensor], eps: float,
+                      out_dtype: Optional[torch.dtype]) -> Optional[torch.Tensor]:
+    """x fp32 [T, W], in place: x += sum over up to three ``adds`` = (a [T, W], aw) of a, or of
+    RMS-normed a times aw where aw is given; returns RMSNorm(x) * w in out_dtype (None: no
+    output)."""
+    if not _gpu(x):
+        return ref.residual_sum_norm(x, adds, w, eps, out_dtype)
+    out = torch.empty(x.shape, dtype=out_dtype, device=x.device) if out_dtype is not None else None
+    a = list(adds) + [(None, None)] * (3 - len(adds))
+    _k().residual_sum_norm(out, x, a[0][0], a[0][1], a[1][0], a[1][1], a[2][0], a[2][1], w, eps)
+    return out
+
+
+def qk_norm_store(qkv: torch.Tensor, positions: torch.Tensor, qw: torch.Tensor,
+                  kw: Optional[torch.Tensor], eps: float, table: Optional[torch.Tensor],
+                  v_table: Optional[torch.Tensor], k_cache: Optional[torch.Tensor],
+                  v_cache: Optional[torch.Tensor], slot_mapping: torch.Tensor, H: int, G: int,
+                  dk: int, dv: int, block_size: int = 0, interleaved: bool = False) -> torch.Tensor:
+    """q [T, H, dk] from qkv [T, H dk (+ G dk + G dv)] (a column slice): normed over all heads
+    at once, weighted, rotated; with k_cache also k (likewise) and v (rotated by v_table) into
+    the paged cache.  See ``ref.qk_norm_store``."""
+    if not _gpu(qkv):
+        return ref.qk_norm_store(qkv, positions, qw, kw, eps, table, v_table, k_cache, v_cache,
+                                 slot_mapping, H, G, dk, dv, block_size, interleaved)
+    q = torch.empty(qkv.shape[0], H, dk, dtype=qkv.dtype, device=qkv.device)
+    _k().qk_norm_store(q, qkv, positions, qw, kw, table, v_table, k_cache, v_cache, slot_mapping,
+                       H, G, dk, dv, int(block_size), float(eps), interleaved)
+    return q
+
+
+def delta_gates(low: torch.Tensor, a2: torch.Tensor, g2: torch.Tensor, neg_a: torch.Tensor,
+                dt_bias: torch.Tensor) -> tuple:
+    """(decays fp32 [T, H d], output-gate pre-activations [T, H dv]) from the two bottlenecks
+    low [T, ra + rg] (a column slice): the second projections of both in one launch, the
+    decay's softplus and exponentials in its epilogue; see ``ref.delta_gates``."""
+    if not _gpu(low):
+        return ref.delta_gates(low, a2, g2, neg_a, dt_bias)
+    T = low.shape[0]
+    decay = torch.empty(T, a2.shape[0], dtype=torch.float32, device=low.device)
+    gate = torch.empty(T, g2.shape[0], dtype=low.dtype, device=low.device)
+    _k().delta_gates(decay, gate, low, a2, g2, neg_a, dt_bias)
+    return decay, gate
+
+
+def channel_delta_scan(qkv: torch.Tensor, b: torch.Tensor, decay: torch.Tensor,
+                       state: torch.Tensor, meta, H: int, G: int, d: int, dv: int) -> torch.Tensor:
+    """fp32 [T, H dv]: the gated delta rule with a decay per key channel over every step
+    sequence's rows from / into state [slots, H, d, dv]; qkv fp32 [T, 2 G d + H dv] = q | k | v,
+    b [T, H] (a column slice) write-strength pre-activations, decay fp32 [T, H d]; see
+    ``ref.channel_delta_scan``."""
+    if not _gpu(qkv):
+        return ref.channel_delta_scan(qkv, b, decay, state, ref.step_sequences(meta), H, G, d, dv)
+    out = torch.empty(qkv.shape[0], H * dv, dtype=torch.float32, device=qkv.device)
+    _k().channel_delta_scan(out, qkv, b, decay, state, meta.query_start_loc,
+                            meta.prefill_seq_lens, meta.decode_ctx_lens, meta.state_slots,
+                            meta.num_prefills, meta.num_decodes, meta.num_prefill_tokens, H, G,
+                            d, dv)
+    return out
+
+
+def logit_softcap(logits: torch.Tensor, cap: float) -> torch.Tensor:
+    """fp32 cap * tanh(logits / cap); logits [rows, V] (rows may be strided)."""
+    if not _gpu(logits):
+        return ref.logit_softcap(logits, cap)
+    out = torch.empty(logits.shape, dtype=torch.float32, device=logits.device)
+    _k().logit_softcap(out, logits, float(cap))
+    return out

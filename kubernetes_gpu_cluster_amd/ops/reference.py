@@ -456,16 +456,22 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
                      window: int, keep_first: int,
                      gate: Optional[torch.Tensor], softcap: float = 0.0,
                      out_scale: float = 1.0,
-                     elem_gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                     elem_gate: Optional[torch.Tensor] = None, pool: int = 0,
+                     block_size: int = 0, v_table: Optional[torch.Tensor] = None,
+                     interleaved: bool = False) -> torch.Tensor:
     """q [T, H, dk] (rotated; the step's k / v already stored) -> [T, H*dv].  Row t at
     position p = positions[t] attends the cached keys j <= p with p - j < window or
     j < keep_first (window <= 0: all of them) of the sequence whose block table is
     row_tables[t]; scores q.k * scale, then softcap * tanh(score / softcap) when
     softcap > 0; softmax and the weighted sum in fp32; each head's output times
     gate[t, head] (fp32) when given, the concatenated heads times sigmoid(elem_gate
-    [T, H*dv]) when given, and times out_scale."""
+    [T, H*dv]) when given, and times out_scale.  ``pool`` > 0: the row also sees the mean
+    row (``pool_kv_rows``) of every block of ``pool`` tokens that lies wholly before its
+    window; pages then hold ``block_size`` token rows followed by the pooled rows.
+    ``v_table`` [max_pos, dv] (cos | sin): each head's output is turned back by the row's
+    position (the cached values were turned by theirs)."""
     T, H, dk = q.shape
-    G, bs, dv = k_cache.shape[1], k_cache.shape[2], v_cache.shape[3]
+    G, bs, dv = k_cache.shape[1], block_size or k_cache.shape[2], v_cache.shape[3]
     out = torch.zeros(T, H, dv, dtype=torch.float32)
     for t in range(T):
         p = int(positions[t])
@@ -474,15 +480,23 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
         j = torch.arange(p + 1)
         if window > 0:
             j = j[(p - j < window) | (j < keep_first)]
-        blk = row_tables[t].long()[j // bs]
-        k = k_cache[blk, :, j % bs].float()           # [n, G, dk]
-        v = v_cache[blk, :, j % bs].float()
+        page, row = j // bs, j % bs
+        if pool > 0:
+            b = torch.arange(max(0, (p - window + 1) // pool))
+            bp, br = pooled_row(b, pool, bs)
+            page, row = torch.cat([page, bp]), torch.cat([row, br])
+        blk = row_tables[t].long()[page]
+        k = k_cache[blk, :, row].float()              # [n, G, dk]
+        v = v_cache[blk, :, row].float()
         qt = q[t].float().view(G, H // G, dk)
         s = torch.einsum("ghd,ngd->ghn", qt, k) * scale
         if softcap > 0:
             s = softcap * torch.tanh(s / softcap)
         pr = torch.softmax(s, dim=-1)
         out[t] = torch.einsum("ghn,ngv->ghv", pr, v).reshape(H, dv)
+    if v_table is not None:
+        cs = v_table[positions.long().clamp(0, v_table.shape[0] - 1)]
+        out = _rotate(out, cs[:, None, : dv // 2], -cs[:, None, dv // 2:], interleaved)
     if gate is not None:
         out = out * gate.float()[:, :, None]
     if elem_gate is not None:
@@ -961,3 +975,147 @@ def moe_route_softmax_all(logits: torch.Tensor, correction: torch.Tensor, k: int
     ident = ids >= n_real
     idw = (w * ident).sum(-1)
     return w.masked_fill(ident, 0.0), ids.to(torch.int32), idw
+
+
+# ---------------------------------------------------------------- Generax-style decoders
+# (whole-projection q / k norms, rotated values, pooled blocks in the paged cache, the gated
+# delta rule with a decay per key channel, several sublayer results joining the stream at once)
+def rope_table_linear(dims: int, max_pos: int, base: float, factor: float = 1.0) -> torch.Tensor:
+    """[max_pos, dims] fp32: cos | sin of p * base^(-2i/dims) / factor, i < dims/2.  The angles
+    are evaluated in fp64, so the table is exact to fp32 rounding at any position."""
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    f = float(base) ** (-2.0 * i / dims) / float(factor)
+    a = torch.arange(max_pos, dtype=torch.float64)[:, None] * f[None]
+    return torch.cat([a.cos(), a.sin()], dim=-1).float()
+
+
+def _rotate(x: torch.Tensor, c: torch.Tensor, s: torch.Tensor, interleaved: bool) -> torch.Tensor:
+    """Turn the first 2 * c.shape[-1] entries of x's last dimension pairwise: (u, v) ->
+    (u c - v s, v c + u s), pairs (i, i + n/2) or (2i, 2i + 1); the rest passes unchanged."""
+    r = 2 * c.shape[-1]
+    if interleaved:
+        a, b = x[..., 0:r:2], x[..., 1:r:2]
+        ab = torch.stack([a * c - b * s, b * c + a * s], dim=-1).flatten(-2)
+        return torch.cat([ab, x[..., r:]], dim=-1)
+    a, b = x[..., : r // 2], x[..., r // 2: r]
+    return torch.cat([a * c - b * s, b * c + a * s, x[..., r:]], dim=-1)
+
+
+def residual_sum_norm(x: torch.Tensor, adds: list, w: Optional[torch.Tensor], eps: float,
+                      out_dtype: Optional[torch.dtype]) -> Optional[torch.Tensor]:
+    """x (fp32, in place) += the sum over ``adds`` = [(a, aw), ...] of a, or of
+    a / rms(a) * aw where aw is given; returns x / rms(x) * w in out_dtype (None: nothing)."""
+    for a, aw in adds:
+        a = a.float()
+        if aw is not None:
+            a = a * torch.rsqrt(a.pow(2).mean(-1, keepdim=True) + eps) * aw.float()
+        x += a
+    if out_dtype is None:
+        return None
+    return (x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w.float()).to(out_dtype)
+
+
+def qk_norm_store(qkv: torch.Tensor, positions: torch.Tensor, qw: torch.Tensor,
+                  kw: Optional[torch.Tensor], eps: float, table: Optional[torch.Tensor],
+                  v_table: Optional[torch.Tensor], k_cache: Optional[torch.Tensor],
+                  v_cache: Optional[torch.Tensor], slot_mapping: torch.Tensor, H: int, G: int,
+                  dk: int, dv: int, block_size: int, interleaved: bool) -> torch.Tensor:
+    """qkv [T, H dk (+ G dk + G dv)] -> q [T, H, dk]: the whole q row (all heads at once) over
+    its root mean square, times qw [H dk], then rotated (table [max_pos, rot]: cos | sin).  With
+    k_cache: k likewise with kw, v rotated over all dv dimensions when v_table is given, both
+    stored in the paged cache at ``slot_mapping`` (< 0: no write; ``block_size`` token rows per
+    page, 0: the page's rows).  fp32 math."""
+    T = qkv.shape[0]
+    pos = positions.long()
+
+    def norm(x, w):
+        return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w.float()
+
+    def rot(x, tab):
+        if tab is None:
+            return x
+        cs = tab[pos.clamp(0, tab.shape[0] - 1)][:, None]
+        n = tab.shape[1] // 2
+        return _rotate(x, cs[..., :n], cs[..., n:], interleaved)
+    q = rot(norm(qkv[:, : H * dk].float(), qw).view(T, H, dk), table)
+    if k_cache is not None:
+        k = rot(norm(qkv[:, H * dk: (H + G) * dk].float(), kw).view(T, G, dk), table)
+        v = rot(qkv[:, (H + G) * dk: (H + G) * dk + G * dv].float().view(T, G, dv), v_table)
+        bs = block_size or k_cache.shape[2]
+        ok = slot_mapping >= 0
+        sl = slot_mapping[ok].long()
+        k_cache[sl // bs, :, sl % bs] = k[ok].to(k_cache.dtype)
+        v_cache[sl // bs, :, sl % bs] = v[ok].to(v_cache.dtype)
+    return q.to(qkv.dtype)
+
+
+def pooled_row(b, pool: int, block_size: int):
+    """(page index in the sequence, row in the page) of pooled block b: it lives in the page
+    of its last token, after the page's token rows, in block order."""
+    page = (b * pool + pool - 1) // block_size
+    return page, block_size + b - page * block_size // pool
+
+
+def pool_kv_rows(k_cache: torch.Tensor, v_cache: torch.Tensor, positions: torch.Tensor,
+                 slot_mapping: torch.Tensor, row_tables: torch.Tensor, pool: int,
+                 block_size: int) -> None:
+    """For every step token that completes a block of ``pool`` tokens (and is stored), write
+    the block's mean cached key and value into its pooled row."""
+    for t in range(positions.shape[0]):
+        p = int(positions[t])
+        if p < 0 or (p + 1) % pool or int(slot_mapping[t]) < 0:
+            continue
+        j = torch.arange(p + 1 - pool, p + 1)
+        blk = row_tables[t].long()[j // block_size]
+        page, row = pooled_row(p // pool, pool, block_size)
+        dst = int(row_tables[t][page])
+        for c in (k_cache, v_cache):
+            c[dst, :, row] = c[blk, :, j % block_size].float().mean(0).to(c.dtype)
+
+
+def delta_gates(low: torch.Tensor, a2: torch.Tensor, g2: torch.Tensor, neg_a: torch.Tensor,
+                dt_bias: torch.Tensor) -> tuple:
+    """low [T, ra + rg] (the two bottlenecks side by side), a2 [H d, ra], g2 [H dv, rg], neg_a
+    and dt_bias fp32 [H d] -> (decays fp32 [T, H d] = exp(neg_a softplus(a2 low_a + dt_bias)),
+    gate pre-activations [T, H dv] = g2 low_g in low's dtype)."""
+    ra = a2.shape[1]
+    z = low[:, :ra].float() @ a2.float().t() + dt_bias.float()
+    decay = torch.exp(neg_a.float() * torch.nn.functional.softplus(z))
+    return decay, (low[:, ra:].float() @ g2.float().t()).to(low.dtype)
+
+
+def channel_delta_scan(qkv: torch.Tensor, b: torch.Tensor, decay: torch.Tensor,
+                       state: torch.Tensor, seqs: list, H: int, G: int, d: int,
+                       dv: int) -> torch.Tensor:
+    """The gated delta rule with a decay per key channel.  qkv fp32 [T, 2 G d + H dv] = q | k | v
+    (after convolution and SiLU), b [T, H] write-strength pre-activations, decay fp32 [T, H d].
+    q and k become unit vectors per head (x / sqrt(sum x^2 + 1e-6)), q times d^-1/2.  Per head h
+    (q / k head h // (H / G)), with beta = sigmoid(b):
+        S = diag(decay) S;  u = beta (v - S^T k);  S = S + k u^T;  o = S^T q         (S [d, dv])
+    from state[slot] [H, d, dv] fp32 (zeros at position 0), written back.  -> fp32 [T, H dv]."""
+    T = qkv.shape[0]
+    q = qkv[:, : G * d].float().view(T, G, d)
+    k = qkv[:, G * d: 2 * G * d].float().view(T, G, d)
+    v = qkv[:, 2 * G * d: 2 * G * d + H * dv].float().view(T, H, dv)
+    q = q * torch.rsqrt(q.pow(2).sum(-1, keepdim=True) + 1e-6) * d ** -0.5
+    k = k * torch.rsqrt(k.pow(2).sum(-1, keepdim=True) + 1e-6)
+    q, k = q.repeat_interleave(H // G, dim=1), k.repeat_interleave(H // G, dim=1)
+    beta = torch.sigmoid(b.float())
+    g = decay.view(T, H, d)
+    out = torch.zeros(T, H, dv, dtype=torch.float32)
+    for a, n, p0, slot in seqs:
+        if slot < 0:
+            continue
+        S = torch.zeros(H, d, dv) if p0 == 0 else state[slot].clone()
+        for t in range(a, a + n):
+            S = g[t][:, :, None] * S
+            u = beta[t, :, None] * (v[t] - torch.einsum("hdv,hd->hv", S, k[t]))
+            S = S + k[t][:, :, None] * u[:, None, :]
+            out[t] = torch.einsum("hdv,hd->hv", S, q[t])
+        state[slot] = S
+    return out.view(T, H * dv)
+
+
+def logit_softcap(logits: torch.Tensor, cap: float) -> torch.Tensor:
+    """fp32 cap * tanh(logits / cap)."""
+    return cap * torch.tanh(logits.float() / cap)
