@@ -78,11 +78,14 @@ void layer_norm(Tensor out, Tensor x, Tensor w, Tensor b, double eps) {
 void silu_mul(Tensor out, Tensor x) {
   check_gpu(x, "x");
   c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
-  TORCH_CHECK(x.dim() == 2 && x.is_contiguous() && out.is_contiguous(), "kgc.silu_mul: contiguous 2-D");
+  // rows of both may be column slices of wider matrices
+  TORCH_CHECK(x.dim() == 2 && x.stride(1) == 1 && out.dim() == 2 && out.stride(1) == 1 &&
+              out.device() == x.device(), "kgc.silu_mul: 2-D, unit column stride");
   const int64_t I = x.size(1) / 2;
   TORCH_CHECK(x.size(1) % 2 == 0 && out.size(0) == x.size(0) && out.size(1) == I &&
               out.scalar_type() == x.scalar_type() && act_dtype(x), "kgc.silu_mul: shapes / dtypes");
-  kgc::launch_silu_mul(dt_code(x), out.data_ptr(), x.data_ptr(), x.size(0), (int)I, stream());
+  kgc::launch_silu_mul(dt_code(x), out.data_ptr(), out.stride(0), x.data_ptr(), x.stride(0),
+                       x.size(0), (int)I, stream());
 }
 
 // KV cache element type: the activation dtype, or fp8 e4m3 (--kv-cache-dtype fp8)
@@ -1363,6 +1366,13 @@ void rope_kv_store(Tensor qkv, Tensor positions, std::optional<Tensor> table, Te
                             (int)k_cache.size(2), (int)k_cache.size(0), interleaved, stream());
 }
 
+const float* f32_opt(const std::optional<Tensor>& t, int64_t numel, const char* name) {
+  if (!t.has_value()) return nullptr;
+  check_f32(*t, name);
+  TORCH_CHECK(t->numel() == numel, "kgc: ", name, " must have ", numel, " entries");
+  return t->data_ptr<float>();
+}
+
 const int* i32_ptr(const std::optional<Tensor>& t, int64_t min_numel, const char* name) {
   if (!t.has_value()) {
     TORCH_CHECK(min_numel == 0, "kgc: ", name, " missing");
@@ -1388,7 +1398,9 @@ void window_attention(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
                       std::optional<Tensor> work_blk, int64_t P, int64_t D, int64_t Tp,
                       double scale, int64_t window, int64_t keep_first,
                       std::optional<Tensor> gate, bool fast, double softcap, double out_scale,
-                      std::optional<Tensor> elem_gate) {
+                      std::optional<Tensor> elem_gate, int64_t pool, int64_t block_size,
+                      std::optional<Tensor> v_table, bool interleaved,
+                      std::optional<Tensor> slots) {
   check_gpu(q, "q");
   c10::hip::HIPGuardMasqueradingAsCUDA g(q.device());
   TORCH_CHECK(q.dim() == 3 && q.is_contiguous() && act_dtype(q), "kgc.window_attention: q [T, H, dk]");
@@ -1432,8 +1444,28 @@ void window_attention(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
     egp = elem_gate->data_ptr();
     egs = elem_gate->stride(0);
   }
+  // pooled blocks: a page holds bs token rows, then one row per block that ends in it
+  const int prow = (int)k_cache.size(2);
+  const int bs = pool > 0 ? (int)block_size : prow;
+  if (pool > 0)
+    TORCH_CHECK(window > 0 && keep_first == 0 && bs >= 1 && pool < (int64_t(1) << 24) &&
+                prow == bs + (bs + pool - 1) / pool && v_cache.is_contiguous() &&
+                slots.has_value() && slots->is_cuda() && slots->scalar_type() == at::kLong &&
+                slots->numel() >= T && slots->is_contiguous(),
+                "kgc.window_attention: pooled blocks need a window, no kept first tokens, pages of "
+                "block_size + ceil(block_size / pool) rows and the step's slots");
+  const float* vtp = nullptr;
+  int64_t vrows = 0;
+  if (v_table.has_value()) {
+    check_f32(*v_table, "v_table");
+    TORCH_CHECK(v_table->dim() == 2 && v_table->is_contiguous() && v_table->size(1) == dv &&
+                dv % 2 == 0 && v_table->size(0) >= 1 && v_table->device() == q.device(),
+                "kgc.window_attention: v_table [max_pos, dv]");
+    vtp = v_table->data_ptr<float>();
+    vrows = v_table->size(0);
+  }
   const kgc::WindowExtra ex{T > 1 ? out.stride(0) : H * dv, (float)softcap, (float)out_scale, egp,
-                            egs};
+                            egs, (int)pool, prow, vtp, (int)vrows, interleaved};
   // the matrix-core kernel stores 8-byte pieces of a row
   const bool out_vec = reinterpret_cast<uintptr_t>(out.data_ptr()) % 8 == 0 &&
                        ex.ors * out.element_size() % 8 == 0;
@@ -1452,10 +1484,20 @@ void window_attention(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
   const int* pp = i32_ptr(pbt, P, "prefill block tables");
   const int* cp = i32_ptr(ctx_lens, D, "ctx_lens");
   const int* dp = i32_ptr(dbt, D, "decode block tables");
-  const int bs = (int)k_cache.size(2), nb = (int)k_cache.size(0), dt = dt_code(q);
+  const int nb = (int)k_cache.size(0), dt = dt_code(q);
   int rest = 3;                   // row kinds the one-wave kernel still has to run
+  const bool decode_fast = fast && aligned && D > 0 &&
+                           kgc::window_decode_ok((int)dk, (int)dv, (int)(H / G)) &&
+                           kgc::window_decode_lds((int)dk, (int)dv, (int)(H / G)) <= 64 * 1024;
+  if (pool > 0) {                 // (the decode kernel pools its own rows)
+    const int rows = (int)(Tp + (decode_fast ? 0 : D));
+    kgc::launch_pool_kv(dt, k_cache.data_ptr(), v_cache.data_ptr(), slots->data_ptr<int64_t>(), qp,
+                        sp, pp, cp, dp, (int)bts, (int)P, (int)Tp, 0, rows, (int)G, (int)dk,
+                        (int)dv, (int)krs, (int)vrs, bs, prow, nb, (int)pool, stream());
+  }
   if (fast && aligned && out_vec && P > 0 && work_seq.has_value() && work_blk.has_value() &&
-      kgc::window_prefill_mfma_ok(dt, (int)dk, (int)dv)) {
+      kgc::window_prefill_mfma_ok(dt, (int)dk, (int)dv) &&
+      (vtp == nullptr || interleaved || dv % 32 == 0)) {   // a pair within one lane
     const int64_t nw = work_seq->numel();
     TORCH_CHECK(work_blk->numel() == nw && work_seq->scalar_type() == at::kInt &&
                 work_blk->scalar_type() == at::kInt && work_seq->is_cuda() && work_blk->is_cuda(),
@@ -1468,8 +1510,7 @@ void window_attention(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
                                     stream());
     rest &= ~1;
   }
-  if (fast && aligned && D > 0 && kgc::window_decode_ok((int)dk, (int)dv, (int)(H / G)) &&
-      kgc::window_decode_lds((int)dk, (int)dv, (int)(H / G)) <= 64 * 1024) {
+  if (decode_fast) {
     kgc::launch_window_decode(dt, out.data_ptr(), q.data_ptr(), k_cache.data_ptr(),
                               v_cache.data_ptr(), cp, dp, (int)bts, (int)Tp, (int)D, (int)H,
                               (int)G, (int)dk, (int)dv, (int)krs, (int)vrs, bs, nb, (float)scale,
@@ -1482,6 +1523,66 @@ void window_attention(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
                                v_cache.data_ptr(), qp, sp, pp, cp, dp, (int)bts, (int)P, (int)Tp,
                                (int)T, (int)H, (int)G, (int)dk, (int)dv, (int)krs, (int)vrs, bs, nb,
                                (float)scale, (int)window, (int)keep_first, gp, rest, ex, stream());
+}
+
+void qk_norm_store(Tensor q_out, Tensor qkv, Tensor positions, Tensor qw, std::optional<Tensor> kw,
+                   std::optional<Tensor> table, std::optional<Tensor> v_table,
+                   std::optional<Tensor> k_cache, std::optional<Tensor> v_cache, Tensor slots,
+                   int64_t H, int64_t G, int64_t dk, int64_t dv, int64_t block_size, double eps,
+                   bool interleaved) {
+  check_gpu(qkv, "qkv");
+  c10::hip::HIPGuardMasqueradingAsCUDA g(qkv.device());
+  const bool kv = k_cache.has_value();
+  TORCH_CHECK(H >= 1 && G >= 1 && dk >= 1 && dv >= 1 && kgc::qk_norm_store_ok((int)H, (int)G, (int)dk, (int)dv),
+              "kgc.qk_norm_store: head sizes");
+  TORCH_CHECK(qkv.dim() == 2 && qkv.stride(1) == 1 && act_dtype(qkv) &&
+              qkv.size(1) >= H * dk + (kv ? G * (dk + dv) : 0),
+              "kgc.qk_norm_store: qkv [T, H dk (+ G dk + G dv)]");
+  const int64_t T = qkv.size(0);
+  TORCH_CHECK(q_out.is_cuda() && q_out.device() == qkv.device() && q_out.is_contiguous() &&
+              q_out.numel() == T * H * dk && q_out.scalar_type() == qkv.scalar_type(),
+              "kgc.qk_norm_store: q_out");
+  TORCH_CHECK(positions.scalar_type() == at::kLong && positions.numel() == T &&
+              positions.is_contiguous() && slots.scalar_type() == at::kLong &&
+              slots.numel() == T && slots.is_contiguous() && positions.is_cuda() && slots.is_cuda(),
+              "kgc.qk_norm_store: positions / slots int64 [T]");
+  const float *tp = nullptr, *vp = nullptr, *kwp = nullptr;
+  int64_t rot = 0, rows = 0, vrows = 0;
+  if (table.has_value()) {
+    check_f32(*table, "table");
+    TORCH_CHECK(table->dim() == 2 && table->is_contiguous() && table->size(1) % 2 == 0 &&
+                table->size(1) <= dk && table->size(0) >= 1 && table->device() == qkv.device(),
+                "kgc.qk_norm_store: table [max_pos, rot]");
+    tp = table->data_ptr<float>();
+    rot = table->size(1);
+    rows = table->size(0);
+  }
+  void *kp = nullptr, *vcp = nullptr;
+  int bs = 1, prow = 1, nb = 0;
+  if (kv) {
+    TORCH_CHECK(v_cache.has_value() && kw.has_value(), "kgc.qk_norm_store: k needs v and a weight");
+    check_plain_cache(*k_cache, *v_cache, qkv, G, dk, dv);
+    kwp = f32_opt(kw, G * dk, "kw");
+    kp = k_cache->data_ptr();
+    vcp = v_cache->data_ptr();
+    prow = (int)k_cache->size(2);
+    bs = block_size > 0 ? (int)block_size : prow;
+    TORCH_CHECK(bs <= prow, "kgc.qk_norm_store: block_size");
+    nb = (int)k_cache->size(0);
+    if (v_table.has_value()) {
+      check_f32(*v_table, "v_table");
+      TORCH_CHECK(v_table->dim() == 2 && v_table->is_contiguous() && v_table->size(1) == dv &&
+                  dv % 2 == 0 && v_table->size(0) >= 1 && v_table->device() == qkv.device(),
+                  "kgc.qk_norm_store: v_table [max_pos, dv]");
+      vp = v_table->data_ptr<float>();
+      vrows = v_table->size(0);
+    }
+  }
+  kgc::launch_qk_norm_store(dt_code(qkv), q_out.data_ptr(), qkv.data_ptr(), qkv.stride(0),
+                            positions.data_ptr<int64_t>(), f32_opt(qw, H * dk, "qw"), kwp, tp,
+                            (int)rot, (int)rows, vp, (int)vrows, kp, vcp,
+                            slots.data_ptr<int64_t>(), (int)T, (int)H, (int)G, (int)dk, (int)dv,
+                            bs, prow, nb, (float)eps, interleaved, stream());
 }
 
 void mlstm_scan(Tensor out, Tensor qkvg, Tensor gates, Tensor S, Tensor n, Tensor m,
@@ -1514,13 +1615,6 @@ void mlstm_scan(Tensor out, Tensor qkvg, Tensor gates, Tensor S, Tensor n, Tenso
 }
 
 // ---- scaled residual stream, token shift, minGRU, latent attention rows, sigmoid routing --
-const float* f32_opt(const std::optional<Tensor>& t, int64_t numel, const char* name) {
-  if (!t.has_value()) return nullptr;
-  check_f32(*t, name);
-  TORCH_CHECK(t->numel() == numel, "kgc: ", name, " must have ", numel, " entries");
-  return t->data_ptr<float>();
-}
-
 // ---- parallel mixers: convolution state, Mamba-2, gated delta rule, gated RMS norm ----------
 void check_step(const char* op, int64_t T, int64_t P, int64_t D, int64_t Tp) {
   TORCH_CHECK(Tp + D == T && P >= 0 && D >= 0 && (P > 0) == (Tp > 0), "kgc.", op, ": step counts");
@@ -2096,9 +2190,124 @@ void moe_finish(Tensor out, std::optional<Tensor> routed, std::optional<Tensor> 
                          (int)k, (int)W, stream());
 }
 
+// ---- Generax-style decoders: several results joining the stream, channel-wise delta rule -----
+void residual_sum_norm(std::optional<Tensor> out, Tensor x, std::optional<Tensor> a0,
+                       std::optional<Tensor> w0, std::optional<Tensor> a1, std::optional<Tensor> w1,
+                       std::optional<Tensor> a2, std::optional<Tensor> w2, std::optional<Tensor> w,
+                       double eps) {
+  check_f32(x, "x");
+  c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
+  TORCH_CHECK(x.dim() == 2 && x.is_contiguous(), "kgc.residual_sum_norm: x [rows, W]");
+  const int64_t rows = x.size(0), W = x.size(1);
+  int dt = kgc::DT_F32, odt = kgc::DT_F32;
+  kgc::ResidualAdds adds{};
+  const std::optional<Tensor>*as[3] = {&a0, &a1, &a2}, *ws[3] = {&w0, &w1, &w2};
+  for (int j = 0; j < 3; ++j) {
+    const auto& a = *as[j];
+    TORCH_CHECK(a.has_value() || !ws[j]->has_value(), "kgc.residual_sum_norm: weight without addend");
+    if (!a.has_value()) continue;
+    TORCH_CHECK(j == 0 || as[j - 1]->has_value(), "kgc.residual_sum_norm: addends come first");
+    TORCH_CHECK(a->is_cuda() && a->is_contiguous() && a->sizes() == x.sizes() && act_dtype(*a) &&
+                a->device() == x.device() && (j == 0 || dt_code(*a) == dt),
+                "kgc.residual_sum_norm: addends [rows, W] of one dtype");
+    dt = dt_code(*a);
+    adds.a[j] = a->data_ptr();
+    adds.w[j] = f32_opt(*ws[j], W, "addend weight");
+  }
+  void* op = nullptr;
+  if (out.has_value()) {
+    TORCH_CHECK(out->is_cuda() && out->is_contiguous() && out->sizes() == x.sizes() &&
+                act_dtype(*out) && out->device() == x.device() && w.has_value() &&
+                out->data_ptr() != x.data_ptr(), "kgc.residual_sum_norm: out, w");
+    odt = dt_code(*out);
+    if (!a0.has_value()) dt = odt;
+    TORCH_CHECK(odt == kgc::DT_F32 || odt == dt,
+                "kgc.residual_sum_norm: out is fp32 or of the addends' dtype");
+    op = out->data_ptr();
+  }
+  kgc::launch_residual_sum_norm(dt, odt, op, x.data_ptr<float>(), adds, f32_opt(w, W, "w"),
+                                (int)rows, (int)W, (float)eps, stream());
+}
+
+void delta_gates(Tensor decay, Tensor gate, Tensor low, Tensor a2, Tensor g2, Tensor neg_a,
+                 Tensor dt_bias) {
+  check_gpu(low, "low");
+  check_f32(decay, "decay");
+  c10::hip::HIPGuardMasqueradingAsCUDA g(low.device());
+  const int64_t T = low.size(0);
+  TORCH_CHECK(a2.dim() == 2 && g2.dim() == 2 && a2.is_contiguous() && g2.is_contiguous() &&
+              a2.device() == low.device() && g2.device() == low.device() &&
+              a2.scalar_type() == low.scalar_type() && g2.scalar_type() == low.scalar_type(),
+              "kgc.delta_gates: a2 [H d, ra], g2 [H dv, rg] of low's dtype");
+  const int64_t Nd = a2.size(0), ra = a2.size(1), Ng = g2.size(0), rg = g2.size(1);
+  TORCH_CHECK(Nd >= 1 && Ng >= 1 && ra >= 1 && rg >= 1, "kgc.delta_gates: sizes");
+  check_cols(low, T, ra + rg, low, "low");
+  TORCH_CHECK(decay.is_contiguous() && decay.numel() == T * Nd && decay.device() == low.device() &&
+              gate.is_contiguous() && gate.numel() == T * Ng && gate.device() == low.device() &&
+              gate.scalar_type() == low.scalar_type(), "kgc.delta_gates: decay [T, H d], gate [T, H dv]");
+  kgc::launch_delta_gates(dt_code(low), decay.data_ptr<float>(), gate.data_ptr(), low.data_ptr(),
+                          low.stride(0), a2.data_ptr(), g2.data_ptr(), f32_opt(neg_a, Nd, "neg_a"),
+                          f32_opt(dt_bias, Nd, "dt_bias"), (int)T, (int)Nd, (int)Ng, (int)ra,
+                          (int)rg, stream());
+}
+
+void channel_delta_scan(Tensor out, Tensor qkv, Tensor b, Tensor decay, Tensor S,
+                        std::optional<Tensor> qsl, std::optional<Tensor> seq_lens,
+                        std::optional<Tensor> ctx_lens, Tensor slots, int64_t P, int64_t D,
+                        int64_t Tp, int64_t H, int64_t G, int64_t d, int64_t V) {
+  check_gpu(qkv, "qkv");
+  check_f32(out, "out");
+  check_f32(qkv, "qkv");
+  check_f32(decay, "decay");
+  check_f32(S, "S");
+  c10::hip::HIPGuardMasqueradingAsCUDA g(qkv.device());
+  TORCH_CHECK(H >= 1 && H <= 65535 && G >= 1 && H % G == 0 && V >= 1 && d >= 1 &&
+              d <= kgc::channel_delta_max_rows(), "kgc.channel_delta_scan: head sizes (d <= 256)");
+  TORCH_CHECK(qkv.dim() == 2 && qkv.is_contiguous() && qkv.size(1) == 2 * G * d + H * V,
+              "kgc.channel_delta_scan: qkv [T, 2 G d + H V]");
+  const int64_t T = qkv.size(0);
+  check_step("channel_delta_scan", T, P, D, Tp);
+  check_cols(b, T, H, qkv, "b");
+  TORCH_CHECK(decay.is_contiguous() && decay.numel() == T * H * d && decay.device() == qkv.device(),
+              "kgc.channel_delta_scan: decay [T, H d]");
+  TORCH_CHECK(out.is_contiguous() && out.numel() == T * H * V && out.device() == qkv.device(),
+              "kgc.channel_delta_scan: out [T, H V]");
+  TORCH_CHECK(S.is_contiguous() && S.dim() == 4 && S.size(1) == H && S.size(2) == d &&
+              S.size(3) == V && S.device() == qkv.device(),
+              "kgc.channel_delta_scan: state [slots, H, d, V]");
+  kgc::launch_channel_delta_scan(dt_code(b), out.data_ptr<float>(), qkv.data_ptr<float>(),
+                                 b.data_ptr(), b.stride(0), decay.data_ptr<float>(),
+                                 S.data_ptr<float>(), i32_ptr(qsl, P ? P + 1 : 0, "query_start_loc"),
+                                 i32_ptr(seq_lens, P, "seq_lens"), i32_ptr(ctx_lens, D, "ctx_lens"),
+                                 i32_ptr(slots, P + D, "state slots"), (int)P, (int)D, (int)Tp,
+                                 (int)H, (int)G, (int)d, (int)V, (int)S.size(0), stream());
+}
+
+void logit_softcap(Tensor out, Tensor x, double cap) {
+  check_gpu(x, "x");
+  check_f32(out, "out");
+  c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
+  TORCH_CHECK(x.dim() == 2 && x.stride(1) == 1 && act_dtype(x) && out.is_contiguous() &&
+              out.sizes() == x.sizes() && out.device() == x.device() && cap > 0,
+              "kgc.logit_softcap: x, fp32 out [rows, V], cap > 0");
+  kgc::launch_logit_softcap(dt_code(x), out.data_ptr<float>(), x.data_ptr(), x.stride(0), x.size(0),
+                            (int)x.size(1), (float)cap, stream());
+}
+
 }  // namespace
 
 TORCH_LIBRARY(kgc, m) {
+  m.def("residual_sum_norm(Tensor(a!)? out, Tensor(b!) x, Tensor? a0, Tensor? w0, Tensor? a1, "
+        "Tensor? w1, Tensor? a2, Tensor? w2, Tensor? w, float eps) -> ()");
+  m.def("qk_norm_store(Tensor(a!) q_out, Tensor qkv, Tensor positions, Tensor qw, Tensor? kw, "
+        "Tensor? table, Tensor? v_table, Tensor(b!)? k_cache, Tensor(c!)? v_cache, Tensor slots, "
+        "int H, int G, int dk, int dv, int block_size, float eps, bool interleaved) -> ()");
+  m.def("delta_gates(Tensor(a!) decay, Tensor(b!) gate, Tensor low, Tensor a2, Tensor g2, "
+        "Tensor neg_a, Tensor dt_bias) -> ()");
+  m.def("channel_delta_scan(Tensor(a!) out, Tensor qkv, Tensor b, Tensor decay, Tensor(b!) S, "
+        "Tensor? qsl, Tensor? seq_lens, Tensor? ctx_lens, Tensor slots, int P, int D, int Tp, "
+        "int H, int G, int d, int V) -> ()");
+  m.def("logit_softcap(Tensor(a!) out, Tensor x, float cap) -> ()");
   m.def("gla_scan(Tensor(a!) out, Tensor proj, Tensor low, Tensor a2, Tensor a2_bias, Tensor(b!) S, "
         "Tensor? qsl, Tensor? seq_lens, Tensor? ctx_lens, Tensor slots, int P, int D, int Tp, int H, "
         "int d, int V, float tau) -> ()");
@@ -2150,10 +2359,11 @@ TORCH_LIBRARY(kgc, m) {
         "float cap) -> ()");
   m.def("rope_kv_store(Tensor qkv, Tensor positions, Tensor? table, Tensor(a!) q_out, Tensor(b!) k_cache, "
         "Tensor(c!) v_cache, Tensor slots, int H, int G, int dk, int dv, bool interleaved) -> ()");
-  m.def("window_attention(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor? qsl, "
+  m.def("window_attention(Tensor(a!) out, Tensor q, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor? qsl, "
         "Tensor? seq_lens, Tensor? pbt, Tensor? ctx_lens, Tensor? dbt, Tensor? work_seq, Tensor? work_blk, "
         "int P, int D, int Tp, float scale, int window, int keep_first, Tensor? gate, bool fast, "
-        "float softcap, float out_scale, Tensor? elem_gate) -> ()");
+        "float softcap, float out_scale, Tensor? elem_gate, int pool, int block_size, "
+        "Tensor? v_table, bool interleaved, Tensor? slots) -> ()");
   m.def("mlstm_scan(Tensor(a!) out, Tensor qkvg, Tensor gates, Tensor(b!) S, Tensor(c!) n, Tensor(d!) m, "
         "Tensor? qsl, Tensor? seq_lens, Tensor? ctx_lens, Tensor slots, int P, int D, int Tp, int H, int d, "
         "int dv) -> ()");
@@ -2268,6 +2478,11 @@ TORCH_LIBRARY_IMPL(kgc, CUDA, m) {
   m.impl("gla_scan", &gla_scan);
   m.impl("selective_scan", &selective_scan);
   m.impl("norm_kv_store", &norm_kv_store);
+  m.impl("residual_sum_norm", &residual_sum_norm);
+  m.impl("qk_norm_store", &qk_norm_store);
+  m.impl("delta_gates", &delta_gates);
+  m.impl("channel_delta_scan", &channel_delta_scan);
+  m.impl("logit_softcap", &logit_softcap);
   m.impl("polynorm", &polynorm);
   m.impl("swiglu_clamp", &swiglu_clamp);
   m.impl("embed_pos", &embed_pos);

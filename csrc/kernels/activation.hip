@@ -6,14 +6,15 @@
 
 namespace kgc {
 
-// grid (ceil(I/8/256), rows): one 16-byte vector per thread, no index division
+// grid (ceil(I/8/256), rows): one 16-byte vector per thread, no index division.  Rows of x and
+// out may be column slices of wider matrices (strides xs, os).
 template <typename T>
-__global__ __launch_bounds__(256) void silu_mul_kernel(T* __restrict__ out,
-                                                       const T* __restrict__ x, int I) {
+__global__ __launch_bounds__(256) void silu_mul_kernel(T* __restrict__ out, int64_t os,
+                                                       const T* __restrict__ x, int64_t xs, int I) {
   const int c = blockIdx.x * 256 + threadIdx.x;
   if (c * 8 >= I) return;
   const int64_t r = blockIdx.y;
-  const T* xr = x + r * 2 * I;
+  const T* xr = x + r * xs;
   Pack8<T> g, u, o;
   g.u = *reinterpret_cast<const u32x4*>(xr + c * 8);
   u.u = *reinterpret_cast<const u32x4*>(xr + I + c * 8);
@@ -22,45 +23,69 @@ __global__ __launch_bounds__(256) void silu_mul_kernel(T* __restrict__ out,
     const float gf = to_f(g.h[j]);
     o.h[j] = from_f<T>(gf / (1.f + __expf(-gf)) * to_f(u.h[j]));
   }
-  *reinterpret_cast<u32x4*>(out + r * I + c * 8) = o.u;
+  *reinterpret_cast<u32x4*>(out + r * os + c * 8) = o.u;
 }
 
-// any element type and any I (fp32 activations, intermediate sizes that are no multiple of 8)
+// any element type, any I and any alignment
 template <typename T>
-__global__ __launch_bounds__(256) void silu_mul_any_kernel(T* __restrict__ out,
-                                                           const T* __restrict__ x, int I) {
+__global__ __launch_bounds__(256) void silu_mul_any_kernel(T* __restrict__ out, int64_t os,
+                                                           const T* __restrict__ x, int64_t xs,
+                                                           int I) {
   const int64_t r = blockIdx.y;
-  const T* xr = x + r * 2 * I;
+  const T* xr = x + r * xs;
   for (int c = blockIdx.x * 256 + threadIdx.x; c < I; c += gridDim.x * 256) {
     const float gf = to_f(xr[c]);
-    out[r * I + c] = from_f<T>(gf / (1.f + expf(-gf)) * to_f(xr[I + c]));
+    out[r * os + c] = from_f<T>(gf / (1.f + expf(-gf)) * to_f(xr[I + c]));
   }
 }
 
-void launch_silu_mul(int dtype, void* out, const void* x, int64_t rows, int I, hipStream_t s) {
-  if (dtype == DT_F32 || (I & 7)) {
-    for (int64_t r0 = 0; r0 < rows; r0 += 65535) {
-      const int64_t n = std::min<int64_t>(rows - r0, 65535);
-      const dim3 grid(std::min((I + 255) / 256, 64), (unsigned)n);
-      if (dtype == DT_F32)
-        silu_mul_any_kernel<float><<<grid, 256, 0, s>>>((float*)out + r0 * I,
-                                                        (const float*)x + r0 * 2 * I, I);
-      else if (dtype == DT_BF16)
-        silu_mul_any_kernel<bf16><<<grid, 256, 0, s>>>((bf16*)out + r0 * I,
-                                                       (const bf16*)x + r0 * 2 * I, I);
-      else
-        silu_mul_any_kernel<f16><<<grid, 256, 0, s>>>((f16*)out + r0 * I,
-                                                      (const f16*)x + r0 * 2 * I, I);
-    }
-    return;
-  }
+template <typename T>
+static void silu_mul_rows(T* out, int64_t os, const T* x, int64_t xs, int64_t rows, int I,
+                          hipStream_t s) {
+  bool vec = !std::is_same_v<T, float> && I % 8 == 0 && xs % 8 == 0 && os % 8 == 0 &&
+             reinterpret_cast<uintptr_t>(x) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0;
   for (int64_t r0 = 0; r0 < rows; r0 += 65535) {   // gridDim.y <= 65535
-    const int64_t n = std::min<int64_t>(rows - r0, 65535);
-    const dim3 grid(((I >> 3) + 255) / 256, (unsigned)n);
+    const unsigned n = (unsigned)std::min<int64_t>(rows - r0, 65535);
+    if constexpr (!std::is_same_v<T, float>) {
+      if (vec) {
+        silu_mul_kernel<T><<<dim3(((I >> 3) + 255) / 256, n), 256, 0, s>>>(
+            out + r0 * os, os, x + r0 * xs, xs, I);
+        continue;
+      }
+    }
+    silu_mul_any_kernel<T><<<dim3(std::min((I + 255) / 256, 64), n), 256, 0, s>>>(
+        out + r0 * os, os, x + r0 * xs, xs, I);
+  }
+}
+
+void launch_silu_mul(int dtype, void* out, int64_t os, const void* x, int64_t xs, int64_t rows,
+                     int I, hipStream_t s) {
+  if (dtype == DT_F32) silu_mul_rows<float>((float*)out, os, (const float*)x, xs, rows, I, s);
+  else if (dtype == DT_BF16) silu_mul_rows<bf16>((bf16*)out, os, (const bf16*)x, xs, rows, I, s);
+  else silu_mul_rows<f16>((f16*)out, os, (const f16*)x, xs, rows, I, s);
+}
+
+// ---- tanh cap on the logits -----------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void logit_softcap_kernel(float* __restrict__ out,
+                                                            const T* __restrict__ x, int64_t xs,
+                                                            int V, float cap, float inv) {
+  const int64_t r = blockIdx.y;
+  for (int c = blockIdx.x * 256 + threadIdx.x; c < V; c += gridDim.x * 256)
+    out[r * V + c] = cap * tanhf(to_f(x[r * xs + c]) * inv);
+}
+
+void launch_logit_softcap(int dtype, float* out, const void* x, int64_t xs, int64_t rows, int V,
+                          float cap, hipStream_t s) {
+  for (int64_t r0 = 0; r0 < rows; r0 += 65535) {
+    const dim3 grid(std::min((V + 255) / 256, 128), (unsigned)std::min<int64_t>(rows - r0, 65535));
+    float* o = out + r0 * V;
     if (dtype == DT_BF16)
-      silu_mul_kernel<bf16><<<grid, 256, 0, s>>>((bf16*)out + r0 * I, (const bf16*)x + r0 * 2 * I, I);
+      logit_softcap_kernel<bf16><<<grid, 256, 0, s>>>(o, (const bf16*)x + r0 * xs, xs, V, cap, 1.f / cap);
+    else if (dtype == DT_F16)
+      logit_softcap_kernel<f16><<<grid, 256, 0, s>>>(o, (const f16*)x + r0 * xs, xs, V, cap, 1.f / cap);
     else
-      silu_mul_kernel<f16><<<grid, 256, 0, s>>>((f16*)out + r0 * I, (const f16*)x + r0 * 2 * I, I);
+      logit_softcap_kernel<float><<<grid, 256, 0, s>>>(o, (const float*)x + r0 * xs, xs, V, cap, 1.f / cap);
   }
 }
 

@@ -2,7 +2,11 @@
 // (k [nb, G, bs, dk], v [nb, G, bs, dv]; dk != dv allowed, any sizes), for the hybrid
 // decoders.  Rows are addressed through their strides (krs, vrs elements per cache row), so
 // the values may be columns of the key rows (one latent cache row per token).  Query i sees key j when j <= i and (i - j < window or j < keep_first);
-// window <= 0 means plain causal attention.
+// window <= 0 means plain causal attention.  With pooled blocks (pool > 0) a page holds
+// ceil(bs / pool) further rows after its bs token rows: the mean key (value) row of every block
+// of pool tokens whose last token lies in the page; query i also sees the blocks that end
+// before its window.  Values may be cached turned by their positions (pairs over all dv
+// dimensions); a head's output is then turned back by the query's position.
 //
 //   rope_kv_store     rotates q and k on the first `rot` dims of a head (pair i, i + rot/2,
 //                     or 2i, 2i + 1; cos / sin from an fp32 table), writes q, and k / v
@@ -13,6 +17,9 @@
 //                     online softmax.  Prefill chunks and decode rows of a step take the
 //                     same path, so a position's result does not depend on how the prompt
 //                     was cut.  Scores, softmax weights and the weighted sum are fp32.
+//   qk_norm_store     RMS norm over the whole q row and the whole k row, rotation of q, k and
+//                     v, write of q and into the cache
+//   pool_kv           mean rows of the blocks that a step's tokens complete
 #include "common.h"
 #include "launch.h"
 
@@ -105,6 +112,63 @@ __global__ __launch_bounds__(256) void norm_kv_store_kernel(
   }
 }
 
+// whole blocks of `pool` tokens that end before the window of a query at `pos`
+__device__ __forceinline__ int pooled_count(int pos, int window, int pool) {
+  const int n = pos - window + 1;
+  return n > 0 ? n / pool : 0;
+}
+
+// pooled block b lives in the page of its last token, after the page's token rows
+__device__ __forceinline__ void pooled_place(int b, int pool, int bs, int& page, int& row) {
+  page = (b * pool + pool - 1) / bs;
+  row = bs + b - page * bs / pool;
+}
+
+// The mean row of the block that ends at token `pos`, for kv head g: threads tid, tid + nthr,
+// ... take one column each (keys, then values).
+template <typename T>
+__device__ __forceinline__ void pool_block(T* k_cache, T* v_cache, const int* bt, int pos,
+                                           int pool, int g, int G, int dk, int dv, int krs,
+                                           int vrs, int bs, int prow, int num_blocks, int tid,
+                                           int nthr) {
+  int pg, pr;
+  pooled_place(pos / pool, pool, bs, pg, pr);
+  int db = bt[pg];
+  if (db < 0 || db >= num_blocks) db = 0;
+  const int64_t dst = (int64_t)(db * G + g) * prow + pr;
+  const float inv = 1.f / (float)pool;
+  for (int c = tid; c < dk + dv; c += nthr) {
+    T* base = c < dk ? k_cache + c : v_cache + (c - dk);
+    const int rs = c < dk ? krs : vrs;
+    float a = 0.f;
+    for (int j = pos + 1 - pool; j <= pos; ++j) {
+      int b = bt[j / bs];
+      if (b < 0 || b >= num_blocks) b = 0;
+      a += to_f(base[((int64_t)(b * G + g) * prow + j % bs) * rs]);
+    }
+    base[dst * rs] = from_f<T>(a * inv);
+  }
+}
+
+// the table row of a position (never past the table)
+__device__ __forceinline__ const float* rot_row(const WindowExtra& ex, int pos, int dv) {
+  return ex.vtab + (int64_t)min(pos, ex.vrows - 1) * dv;
+}
+
+// column c of a head's output turned back by the row's position: `self` and `other` are the
+// pair's members, cs the table row (cos | sin)
+__device__ __forceinline__ float turn_back(float self, float other, const float* cs, int c,
+                                           int dv, bool inter) {
+  const int half = dv >> 1;
+  const int m = inter ? c >> 1 : (c < half ? c : c - half);
+  const bool first = inter ? !(c & 1) : c < half;
+  const float cn = cs[m], sn = cs[half + m];
+  return first ? self * cn + other * sn : self * cn - other * sn;
+}
+__device__ __forceinline__ int turn_partner(int c, int dv, bool inter) {
+  return inter ? c ^ 1 : (c < (dv >> 1) ? c + (dv >> 1) : c - (dv >> 1));
+}
+
 constexpr int MAX_DV_PER_LANE = 16;    // dv <= 1024
 
 // scaled score -> cap * tanh(score / cap) when a cap is set
@@ -120,7 +184,8 @@ __device__ __forceinline__ float elem_gate(const WindowExtra& ex, int64_t t, int
   return 1.f / (1.f + expf(-g));
 }
 
-// grid (T, H), one wave.  LDS: q row [dk] fp32, p [64], value-row offsets [64].
+// grid (T, H), one wave.  LDS: q row [dk] fp32, p [64], value-row offsets [64], and with
+// rotated values the output row [dv].
 template <typename T>
 __global__ __launch_bounds__(64) void window_attention_kernel(
     T* __restrict__ out, const T* __restrict__ q, const T* __restrict__ k_cache,
@@ -160,7 +225,8 @@ __global__ __launch_bounds__(64) void window_attention_kernel(
   for (int c = lane; c < dk; c += 64) qs[c] = to_f(qrow[c]);
   __syncthreads();
   const int lo_w = window > 0 ? max(0, pos - window + 1) : 0;
-  const int ns = min(keep_first, lo_w);           // kept first tokens outside the window
+  // kept first tokens outside the window, or the pooled blocks before it
+  const int ns = ex.pool > 0 ? pooled_count(pos, window, ex.pool) : min(keep_first, lo_w);
   const int total = ns + (pos - lo_w + 1);
   float m = -INFINITY, l = 0.f;
   float acc[MAX_DV_PER_LANE];
@@ -173,9 +239,11 @@ __global__ __launch_bounds__(64) void window_attention_kernel(
     int ro = 0;
     if (ok) {
       const int j = idx < ns ? idx : lo_w + (idx - ns);
-      int b = bt[j / bs];
+      int pg = j / bs, pr = j % bs;
+      if (ex.pool > 0 && idx < ns) pooled_place(idx, ex.pool, bs, pg, pr);
+      int b = bt[pg];
       if (b < 0 || b >= num_blocks) b = 0;       // never index outside the pool
-      ro = (b * G + g) * bs + (j % bs);
+      ro = (b * G + g) * ex.prow + pr;
       const T* kr = k_cache + (int64_t)ro * krs;
       float d = 0.f;
       for (int c = 0; c < dk; ++c) d += qs[c] * to_f(kr[c]);
@@ -203,6 +271,20 @@ __global__ __launch_bounds__(64) void window_attention_kernel(
   }
   const float gt = (gate != nullptr ? gate[(int64_t)t * H + h] : 1.f) * ex.out_scale;
   const float inv = gt / l;
+  if (ex.vtab != nullptr) {
+    float* os = (float*)(voff + 64);              // [dv]
+#pragma unroll
+    for (int u = 0; u < MAX_DV_PER_LANE; ++u)
+      if (lane + 64 * u < dv) os[lane + 64 * u] = acc[u];
+    __syncthreads();
+    const float* cs = rot_row(ex, pos, dv);
+#pragma unroll
+    for (int u = 0; u < MAX_DV_PER_LANE; ++u) {
+      const int c = lane + 64 * u;
+      if (c < dv)
+        acc[u] = turn_back(acc[u], os[turn_partner(c, dv, ex.vinter)], cs, c, dv, ex.vinter);
+    }
+  }
 #pragma unroll
   for (int u = 0; u < MAX_DV_PER_LANE; ++u) {
     const int c = lane + 64 * u;
@@ -279,10 +361,12 @@ __device__ __forceinline__ void load2(const T* p, float& a, float& b) {
 constexpr int DEC_WAVES = 8;          // waves per workgroup (4 when the grid is large)
 constexpr int DEC_UMAX = 4;          // value columns per lane: 2 * DEC_UMAX * 64 >= dv
 
-template <typename T, int QH, int NWV>
+// EXT: pooled blocks and rotated values (the caches are not __restrict__ there: the workgroup
+// of a kv head's first query heads also writes the mean row of a block its row completes,
+// which no row of the step sees yet).
+template <typename T, int QH, int NWV, bool EXT>
 __global__ __launch_bounds__(64 * NWV) void window_decode_kernel(
-    T* __restrict__ out, const T* __restrict__ q, const T* __restrict__ k_cache,
-    const T* __restrict__ v_cache, const int* __restrict__ ctx_lens, const int* __restrict__ dbt,
+    T* __restrict__ out, const T* __restrict__ q, const T* k_cache, const T* v_cache, const int* __restrict__ ctx_lens, const int* __restrict__ dbt,
     int bt_stride, int Tp, int H, int G, int dk, int dv, int krs, int vrs, int bs, int num_blocks,
     float scale, int window, int keep_first, const float* __restrict__ gate, WindowExtra ex) {
   extern __shared__ float lds[];
@@ -308,7 +392,15 @@ __global__ __launch_bounds__(64 * NWV) void window_decode_kernel(
   for (int e = threadIdx.x; e < QH * dv; e += 64 * NWV) accs[e] = 0.f;
   __syncthreads();
   const int lo_w = window > 0 ? max(0, pos - window + 1) : 0;
-  const int ns = min(keep_first, lo_w);
+  int ns = min(keep_first, lo_w);
+  if constexpr (EXT) {
+    if (ex.pool > 0) {
+      ns = pooled_count(pos, window, ex.pool);
+      if (blockIdx.z == 0 && (pos + 1) % ex.pool == 0)
+        pool_block<T>(const_cast<T*>(k_cache), const_cast<T*>(v_cache), bt, pos, ex.pool, g, G, dk,
+                      dv, krs, vrs, bs, ex.prow, num_blocks, threadIdx.x, 64 * NWV);
+    }
+  }
   const int total = ns + (pos - lo_w + 1);
   const int nchunks = (total + 63) >> 6;
   float m[QH], l[QH], acc[QH][DEC_UMAX][2];
@@ -334,9 +426,13 @@ __global__ __launch_bounds__(64 * NWV) void window_decode_kernel(
     int ro = 0;
     if (ok) {
       const int j = idx < ns ? idx : lo_w + (idx - ns);
-      int b = bt[j / bs];
+      int pg = j / bs, pr = j % bs;
+      if constexpr (EXT) {
+        if (ex.pool > 0 && idx < ns) pooled_place(idx, ex.pool, bs, pg, pr);
+      }
+      int b = bt[pg];
       if (b < 0 || b >= num_blocks) b = 0;
-      ro = (b * G + g) * bs + (j % bs);
+      ro = (b * G + g) * (EXT ? ex.prow : bs) + pr;
       const T* kr = k_cache + (int64_t)ro * krs;
       constexpr int KB = 8;                       // 16-byte pieces of the key row in flight
       for (int c0 = 0; c0 < dk; c0 += 8 * KB) {
@@ -507,8 +603,16 @@ __global__ __launch_bounds__(64 * NWV) void window_decode_kernel(
       if (mw != -INFINITY) L += ml[w * QH + h] * expf(mw - M);
     }
     const float gt = (gate != nullptr ? gate[(int64_t)t * H + h0 + h] : 1.f) * ex.out_scale;
+    float a = accs[e];
+    if constexpr (EXT) {
+      if (ex.vtab != nullptr) {
+        const int c = e - h * dv;
+        a = turn_back(a, accs[h * dv + turn_partner(c, dv, ex.vinter)], rot_row(ex, pos, dv), c,
+                      dv, ex.vinter);
+      }
+    }
     out[(int64_t)t * ex.ors + h0 * dv + e] =
-        from_f<T>(accs[e] * gt / L * elem_gate<T>(ex, t, h0 * dv + e));
+        from_f<T>(a * gt / L * elem_gate<T>(ex, t, h0 * dv + e));
   }
 }
 
@@ -524,9 +628,12 @@ __global__ __launch_bounds__(64 * NWV) void window_decode_kernel(
 //                    is 8 (m >> 2) + (m & 3), + 4 for the second tile of a 32-key pair).
 // The fp32 weights enter that product as a bf16/f16 pair (value + remainder), two MFMAs,
 // so they carry ~16 mantissa bits rather than 8.
+// EXT: tiles of pooled blocks take the place of the kept first tokens, and with values rotated
+// in halves the rows of V^T alternate 16 columns of the first half and 16 of the second, so
+// that both members of a pair sit in one lane's accumulators and are turned back in registers.
 constexpr int PFW_BM = 64, PFW_BN = 64, PFW_KPAD = 8, PFW_VPAD = 8;
 
-template <typename T, int KSM, int DTM>
+template <typename T, int KSM, int DTM, bool EXT>
 __global__ __launch_bounds__(256, KSM <= 4 ? 3 : 2) void window_prefill_mfma_kernel(
     T* __restrict__ out, const T* __restrict__ q, const T* __restrict__ k_cache,
     const T* __restrict__ v_cache, const int* __restrict__ qsl, const int* __restrict__ seq_lens,
@@ -569,7 +676,10 @@ __global__ __launch_bounds__(256, KSM <= 4 ? 3 : 2) void window_prefill_mfma_ker
   float m = -INFINITY, l = 0.f;
   const int p_min = ctx0 + r0, p_max = ctx0 + r0 + rows - 1;
   const int lo_min = window > 0 ? max(0, p_min - window + 1) : 0;
-  const int ns = window > 0 ? min(keep_first, lo_min) : 0;
+  int ns = window > 0 ? min(keep_first, lo_min) : 0;
+  const bool pooled = EXT && ex.pool > 0;
+  if (pooled) ns = pooled_count(p_max, window, ex.pool);     // what the last row sees
+  const bool halves = EXT && ex.vtab != nullptr && !ex.vinter;
   const int nsink = (ns + PFW_BN - 1) / PFW_BN;
   const int nmain = (p_max - lo_min + PFW_BN) / PFW_BN;
   // the wave's own span of visible keys (tiles outside it are staged but not computed)
@@ -583,18 +693,25 @@ __global__ __launch_bounds__(256, KSM <= 4 ? 3 : 2) void window_prefill_mfma_ker
     const int in = bs_shift >= 0 ? key & (bs - 1) : key - pg * bs;
     int bl = bt[pg];
     if (bl < 0 || bl >= num_blocks) bl = 0;
-    return (int64_t)(bl * G + g) * bs + in;
+    return (int64_t)(bl * G + g) * (EXT ? ex.prow : bs) + in;
+  };
+  auto block_row = [&](int b) -> int64_t {
+    int pg, pr;
+    pooled_place(b, ex.pool, bs, pg, pr);
+    int bl = bt[pg];
+    if (bl < 0 || bl >= num_blocks) bl = 0;
+    return (int64_t)(bl * G + g) * ex.prow + pr;
   };
   const int sr = threadIdx.x >> 4, sc = threadIdx.x & 15;     // K staging: 16 lanes per key row
   for (int tile = 0; tile < nsink + nmain; ++tile) {
-    const bool sink = tile < nsink;
+    const bool sink = tile < nsink, ptile = pooled && sink;
     const int kb = sink ? tile * PFW_BN : lo_min + (tile - nsink) * PFW_BN;
     const int hi = sink ? min(ns, kb + PFW_BN) : min(p_max + 1, kb + PFW_BN);
     __syncthreads();                         // the previous tile's fragments were read
 #pragma unroll
     for (int kq = 0; kq < 4; ++kq) {
       const int ks = sr + 16 * kq, key = kb + ks;
-      const T* src = key < hi ? k_cache + page_row(key) * krs : nullptr;
+      const T* src = key < hi ? k_cache + (ptile ? block_row(key) : page_row(key)) * krs : nullptr;
       for (int c = sc; c < kchunks; c += 16) {
         u32x4 val = u32x4{0u, 0u, 0u, 0u};
         if (src != nullptr) val = *reinterpret_cast<const u32x4*>(src + 8 * c);
@@ -603,20 +720,29 @@ __global__ __launch_bounds__(256, KSM <= 4 ? 3 : 2) void window_prefill_mfma_ker
     }
     {
       const int ks = threadIdx.x & (PFW_BN - 1), key = kb + ks;   // a wave's lanes: consecutive keys
-      const T* src = key < hi ? v_cache + page_row(key) * vrs : nullptr;
+      const T* src = key < hi ? v_cache + (ptile ? block_row(key) : page_row(key)) * vrs : nullptr;
       for (int c = threadIdx.x >> 6; c < vchunks; c += 4) {
         Pack8<T> val;
         val.u = u32x4{0u, 0u, 0u, 0u};
         if (src != nullptr) val.u = *reinterpret_cast<const u32x4*>(src + 8 * c);
+        int r = 8 * c;
+        if constexpr (EXT) {
+          if (halves) {
+            const int hf = r >= (dv >> 1), cc = hf ? r - (dv >> 1) : r;
+            r = (cc >> 4) * 32 + 16 * hf + (cc & 15);
+          }
+        }
 #pragma unroll
-        for (int e2 = 0; e2 < 8; ++e2) Vt[(8 * c + e2) * vst + ks] = val.h[e2];
+        for (int e2 = 0; e2 < 8; ++e2) Vt[(r + e2) * vst + ks] = val.h[e2];
       }
     }
     __syncthreads();
     if (16 * wave >= rows) continue;                       // no rows in this wave
     // nothing of this tile is visible to the wave's rows (kept first tokens can sit in a
     // main tile when the earliest window starts before them)
-    if (kb > wp_hi || (!sink && hi <= w_lo && kb >= keep_first)) continue;
+    if (ptile ? kb >= pooled_count(wp_hi, window, ex.pool)
+              : kb > wp_hi || (!sink && hi <= w_lo && kb >= keep_first))
+      continue;
     // ---- S^T tiles j = 0..3: keys 32 (j >> 1) + keyA + 4 (j & 1)
     f32x4 s[4];
 #pragma unroll
@@ -636,8 +762,10 @@ __global__ __launch_bounds__(256, KSM <= 4 ? 3 : 2) void window_prefill_mfma_ker
     // ---- visibility and online softmax (query = lane & 15).  A tile whose 64 keys are
     // all valid, not after the wave's first row and inside the window of its last row is
     // seen in full by every row of the wave: no per-element test.
-    const bool full = hi == kb + PFW_BN && kb + PFW_BN - 1 <= wp_lo &&
-                      (window <= 0 || wp_hi - kb < window) && wp_lo + 15 == wp_hi;
+    const int nblk = ptile ? pooled_count(qpos, window, ex.pool) : 0;
+    const bool full = ptile ? kb + PFW_BN <= pooled_count(wp_lo, window, ex.pool) && wp_lo + 15 == wp_hi
+                            : hi == kb + PFW_BN && kb + PFW_BN - 1 <= wp_lo &&
+                                  (window <= 0 || wp_hi - kb < window) && wp_lo + 15 == wp_hi;
     float tmax = -INFINITY;
     if (full) {
 #pragma unroll
@@ -653,8 +781,9 @@ __global__ __launch_bounds__(256, KSM <= 4 ? 3 : 2) void window_prefill_mfma_ker
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
           const int key = kb + (j >> 1) * 32 + 8 * qd + 4 * (j & 1) + i;
-          const bool vis = rowok && key < hi && key <= qpos &&
-                           (window <= 0 || qpos - key < window || key < keep_first);
+          const bool vis = ptile ? rowok && key < nblk
+                                 : rowok && key < hi && key <= qpos &&
+                                       (window <= 0 || qpos - key < window || key < keep_first);
           s[j][i] = vis ? cap_score(s[j][i] * scale, ex.softcap) : -INFINITY;
           tmax = fmaxf(tmax, s[j][i]);
         }
@@ -705,18 +834,175 @@ __global__ __launch_bounds__(256, KSM <= 4 ? 3 : 2) void window_prefill_mfma_ker
     const float gt = (gate != nullptr ? gate[(int64_t)(q0 + myrow) * H + h] : 1.f) * ex.out_scale;
     const float inv = l > 0.f ? gt / l : 0.f;
     T* orow = out + (int64_t)(q0 + myrow) * ex.ors + h * dv;
+    if constexpr (EXT) {
+      if (ex.vtab != nullptr) {
+        const float* cs = rot_row(ex, qpos, dv);
+        const int half = dv >> 1;
+        if (halves) {
+#pragma unroll
+          for (int t2 = 0; t2 < DTM; t2 += 2) {
+            if (t2 < ndt) {
+              const int m0 = 8 * t2 + 4 * qd;              // 16 (t2 / 2) + 4 qd
+#pragma unroll
+              for (int i = 0; i < 4; ++i) {
+                const float a = o[t2][i], b = o[t2 + 1][i], c = cs[m0 + i], sn = cs[half + m0 + i];
+                o[t2][i] = a * c + b * sn;
+                o[t2 + 1][i] = b * c - a * sn;
+              }
+            }
+          }
+        } else {
+#pragma unroll
+          for (int t2 = 0; t2 < DTM; ++t2) {
+            if (t2 < ndt) {
+              const int m0 = 8 * t2 + 2 * qd;
+#pragma unroll
+              for (int i = 0; i < 4; i += 2) {
+                const float a = o[t2][i], b = o[t2][i + 1];
+                const float c = cs[m0 + (i >> 1)], sn = cs[half + m0 + (i >> 1)];
+                o[t2][i] = a * c + b * sn;
+                o[t2][i + 1] = b * c - a * sn;
+              }
+            }
+          }
+        }
+      }
+    }
 #pragma unroll
     for (int t2 = 0; t2 < DTM; ++t2) {
       if (t2 < ndt) {
+        const int c0 = halves ? (t2 & 1) * (dv >> 1) + 16 * (t2 >> 1) + 4 * qd : 16 * t2 + 4 * qd;
         Pack4<T> w4;
 #pragma unroll
         for (int i = 0; i < 4; ++i)
-          w4.h[i] = from_f<T>(o[t2][i] * inv *
-                              elem_gate<T>(ex, q0 + myrow, h * dv + 16 * t2 + 4 * qd + i));
-        *reinterpret_cast<u32x2*>(orow + 16 * t2 + 4 * qd) = w4.u;
+          w4.h[i] = from_f<T>(o[t2][i] * inv * elem_gate<T>(ex, q0 + myrow, h * dv + c0 + i));
+        *reinterpret_cast<u32x2*>(orow + c0) = w4.u;
       }
     }
   }
+}
+
+// VEC consecutive elements as fp32 / from fp32 (VEC 8: 16-byte accesses of 16-bit types)
+template <typename T, int VEC>
+__device__ __forceinline__ void load_vec(const T* p, float (&v)[VEC]) {
+  if constexpr (VEC == 8) load8(p, v);
+  else v[0] = to_f(p[0]);
+}
+template <typename T, int VEC>
+__device__ __forceinline__ void store_vec(T* p, const float (&v)[VEC]) {
+  if constexpr (VEC == 1) {
+    p[0] = from_f<T>(v[0]);
+  } else if constexpr (std::is_same_v<T, float>) {
+    *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+    *reinterpret_cast<float4*>(p + 4) = make_float4(v[4], v[5], v[6], v[7]);
+  } else {
+    Pack8<T> t;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) t.h[e] = from_f<T>(v[e]);
+    *reinterpret_cast<u32x4*>(p) = t.u;
+  }
+}
+
+// One workgroup per token.  qkv row = q [H dk] (| k [G dk] | v [G dv] when a cache is given):
+// the whole q row and the whole k row over their root mean squares times a weight per column,
+// rotation of q and k on the first `rot` dims (table: cos | sin) and of v on all dv (vtab);
+// q -> q_out [T, H, dk], k and v -> the cache row of the token's slot.  The row sits in LDS as
+// fp32 between the sums and the outputs.  VEC 8: a thread makes 8 adjacent outputs (head sizes,
+// rotated parts and strides are multiples that keep them in one head and one half).
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void qk_norm_store_kernel(
+    T* __restrict__ q_out, const T* __restrict__ qkv, int64_t qs, const int64_t* __restrict__ positions,
+    const float* __restrict__ qw, const float* __restrict__ kw, const float* __restrict__ table,
+    int rot, int trows, const float* __restrict__ vtab, int vrows, T* __restrict__ k_cache,
+    T* __restrict__ v_cache, const int64_t* __restrict__ slots, int H, int G, int dk, int dv,
+    int bs, int prow, int num_blocks, float eps, bool inter) {
+  extern __shared__ float lds[];
+  __shared__ float scratch[4];
+  const int64_t t = blockIdx.x;
+  const T* row = qkv + t * qs;
+  const int nq = H * dk, nk = k_cache != nullptr ? G * dk : 0, nv = k_cache != nullptr ? G * dv : 0;
+  const int64_t slot = slots[t];
+  const bool store = nk > 0 && slot >= 0 && slot < (int64_t)num_blocks * bs;
+  const int n = nq + (store ? nk + nv : 0);
+  float sq = 0.f, sk = 0.f;
+  for (int e = threadIdx.x * VEC; e < n; e += 256 * VEC) {
+    float v[VEC];
+    load_vec<T, VEC>(row + e, v);
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) {
+      lds[e + i] = v[i];
+      ss += v[i] * v[i];
+    }
+    if (e < nq) sq += ss;
+    else if (e < nq + nk) sk += ss;
+  }
+  sq = block_sum<256>(sq, scratch);
+  if (store) sk = block_sum<256>(sk, scratch);
+  const float rq = 1.f / sqrtf(sq / (float)nq + eps);
+  const float rk = store ? 1.f / sqrtf(sk / (float)nk + eps) : 0.f;
+  int64_t pos = positions[t];
+  if (pos < 0) pos = 0;
+  const float* cs = table != nullptr ? table + (pos < trows ? pos : trows - 1) * rot : nullptr;
+  const float* vcs = vtab != nullptr ? vtab + (pos < vrows ? pos : vrows - 1) * dv : nullptr;
+  const int64_t blk = store ? slot / bs : 0, off = store ? slot % bs : 0;
+  for (int e = threadIdx.x * VEC; e < n; e += 256 * VEC) {
+    const bool isv = e >= nq + nk, isq = e < nq;
+    const int e0 = isq ? e : isv ? e - nq - nk : e - nq, hs = isv ? dv : dk;
+    const int head = e0 / hs, i0 = e0 - head * hs;
+    const float f = isq ? rq : isv ? 1.f : rk;
+    const float* w = isq ? qw : kw;
+    const float* rc = isv ? vcs : cs;
+    const int rd = rc == nullptr ? 0 : isv ? dv : rot, half = rd >> 1;
+    const int b0 = e - i0;                             // the head's first element
+    auto val = [&](int i) { return lds[b0 + i] * (isv ? 1.f : f * w[e0 - i0 + i]); };
+    float v[VEC];
+#pragma unroll
+    for (int k = 0; k < VEC; ++k) {
+      const int i = i0 + k;
+      v[k] = val(i);
+      if (i < rd) {
+        const int p = inter ? i >> 1 : (i < half ? i : i - half);
+        const bool first = inter ? !(i & 1) : i < half;
+        const float o = val(inter ? i ^ 1 : (first ? i + half : i - half));
+        const float c = rc[p], sn = rc[half + p];
+        v[k] = first ? v[k] * c - o * sn : v[k] * c + o * sn;
+      }
+    }
+    T* dst = isq ? q_out + t * nq + e
+                 : isv ? v_cache + ((blk * G + head) * prow + off) * dv + i0
+                       : k_cache + ((blk * G + head) * prow + off) * dk + i0;
+    store_vec<T, VEC>(dst, v);
+  }
+}
+
+// Rows t0 .. of a step that complete a block of `pool` tokens (and are stored) write the
+// block's mean rows; grid (rows, G).
+template <typename T>
+__global__ __launch_bounds__(256) void pool_kv_kernel(
+    T* k_cache, T* v_cache, const int64_t* __restrict__ slots, const int* __restrict__ qsl,
+    const int* __restrict__ seq_lens, const int* __restrict__ pbt, const int* __restrict__ ctx_lens,
+    const int* __restrict__ dbt, int bt_stride, int P, int Tp, int t0, int G, int dk, int dv,
+    int krs, int vrs, int bs, int prow, int num_blocks, int pool) {
+  const int t = t0 + blockIdx.x;
+  if (slots[t] < 0) return;
+  int pos;
+  const int* bt;
+  if (t < Tp) {
+    int lo = 0, hi = P - 1;
+    while (lo < hi) {
+      const int mid = (lo + hi + 1) >> 1;
+      if (qsl[mid] <= t) lo = mid; else hi = mid - 1;
+    }
+    pos = seq_lens[lo] - (qsl[lo + 1] - qsl[lo]) + (t - qsl[lo]);
+    bt = pbt + (int64_t)lo * bt_stride;
+  } else {
+    pos = ctx_lens[t - Tp] - 1;
+    bt = dbt + (int64_t)(t - Tp) * bt_stride;
+  }
+  if (pos < 0 || pos >= bt_stride * bs || (pos + 1) % pool != 0) return;
+  pool_block<T>(k_cache, v_cache, bt, pos, pool, blockIdx.y, G, dk, dv, krs, vrs, bs, prow,
+                num_blocks, threadIdx.x, 256);
 }
 
 }  // namespace
@@ -749,6 +1035,40 @@ void launch_norm_kv_store(int out_dtype, const float* qkv, int64_t qs, const int
       num_blocks, eps, qk_unit, v_unit, coef, every));
 }
 
+bool qk_norm_store_ok(int H, int G, int dk, int dv) {
+  return ((int64_t)(H + G) * dk + (int64_t)G * dv) * 4 <= 64 * 1024;
+}
+
+void launch_qk_norm_store(int dtype, void* q_out, const void* qkv, int64_t qs,
+                          const int64_t* positions, const float* qw, const float* kw,
+                          const float* table, int rot, int trows, const float* vtab, int vrows,
+                          void* k_cache, void* v_cache, const int64_t* slots, int T_, int H, int G,
+                          int dk, int dv, int bs, int prow, int num_blocks, float eps, bool inter,
+                          hipStream_t s) {
+  if (T_ <= 0) return;
+  const bool kv = k_cache != nullptr;
+  const size_t lds = sizeof(float) * (size_t)(H * dk + (kv ? G * (dk + dv) : 0));
+  // eight adjacent elements of one head and one half of the rotated part, 16-byte aligned
+  const bool vec = dk % 8 == 0 && (!kv || dv % 8 == 0) && qs % 8 == 0 &&
+                   reinterpret_cast<uintptr_t>(qkv) % 16 == 0;
+#define KGC_QKN(V)                                                                           \
+  KGC_DISPATCH_T(dtype, qk_norm_store_kernel<T, V><<<T_, 256, lds, s>>>(                     \
+      (T*)q_out, (const T*)qkv, qs, positions, qw, kw, table, rot, trows, vtab, vrows,       \
+      (T*)k_cache, (T*)v_cache, slots, H, G, dk, dv, bs, prow, num_blocks, eps, inter))
+  if (vec) KGC_QKN(8); else KGC_QKN(1);
+#undef KGC_QKN
+}
+
+void launch_pool_kv(int dtype, void* k_cache, void* v_cache, const int64_t* slots, const int* qsl,
+                    const int* seq_lens, const int* pbt, const int* ctx_lens, const int* dbt,
+                    int bt_stride, int P, int Tp, int t0, int rows, int G, int dk, int dv, int krs,
+                    int vrs, int bs, int prow, int num_blocks, int pool, hipStream_t s) {
+  if (rows <= 0) return;
+  KGC_DISPATCH_T(dtype, pool_kv_kernel<T><<<dim3(rows, G), 256, 0, s>>>(
+      (T*)k_cache, (T*)v_cache, slots, qsl, seq_lens, pbt, ctx_lens, dbt, bt_stride, P, Tp, t0, G,
+      dk, dv, krs, vrs, bs, prow, num_blocks, pool));
+}
+
 int window_attention_max_dv() { return 64 * MAX_DV_PER_LANE; }
 
 void launch_window_attention(int dtype, void* out, const void* q, const void* k_cache,
@@ -758,7 +1078,7 @@ void launch_window_attention(int dtype, void* out, const void* q, const void* k_
                              int bs, int num_blocks, float scale, int window, int keep_first,
                              const float* gate, int kinds, WindowExtra ex, hipStream_t s) {
   if (T_ <= 0 || !kinds) return;
-  const size_t lds = (size_t)(dk + 128) * sizeof(float);
+  const size_t lds = (size_t)(dk + 128 + (ex.vtab != nullptr ? dv : 0)) * sizeof(float);
   KGC_DISPATCH_T(dtype, window_attention_kernel<T><<<dim3(T_, H), 64, lds, s>>>(
       (T*)out, (const T*)q, (const T*)k_cache, (const T*)v_cache, qsl, seq_lens, pbt, ctx_lens,
       dbt, bt_stride, P, Tp, H, G, dk, dv, krs, vrs, bs, num_blocks, scale, window, keep_first,
@@ -790,10 +1110,15 @@ static void decode_dispatch(T* out, const T* q, const T* kc, const T* vc, const 
   // 8 waves split a row's keys finest (shortest chain per workgroup); once the grid holds
   // two workgroups per CU, 4-wave workgroups let two of them overlap on a CU instead
   const bool small = (int64_t)grid.x * grid.y * grid.z >= 512;
-#define KGC_DEC(N, W)                                                                        \
-  window_decode_kernel<T, N, W><<<grid, 64 * W, decode_lds(N, W, dk, dv), s>>>(              \
+  const bool ext = ex.pool > 0 || ex.vtab != nullptr;
+#define KGC_DEC_E(N, W, E)                                                                   \
+  window_decode_kernel<T, N, W, E><<<grid, 64 * W, decode_lds(N, W, dk, dv), s>>>(           \
       out, q, kc, vc, ctx_lens, dbt, bt_stride, Tp, H, G, dk, dv, krs, vrs, bs, num_blocks,     \
       scale, window, keep_first, gate, ex)
+#define KGC_DEC(N, W)                                         \
+  do {                                                        \
+    if (ext) KGC_DEC_E(N, W, true); else KGC_DEC_E(N, W, false); \
+  } while (0)
 #define KGC_DEC2(N) \
   do {              \
     if (small) KGC_DEC(N, 4); else KGC_DEC(N, 8); \
@@ -804,6 +1129,7 @@ static void decode_dispatch(T* out, const T* q, const T* kc, const T* vc, const 
   else KGC_DEC2(1);
 #undef KGC_DEC2
 #undef KGC_DEC
+#undef KGC_DEC_E
 }
 
 size_t window_decode_lds(int dk, int dv, int qpg) {
@@ -843,13 +1169,19 @@ static void prefill_dispatch(T* out, const T* q, const T* kc, const T* vc, const
                              WindowExtra ex, hipStream_t s) {
   const dim3 grid(n_work * (blk_rows / PFW_BM), H);
   const size_t lds = window_prefill_mfma_lds(dk, dv);
-#define KGC_PF(K, D)                                                                          \
-  window_prefill_mfma_kernel<T, K, D><<<grid, 256, lds, s>>>(                                 \
+  const bool ext = ex.pool > 0 || ex.vtab != nullptr;
+#define KGC_PF_E(K, D, E)                                                                     \
+  window_prefill_mfma_kernel<T, K, D, E><<<grid, 256, lds, s>>>(                              \
       out, q, kc, vc, qsl, seq_lens, pbt, bt_stride, work_seq, work_blk, blk_rows, H, G, dk,  \
       dv, krs, vrs, bs, num_blocks, scale, window, keep_first, gate, ex)
+#define KGC_PF(K, D)                                       \
+  do {                                                     \
+    if (ext) KGC_PF_E(K, D, true); else KGC_PF_E(K, D, false); \
+  } while (0)
   if (dk <= 128 && dv <= 128) KGC_PF(4, 8);
   else KGC_PF(8, 16);
 #undef KGC_PF
+#undef KGC_PF_E
 }
 
 void launch_window_prefill_mfma(int dtype, void* out, const void* q, const void* k_cache,

@@ -7,6 +7,7 @@
 //   xielu                the xIELU activation
 //   gate_proj            a few fp32 gate outputs per row: act(h . w^T + b)
 //   residual_norm        x += mult * (add, or RMS-normed add * weight); h = RMSNorm(x) * w
+//   residual_sum_norm    x += up to three results, each plain or RMS-normed; h = RMSNorm(x) * w
 //   gate_mul, relu_sq, side_gate   element-wise epilogues between GEMMs
 // All arithmetic is fp32; T is the activation dtype of h / y (bf16, f16 or fp32).
 // One workgroup per row; a row is walked twice (sum of squares, then scale), the second
@@ -362,6 +363,157 @@ __global__ __launch_bounds__(NT) void residual_norm_kernel(
   for (int c = threadIdx.x; c < W; c += NT) o[c] = from_f<O>(xr[c] * r * w[c]);
 }
 
+// x += sum_j a_j, or a_j / rms(a_j) * aw_j where aw_j is given; then out = x / rms(x) * w (out
+// null: none).  A thread keeps EPT columns in registers, VEC adjacent ones at a time, so every
+// addend and x are read once and x written once; EPT = 0 walks the row in passes.
+template <typename T, int VEC>
+__device__ __forceinline__ void ld_cols(const T* p, float (&v)[VEC]) {
+  if constexpr (VEC == 1) {
+    v[0] = to_f(p[0]);
+  } else if constexpr (std::is_same_v<T, float>) {
+    const float4 t = *reinterpret_cast<const float4*>(p);
+    v[0] = t.x; v[1] = t.y; v[2] = t.z; v[3] = t.w;
+  } else {
+    Pack4<T> t;
+    t.u = *reinterpret_cast<const u32x2*>(p);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = to_f(t.h[e]);
+  }
+}
+template <typename T, int VEC>
+__device__ __forceinline__ void st_cols(T* p, const float (&v)[VEC]) {
+  if constexpr (VEC == 1) {
+    p[0] = from_f<T>(v[0]);
+  } else if constexpr (std::is_same_v<T, float>) {
+    *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+  } else {
+    Pack4<T> t;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) t.h[e] = from_f<T>(v[e]);
+    *reinterpret_cast<u32x2*>(p) = t.u;
+  }
+}
+
+template <typename T, typename O, int EPT, int VEC>
+__global__ __launch_bounds__(NT) void residual_sum_norm_kernel(O* __restrict__ out,
+                                                               float* __restrict__ x,
+                                                               ResidualAdds adds,
+                                                               const float* __restrict__ w, int W,
+                                                               float eps) {
+  __shared__ float scratch[3][NT / 64];
+  const int64_t row = blockIdx.x;
+  float* xr = x + row * W;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  // three sums over the workgroup with one barrier
+  auto sums3 = [&](float (&ss)[3]) {
+#pragma unroll
+    for (int j = 0; j < 3; ++j) {
+      ss[j] = wave_sum(ss[j]);
+      if (lane == 0) scratch[j][wave] = ss[j];
+    }
+    __syncthreads();
+#pragma unroll
+    for (int j = 0; j < 3; ++j) {
+      ss[j] = 0.f;
+#pragma unroll
+      for (int v = 0; v < NT / 64; ++v) ss[j] += scratch[j][v];
+    }
+    __syncthreads();
+  };
+  const bool normed = adds.w[0] != nullptr || adds.w[1] != nullptr || adds.w[2] != nullptr;
+  if constexpr (EPT > 0) {
+    constexpr int NC = EPT / VEC;
+    float xv[NC][VEC], av[3][NC][VEC], ss[3] = {0.f, 0.f, 0.f};
+#pragma unroll
+    for (int k = 0; k < NC; ++k) {
+      const int c = (threadIdx.x + k * NT) * VEC;
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) xv[k][e] = 0.f;
+      if (c < W) ld_cols<float, VEC>(xr + c, xv[k]);
+    }
+#pragma unroll
+    for (int j = 0; j < 3; ++j) {
+      const T* ar = static_cast<const T*>(adds.a[j]);
+#pragma unroll
+      for (int k = 0; k < NC; ++k) {
+        const int c = (threadIdx.x + k * NT) * VEC;
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) av[j][k][e] = 0.f;
+        if (ar != nullptr && c < W) ld_cols<T, VEC>(ar + row * W + c, av[j][k]);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) ss[j] += av[j][k][e] * av[j][k][e];
+      }
+    }
+    if (normed) sums3(ss);
+    float sx = 0.f;
+#pragma unroll
+    for (int k = 0; k < NC; ++k) {
+      const int c = (threadIdx.x + k * NT) * VEC;
+      if (c < W) {
+#pragma unroll
+        for (int j = 0; j < 3; ++j) {
+          if (adds.w[j] != nullptr) {
+            const float ra = 1.f / sqrtf(ss[j] / (float)W + eps);
+            float wv[VEC];
+            ld_cols<float, VEC>(adds.w[j] + c, wv);
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) xv[k][e] += av[j][k][e] * ra * wv[e];
+          } else {
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) xv[k][e] += av[j][k][e];
+          }
+        }
+        if (adds.a[0] != nullptr) st_cols<float, VEC>(xr + c, xv[k]);
+      }
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) sx += xv[k][e] * xv[k][e];
+    }
+    if (out == nullptr) return;
+    sx = block_sum<NT>(sx, scratch[0]);
+    const float r = 1.f / sqrtf(sx / (float)W + eps);
+#pragma unroll
+    for (int k = 0; k < NC; ++k) {
+      const int c = (threadIdx.x + k * NT) * VEC;
+      if (c < W) {
+        float wv[VEC], o[VEC];
+        ld_cols<float, VEC>(w + c, wv);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) o[e] = xv[k][e] * r * wv[e];
+        st_cols<O, VEC>(out + row * W + c, o);
+      }
+    }
+    return;
+  }
+  float ss[3] = {0.f, 0.f, 0.f};
+  if (normed) {
+    for (int c = threadIdx.x; c < W; c += NT)
+#pragma unroll
+      for (int j = 0; j < 3; ++j)
+        if (adds.w[j] != nullptr) {
+          const float v = to_f(static_cast<const T*>(adds.a[j])[row * W + c]);
+          ss[j] += v * v;
+        }
+    sums3(ss);
+  }
+  float sx = 0.f;
+  for (int c = threadIdx.x; c < W; c += NT) {
+    float v = xr[c];
+#pragma unroll
+    for (int j = 0; j < 3; ++j)
+      if (adds.a[j] != nullptr) {
+        float a = to_f(static_cast<const T*>(adds.a[j])[row * W + c]);
+        if (adds.w[j] != nullptr) a = a * (1.f / sqrtf(ss[j] / (float)W + eps)) * adds.w[j][c];
+        v += a;
+      }
+    xr[c] = v;
+    sx += v * v;
+  }
+  if (out == nullptr) return;
+  sx = block_sum<NT>(sx, scratch[0]);
+  const float r = 1.f / sqrtf(sx / (float)W + eps);
+  for (int c = threadIdx.x; c < W; c += NT) out[row * W + c] = from_f<O>(xr[c] * r * w[c]);
+}
+
 // out [T, H * dv] (row stride so) = o[t, h, :] (strides st, sh) * sigmoid(g[t, h * dv + :])
 // (row stride sg) * scale
 template <typename T>
@@ -565,6 +717,33 @@ void launch_residual_norm(int dtype, int out_dtype, void* out, float* x, const v
   }
 #undef KGC_RN_W
 #undef KGC_RN
+}
+
+void launch_residual_sum_norm(int dtype, int out_dtype, void* out, float* x, ResidualAdds adds,
+                              const float* w, int rows, int W, float eps, hipStream_t s) {
+  if (rows <= 0) return;
+  bool vec = W % 4 == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0 &&
+             reinterpret_cast<uintptr_t>(out) % 16 == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0;
+  for (int j = 0; j < 3; ++j)
+    vec = vec && reinterpret_cast<uintptr_t>(adds.a[j]) % 16 == 0 &&
+          reinterpret_cast<uintptr_t>(adds.w[j]) % 16 == 0;
+#define KGC_RSN(O, EPT, V) \
+  residual_sum_norm_kernel<T, O, EPT, V><<<rows, NT, 0, s>>>((O*)out, x, adds, w, W, eps)
+#define KGC_RSN_W(O)                                 \
+  do {                                               \
+    if (vec && W <= 4 * NT) KGC_RSN(O, 4, 4);        \
+    else if (vec && W <= 8 * NT) KGC_RSN(O, 8, 4);   \
+    else if (vec && W <= 16 * NT) KGC_RSN(O, 16, 4); \
+    else if (W <= 4 * NT) KGC_RSN(O, 4, 1);          \
+    else KGC_RSN(O, 0, 1);                           \
+  } while (0)
+  if (out == nullptr || out_dtype == DT_F32) {
+    KGC_DISPATCH_T(dtype, KGC_RSN_W(float));
+  } else {
+    KGC_DISPATCH_T(dtype, KGC_RSN_W(T));
+  }
+#undef KGC_RSN_W
+#undef KGC_RSN
 }
 
 void launch_gate_mul(int dtype, void* out, int64_t so, const void* o, int64_t st, int64_t sh,

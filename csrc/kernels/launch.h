@@ -12,7 +12,8 @@ void launch_rms_norm(int dtype, void* out, const void* x, void* residual, const 
                      int rows, int H, int64_t x_stride, float eps, hipStream_t s);
 void launch_layer_norm(int dtype, void* out, const void* x, const void* w, const void* b,
                        int rows, int H, float eps, hipStream_t s);
-void launch_silu_mul(int dtype, void* out, const void* x, int64_t rows, int I, hipStream_t s);
+void launch_silu_mul(int dtype, void* out, int64_t os, const void* x, int64_t xs, int64_t rows,
+                     int I, hipStream_t s);
 // S > 0: qkv is S fp32 split-K slices [S, T, qkv_stride] (slice_stride apart), summed here
 void launch_rope_kv_write(int dtype, const void* qkv, int64_t qkv_stride, int S,
                           int64_t slice_stride, const int64_t* positions, const float* cos_sin, void* q_out,
@@ -272,14 +273,34 @@ int window_attention_max_dv();
 // what an attention inside a wider mixer adds: the row stride of `out` in elements (its
 // rows may be column slices of a wider buffer), a tanh cap on the scaled scores (<= 0:
 // none), a factor on the result, and an element-wise gate: the result is multiplied by
-// sigmoid(egate[t, head * dv + c]) (activation dtype, row stride egs; null: none)
+// sigmoid(egate[t, head * dv + c]) (activation dtype, row stride egs; null: none).  pool > 0:
+// mean rows of blocks of `pool` tokens follow the token rows of a page (prow rows in all; prow =
+// bs without pooled blocks).  vtab (fp32 [vrows, dv], cos | sin; null: none): the output is
+// turned back by the row's position, pairs (m, m + dv/2) or (2m, 2m + 1) when vinter
 struct WindowExtra {
   int64_t ors;
   float softcap;
   float out_scale;
   const void* egate;
   int64_t egs;
+  int pool;
+  int prow;
+  const float* vtab;
+  int vrows;
+  bool vinter;
 };
+// whether a row of (H + G) dk + G dv fp32 values fits the store kernel's LDS
+bool qk_norm_store_ok(int H, int G, int dk, int dv);
+void launch_qk_norm_store(int dtype, void* q_out, const void* qkv, int64_t qs,
+                          const int64_t* positions, const float* qw, const float* kw,
+                          const float* table, int rot, int trows, const float* vtab, int vrows,
+                          void* k_cache, void* v_cache, const int64_t* slots, int T, int H, int G,
+                          int dk, int dv, int bs, int prow, int num_blocks, float eps, bool inter,
+                          hipStream_t s);
+void launch_pool_kv(int dtype, void* k_cache, void* v_cache, const int64_t* slots, const int* qsl,
+                    const int* seq_lens, const int* pbt, const int* ctx_lens, const int* dbt,
+                    int bt_stride, int P, int Tp, int t0, int rows, int G, int dk, int dv, int krs,
+                    int vrs, int bs, int prow, int num_blocks, int pool, hipStream_t s);
 void launch_window_attention(int dtype, void* out, const void* q, const void* k_cache,
                              const void* v_cache, const int* qsl, const int* seq_lens,
                              const int* pbt, const int* ctx_lens, const int* dbt, int bt_stride,
@@ -402,5 +423,25 @@ void launch_embed_pos(int dtype, float* out, const int64_t* ids, const int64_t* 
 void launch_moe_route_softmax_all(float* w, int* ids, float* idw, const float* logits,
                                   int64_t stride, const float* corr, int ntok, int E, int k,
                                   int n_real, hipStream_t s);
+
+// ---- channel_delta.hip / Generax-style decoders --------------------------------------------
+void launch_delta_gates(int dtype, float* decay, void* gate, const void* low, int64_t ls,
+                        const void* a2, const void* g2, const float* neg_a, const float* dt_bias,
+                        int T, int Nd, int Ng, int ra, int rg, hipStream_t s);
+int channel_delta_max_rows();
+void launch_channel_delta_scan(int dtype, float* out, const float* qkv, const void* b,
+                               int64_t bstr, const float* decay, float* S, const int* qsl,
+                               const int* seq_lens, const int* ctx_lens, const int* slots, int P,
+                               int D, int Tp, int H, int G, int d, int V, int num_slots,
+                               hipStream_t s);
+// x += sum of up to three results, each plain or RMS-normed with a weight; out = norm of x
+struct ResidualAdds {
+  const void* a[3];
+  const float* w[3];
+};
+void launch_residual_sum_norm(int dtype, int out_dtype, void* out, float* x, ResidualAdds adds,
+                              const float* w, int rows, int W, float eps, hipStream_t s);
+void launch_logit_softcap(int dtype, float* out, const void* x, int64_t xs, int64_t rows, int V,
+                          float cap, hipStream_t s);
 
 }  // namespace kgc
