@@ -1489,19 +1489,28 @@ void window_attention(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
   const bool decode_fast = fast && aligned && D > 0 &&
                            kgc::window_decode_ok((int)dk, (int)dv, (int)(H / G)) &&
                            kgc::window_decode_lds((int)dk, (int)dv, (int)(H / G)) <= 64 * 1024;
+  if (work_seq.has_value())
+    TORCH_CHECK(work_blk.has_value() && work_blk->numel() == work_seq->numel() &&
+                work_seq->scalar_type() == at::kInt && work_blk->scalar_type() == at::kInt &&
+                work_seq->is_cuda() && work_blk->is_cuda(),
+                "kgc.window_attention: work list int32 [n] on the GPU");
   if (pool > 0) {                 // (the decode kernel pools its own rows)
-    const int rows = (int)(Tp + (decode_fast ? 0 : D));
-    kgc::launch_pool_kv(dt, k_cache.data_ptr(), v_cache.data_ptr(), slots->data_ptr<int64_t>(), qp,
-                        sp, pp, cp, dp, (int)bts, (int)P, (int)Tp, 0, rows, (int)G, (int)dk,
-                        (int)dv, (int)krs, (int)vrs, bs, prow, nb, (int)pool, stream());
+    const int64_t* slp = slots->data_ptr<int64_t>();
+    const bool chunks = P > 0 && work_seq.has_value();
+    if (chunks)
+      kgc::launch_pool_chunks(dt, k_cache.data_ptr(), v_cache.data_ptr(), slp, qp, sp, pp, (int)bts,
+                              work_seq->data_ptr<int>(), work_blk->data_ptr<int>(),
+                              (int)work_seq->numel(), kgc::prefill_block_m(), (int)G, (int)dk,
+                              (int)dv, (int)krs, (int)vrs, bs, prow, nb, (int)pool, stream());
+    const int t0 = chunks ? (int)Tp : 0, t1 = (int)(decode_fast ? Tp : T);
+    kgc::launch_pool_kv(dt, k_cache.data_ptr(), v_cache.data_ptr(), slp, qp, sp, pp, cp, dp,
+                        (int)bts, (int)P, (int)Tp, t0, t1 - t0, (int)G, (int)dk, (int)dv, (int)krs,
+                        (int)vrs, bs, prow, nb, (int)pool, stream());
   }
   if (fast && aligned && out_vec && P > 0 && work_seq.has_value() && work_blk.has_value() &&
       kgc::window_prefill_mfma_ok(dt, (int)dk, (int)dv) &&
       (vtp == nullptr || interleaved || dv % 32 == 0)) {   // a pair within one lane
     const int64_t nw = work_seq->numel();
-    TORCH_CHECK(work_blk->numel() == nw && work_seq->scalar_type() == at::kInt &&
-                work_blk->scalar_type() == at::kInt && work_seq->is_cuda() && work_blk->is_cuda(),
-                "kgc.window_attention: work list int32 [n] on the GPU");
     kgc::launch_window_prefill_mfma(dt, out.data_ptr(), q.data_ptr(), k_cache.data_ptr(),
                                     v_cache.data_ptr(), qp, sp, pp, (int)bts,
                                     work_seq->data_ptr<int>(), work_blk->data_ptr<int>(), (int)nw,

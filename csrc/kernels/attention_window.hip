@@ -141,6 +141,7 @@ __device__ __forceinline__ void pool_block(T* k_cache, T* v_cache, const int* bt
     T* base = c < dk ? k_cache + c : v_cache + (c - dk);
     const int rs = c < dk ? krs : vrs;
     float a = 0.f;
+#pragma unroll 8
     for (int j = pos + 1 - pool; j <= pos; ++j) {
       int b = bt[j / bs];
       if (b < 0 || b >= num_blocks) b = 0;
@@ -976,6 +977,151 @@ __global__ __launch_bounds__(256) void qk_norm_store_kernel(
   }
 }
 
+// The same for head sizes, rotated parts and alignments that are multiples of 16 elements and
+// pairs in halves: a thread owns NU units of two 8-element pieces that rotate into each other
+// (or two adjacent pieces past the rotated part) and keeps them in registers between the sums
+// and the outputs.
+template <typename T, int NU>
+__global__ __launch_bounds__(256) void qk_norm_store_pairs_kernel(
+    T* __restrict__ q_out, const T* __restrict__ qkv, int64_t qs, const int64_t* __restrict__ positions,
+    const float* __restrict__ qw, const float* __restrict__ kw, const float* __restrict__ table,
+    int rot, int trows, const float* __restrict__ vtab, int vrows, T* __restrict__ k_cache,
+    T* __restrict__ v_cache, const int64_t* __restrict__ slots, int H, int G, int dk, int dv,
+    int bs, int prow, int num_blocks, float eps) {
+  __shared__ float scratch[2][4];
+  const int64_t t = blockIdx.x;
+  const T* row = qkv + t * qs;
+  const int64_t slot = slots[t];
+  const bool store = k_cache != nullptr && slot >= 0 && slot < (int64_t)num_blocks * bs;
+  const int uk = dk >> 4, uv = dv >> 4;                // units per head
+  const int nq = H * uk, nk = store ? G * uk : 0, nv = store ? G * uv : 0;
+  int64_t pos = positions[t];
+  if (pos < 0) pos = 0;
+  const float* cs = table != nullptr ? table + (pos < trows ? pos : trows - 1) * rot : nullptr;
+  const float* vcs = vtab != nullptr ? vtab + (pos < vrows ? pos : vrows - 1) * dv : nullptr;
+  float a[NU][8], b[NU][8], sq = 0.f, sk = 0.f;
+  int hd[NU], oa[NU], ob[NU], ri[NU];                  // head, piece offsets in it, pair index or -1
+#pragma unroll
+  for (int n = 0; n < NU; ++n) {
+    const int u = threadIdx.x + 256 * n;
+    hd[n] = -1;
+    if (u < nq + nk + nv) {
+      const bool isv = u >= nq + nk, isq = u < nq;
+      const int per = isv ? uv : uk, u0 = isq ? u : isv ? u - nq - nk : u - nq;
+      const int h = u0 / per, i = u0 - h * per, rd = isv ? (vcs ? dv : 0) : (cs ? rot : 0);
+      hd[n] = h;
+      ri[n] = i < (rd >> 4) ? 8 * i : -1;
+      oa[n] = ri[n] >= 0 ? 8 * i : 16 * i;
+      ob[n] = ri[n] >= 0 ? (rd >> 1) + 8 * i : 16 * i + 8;
+      const T* src = row + (isq ? h * dk : isv ? (H + G) * dk + h * dv : (H + h) * dk);
+      load8(src + oa[n], a[n]);
+      load8(src + ob[n], b[n]);
+      float ss = 0.f;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) ss += a[n][e] * a[n][e] + b[n][e] * b[n][e];
+      if (isq) sq += ss;
+      else if (!isv) sk += ss;
+    }
+  }
+  sq = wave_sum(sq);
+  sk = wave_sum(sk);
+  if ((threadIdx.x & 63) == 0) {
+    scratch[0][threadIdx.x >> 6] = sq;
+    scratch[1][threadIdx.x >> 6] = sk;
+  }
+  __syncthreads();
+  sq = (scratch[0][0] + scratch[0][1]) + (scratch[0][2] + scratch[0][3]);
+  sk = (scratch[1][0] + scratch[1][1]) + (scratch[1][2] + scratch[1][3]);
+  const float rq = 1.f / sqrtf(sq / (float)(H * dk) + eps);
+  const float rk = store ? 1.f / sqrtf(sk / (float)(G * dk) + eps) : 0.f;
+  const int64_t blk = store ? slot / bs : 0, off = store ? slot % bs : 0;
+#pragma unroll
+  for (int n = 0; n < NU; ++n) {
+    if (hd[n] < 0) continue;
+    const int u = threadIdx.x + 256 * n, h = hd[n];
+    const bool isv = u >= nq + nk, isq = u < nq;
+    if (!isv) {
+      const float* w = (isq ? qw : kw) + h * dk;
+      const float f = isq ? rq : rk;
+      float wa[8], wb[8];
+      load8(w + oa[n], wa);
+      load8(w + ob[n], wb);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        a[n][e] *= f * wa[e];
+        b[n][e] *= f * wb[e];
+      }
+    }
+    if (ri[n] >= 0) {
+      const float* rc = isv ? vcs : cs;
+      float c[8], sn[8];
+      load8(rc + ri[n], c);
+      load8(rc + ((isv ? dv : rot) >> 1) + ri[n], sn);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const float x = a[n][e], y = b[n][e];
+        a[n][e] = x * c[e] - y * sn[e];
+        b[n][e] = y * c[e] + x * sn[e];
+      }
+    }
+    T* dst = isq ? q_out + (t * H + h) * dk
+                 : isv ? v_cache + ((blk * G + h) * prow + off) * dv
+                       : k_cache + ((blk * G + h) * prow + off) * dk;
+    store_vec<T, 8>(dst + oa[n], a[n]);
+    store_vec<T, 8>(dst + ob[n], b[n]);
+  }
+}
+
+// Blocks of `pool` tokens completed by prefill chunks: one workgroup per (work item of blk_rows
+// chunk rows, kv head); a thread takes VEC adjacent columns of one block's key or value row.
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void pool_chunks_kernel(
+    T* k_cache, T* v_cache, const int64_t* __restrict__ slots, const int* __restrict__ qsl,
+    const int* __restrict__ seq_lens, const int* __restrict__ pbt, int bt_stride,
+    const int* __restrict__ work_seq, const int* __restrict__ work_blk, int blk_rows, int G, int dk,
+    int dv, int krs, int vrs, int bs, int prow, int num_blocks, int pool) {
+  const int seq = work_seq[blockIdx.x], g = blockIdx.y;
+  const int q0 = qsl[seq], qlen = qsl[seq + 1] - q0, ctx0 = seq_lens[seq] - qlen;
+  const int r0 = work_blk[blockIdx.x] * blk_rows;
+  if (r0 >= qlen || ctx0 < 0) return;
+  const int p0 = ctx0 + r0, p1 = ctx0 + min(qlen, r0 + blk_rows);     // positions [p0, p1)
+  if (p1 > bt_stride * bs) return;
+  const int* bt = pbt + (int64_t)seq * bt_stride;
+  const int b0 = p0 / pool, nblk = p1 / pool - b0;                     // blocks ending in there
+  const int kc = dk / VEC, nc = kc + dv / VEC;
+  const float inv = 1.f / (float)pool;
+  for (int it = threadIdx.x; it < nblk * nc; it += 256) {
+    const int bl = it / nc, c = it - bl * nc, b = b0 + bl, last = b * pool + pool - 1;
+    if (slots[q0 + last - ctx0] < 0) continue;
+    T* base = c < kc ? k_cache + c * VEC : v_cache + (c - kc) * VEC;
+    const int rs = c < kc ? krs : vrs;
+    float acc[VEC];
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) acc[e] = 0.f;
+    int pg = (last + 1 - pool) / bs, in = last + 1 - pool - pg * bs;
+#pragma unroll 4
+    for (int j = 0; j < pool; ++j) {
+      int pb = bt[pg];
+      if (pb < 0 || pb >= num_blocks) pb = 0;
+      float v[VEC];
+      load_vec<T, VEC>(base + ((int64_t)(pb * G + g) * prow + in) * rs, v);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) acc[e] += v[e];
+      if (++in == bs) {
+        in = 0;
+        ++pg;
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) acc[e] *= inv;
+    int dp, dr;
+    pooled_place(b, pool, bs, dp, dr);
+    int db = bt[dp];
+    if (db < 0 || db >= num_blocks) db = 0;
+    store_vec<T, VEC>(base + ((int64_t)(db * G + g) * prow + dr) * rs, acc);
+  }
+}
+
 // Rows t0 .. of a step that complete a block of `pool` tokens (and are stored) write the
 // block's mean rows; grid (rows, G).
 template <typename T>
@@ -1051,6 +1197,19 @@ void launch_qk_norm_store(int dtype, void* q_out, const void* qkv, int64_t qs,
   // eight adjacent elements of one head and one half of the rotated part, 16-byte aligned
   const bool vec = dk % 8 == 0 && (!kv || dv % 8 == 0) && qs % 8 == 0 &&
                    reinterpret_cast<uintptr_t>(qkv) % 16 == 0;
+  const int units = (H * dk + (kv ? G * (dk + dv) : 0)) / 16;
+  if (vec && !inter && dk % 16 == 0 && (!kv || dv % 16 == 0) && rot % 16 == 0 && units <= 1024 &&
+      reinterpret_cast<uintptr_t>(qw) % 16 == 0 && reinterpret_cast<uintptr_t>(kw) % 16 == 0) {
+#define KGC_QKP(N)                                                                           \
+  KGC_DISPATCH_T(dtype, qk_norm_store_pairs_kernel<T, N><<<T_, 256, 0, s>>>(                 \
+      (T*)q_out, (const T*)qkv, qs, positions, qw, kw, table, rot, trows, vtab, vrows,       \
+      (T*)k_cache, (T*)v_cache, slots, H, G, dk, dv, bs, prow, num_blocks, eps))
+    if (units <= 256) KGC_QKP(1);
+    else if (units <= 512) KGC_QKP(2);
+    else KGC_QKP(4);
+#undef KGC_QKP
+    return;
+  }
 #define KGC_QKN(V)                                                                           \
   KGC_DISPATCH_T(dtype, qk_norm_store_kernel<T, V><<<T_, 256, lds, s>>>(                     \
       (T*)q_out, (const T*)qkv, qs, positions, qw, kw, table, rot, trows, vtab, vrows,       \
@@ -1067,6 +1226,20 @@ void launch_pool_kv(int dtype, void* k_cache, void* v_cache, const int64_t* slot
   KGC_DISPATCH_T(dtype, pool_kv_kernel<T><<<dim3(rows, G), 256, 0, s>>>(
       (T*)k_cache, (T*)v_cache, slots, qsl, seq_lens, pbt, ctx_lens, dbt, bt_stride, P, Tp, t0, G,
       dk, dv, krs, vrs, bs, prow, num_blocks, pool));
+}
+
+void launch_pool_chunks(int dtype, void* k_cache, void* v_cache, const int64_t* slots,
+                        const int* qsl, const int* seq_lens, const int* pbt, int bt_stride,
+                        const int* work_seq, const int* work_blk, int n_work, int blk_rows, int G,
+                        int dk, int dv, int krs, int vrs, int bs, int prow, int num_blocks,
+                        int pool, hipStream_t s) {
+  if (n_work <= 0) return;
+#define KGC_PC(V)                                                                            \
+  KGC_DISPATCH_T(dtype, pool_chunks_kernel<T, V><<<dim3(n_work, G), 256, 0, s>>>(            \
+      (T*)k_cache, (T*)v_cache, slots, qsl, seq_lens, pbt, bt_stride, work_seq, work_blk,    \
+      blk_rows, G, dk, dv, krs, vrs, bs, prow, num_blocks, pool))
+  if (dk % 8 == 0 && dv % 8 == 0 && krs % 8 == 0 && vrs % 8 == 0) KGC_PC(8); else KGC_PC(1);
+#undef KGC_PC
 }
 
 int window_attention_max_dv() { return 64 * MAX_DV_PER_LANE; }

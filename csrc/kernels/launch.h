@@ -297,6 +297,11 @@ void launch_qk_norm_store(int dtype, void* q_out, const void* qkv, int64_t qs,
                           void* k_cache, void* v_cache, const int64_t* slots, int T, int H, int G,
                           int dk, int dv, int bs, int prow, int num_blocks, float eps, bool inter,
                           hipStream_t s);
+void launch_pool_chunks(int dtype, void* k_cache, void* v_cache, const int64_t* slots,
+                        const int* qsl, const int* seq_lens, const int* pbt, int bt_stride,
+                        const int* work_seq, const int* work_blk, int n_work, int blk_rows, int G,
+                        int dk, int dv, int krs, int vrs, int bs, int prow, int num_blocks,
+                        int pool, hipStream_t s);
 void launch_pool_kv(int dtype, void* k_cache, void* v_cache, const int64_t* slots, const int* qsl,
                     const int* seq_lens, const int* pbt, const int* ctx_lens, const int* dbt,
                     int bt_stride, int P, int Tp, int t0, int rows, int G, int dk, int dv, int krs,

@@ -1,7 +1,9 @@
 """Microbenchmarks of the hybrid-decoder kernels beside the Llama-path kernel each one is
 closest to, at the layer shapes of the dilavik-w2048 / konovik-w2048 / nolesun-w2048 /
 llama-w2048 presets (``--only nolesun``: the parallel mixers' kernels; ``--only lorenex``: gated
-linear attention, the selective scan, unit-RMS attention inputs, PolyNorm, clamped experts).
+linear attention, the selective scan, unit-RMS attention inputs, PolyNorm, clamped experts;
+``--only generax``: the channel-wise delta rule, pooled blocks, rotated values, whole-row norms,
+each beside its like kernel on the same shapes).
 
     python tools/hybrid_bench.py [--reps 20] > profiles/hybrid_kernels.jsonl
 
@@ -16,6 +18,7 @@ import torch
 
 from kubernetes_gpu_cluster_amd import ops
 from kubernetes_gpu_cluster_amd.ops import reference as ref
+from kubernetes_gpu_cluster_amd.ops.gemm import linear
 
 DEV = torch.device("cuda")
 BF = torch.bfloat16
@@ -448,6 +451,105 @@ def lorenex(reps):
         emit("embed_pos", f"{T}x{W}", us, gbytes=T * W * 10 / 1e9)
 
 
+def generax(reps):
+    """The Generax kernels at the generax-w2048 layer shapes, each beside the closest kernel of
+    the other hybrid decoders at the same sizes."""
+    W, ff = 2048, 5504
+    shapes = (("prefill 32x512", [512] * 32, []), ("prefill 2x8192", [8192] * 2, []),
+              ("decode 64", [], [544] * 64), ("decode 256", [], [544] * 256))
+    for name, P_q, D_ctx in shapes:
+        n = len(P_q) + len(D_ctx)
+        m, _, _ = meta(P_q, list(P_q), D_ctx, 32, DEV, slots=list(range(n)))
+        T = sum(P_q) + len(D_ctx)
+        H, G, d, V, R = 16, 8, 128, 128, 128
+        C = 2 * G * d + H * V
+        qkv = torch.randn(T, C, device=DEV)
+        proj = torch.randn(T, 2 * R + 2 * H, device=DEV, dtype=BF)
+        S = torch.zeros(n, H, d, V, device=DEV)
+        decay = torch.rand(T, H * d, device=DEV) * 0.2 + 0.8
+        sb = 2 * n * H * d * V * 4
+        us = timed(lambda: ops.channel_delta_scan(qkv, proj[:, -H:], decay, S, m, H, G, d, V), reps)
+        emit("channel_delta_scan", name, us, gbytes=(sb + 4 * T * (C + H * d + H * V)) / 1e9,
+             tflop=7 * T * H * d * V / 1e12, like="gated_delta_scan")
+        S.zero_()
+        al, dtb = torch.rand(H, device=DEV), torch.randn(H, device=DEV) - 2
+        us = timed(lambda: ops.gated_delta_scan(qkv, proj[:, -2 * H:], al, dtb, S, m, H, G, d, V), reps)
+        emit("gated_delta_scan", name, us, gbytes=(sb + 4 * T * (C + H * V)) / 1e9,
+             tflop=6 * T * H * d * V / 1e12)
+        a2, g2 = (torch.randn(H * x, R, device=DEV, dtype=BF) * 0.1 for x in (d, V))
+        na, db = -torch.rand(H * d, device=DEV) - 1, torch.randn(H * d, device=DEV) - 3
+        us = timed(lambda: ops.delta_gates(proj[:, :2 * R], a2, g2, na, db), reps)
+        emit("delta_gates", f"{T}x{2 * R}->{H * (d + V)}", us,
+             gbytes=T * (4 * R + 4 * H * d + 2 * H * V) / 1e9, tflop=2 * T * R * H * (d + V) / 1e12,
+             like="two GEMMs + elementwise")
+        us = timed(lambda: (linear(proj[:, :R], a2), linear(proj[:, R:2 * R], g2)), reps)
+        emit("the two GEMMs alone", f"{T}x{R}->{H * d}, {H * V}", us, gbytes=T * (4 * R + 2 * H * (d + V)) / 1e9)
+        o, gate = torch.randn(T, H * V, device=DEV), torch.randn(T, H * V, device=DEV, dtype=BF)
+        nw = torch.ones(H * V, device=DEV)
+        us = timed(lambda: ops.head_norm_gate(o, gate, nw, H, 1e-6, BF), reps)
+        emit("head_norm_gate", f"{T}x{H * V}", us, gbytes=T * H * V * 8 / 1e9, like="gated_rms_norm")
+        feats = torch.empty(T, H * V, device=DEV, dtype=BF)
+        us = timed(lambda: ops.gated_rms_norm(o, gate, nw, H, 1e-6, False, feats), reps)
+        emit("gated_rms_norm", f"{T}x{H * V}", us, gbytes=T * H * V * 8 / 1e9)
+        # results joining the stream: two normed, one plain, beside one plain / one normed
+        x, w = torch.zeros(T, W, device=DEV), torch.ones(W, device=DEV)
+        ys = [torch.randn(T, W, device=DEV, dtype=BF) for _ in range(3)]
+        for k, adds in (("2 normed + 1", [(ys[0], w), (ys[1], w), (ys[2], None)]), ("1", [(ys[0], None)])):
+            us = timed(lambda: ops.residual_sum_norm(x, adds, w, 1e-6, BF), reps)
+            emit(f"residual_sum_norm ({k})", f"{T}x{W}", us, gbytes=T * W * (8 + 2 + 2 * len(adds)) / 1e9,
+                 like="residual_norm")
+        us = timed(lambda: ops.residual_norm(x, ys[0], 1.0, w, 1e-6, BF, add_norm_w=w), reps)
+        emit("residual_norm (1 normed)", f"{T}x{W}", us, gbytes=T * W * 12 / 1e9)
+        wide = torch.randn(T, 3072 + 2 * ff, device=DEV, dtype=BF)
+        buf = torch.empty(T, 2048 + ff, device=DEV, dtype=BF)
+        us = timed(lambda: ops.silu_mul(wide[:, 3072:], buf[:, 2048:]), reps)
+        emit("silu_mul (between column slices)", f"{T}x{ff}", us, gbytes=T * ff * 6 / 1e9, like="silu_mul")
+        gu = torch.randn(T, 2 * ff, device=DEV, dtype=BF)
+        us = timed(lambda: ops.silu_mul(gu), reps)
+        emit("silu_mul", f"{T}x{ff}", us, gbytes=T * ff * 6 / 1e9)
+    H, G, d, bs, win = 16, 4, 128, 32, 1024
+    for name, P_q, P_sl, D_ctx in (("prefill 32x512", [512] * 32, [512] * 32, []),
+                                   ("prefill 8x2048", [2048] * 8, [2048] * 8, []),
+                                   ("prefill 2x8192", [8192] * 2, [8192] * 2, []),
+                                   ("decode 64 @544", [], [], [544] * 64),
+                                   ("decode 256 @544", [], [], [544] * 256),
+                                   ("decode 64 @8000", [], [], [8000] * 64)):
+        m, tables, nb = meta(P_q, P_sl, D_ctx, bs, DEV)
+        T = sum(P_q) + len(D_ctx)
+        pos = torch.cat([torch.arange(s) for s in P_sl]) if P_q else torch.tensor(D_ctx) - 1
+        pos = pos.to(DEV)
+        seq = torch.repeat_interleave(torch.arange(len(P_sl) + len(D_ctx)), torch.tensor(P_q or [1] * len(D_ctx)))
+        slots = tables[seq.to(DEV), pos // bs].long() * bs + pos % bs
+        m.slot_mapping = slots
+        qkv = torch.randn(T, (H + 2 * G) * d, device=DEV, dtype=BF)
+        kc = torch.randn(nb, G, bs, d, device=DEV, dtype=BF)
+        vc = torch.randn(nb, G, bs, d, device=DEV, dtype=BF)
+        one = torch.ones(H * d, device=DEV)
+        tab = ops.ref.rope_table_linear(d, 8192, 1e4, 8.0).to(DEV)
+        us = timed(lambda: ops.qk_norm_store(qkv, pos, one, one[: G * d], 1e-6, tab, tab, kc, vc, slots, H, G, d, d), reps)
+        gb = T * (H + 2 * G) * d * 4 / 1e9
+        emit("qk_norm_store (norms, rotated q k v)", name, us, gbytes=gb, like="rope_kv_store")
+        us = timed(lambda: ops.rope_kv_store(qkv, pos, tab, kc, vc, slots, H, G, d, d), reps)
+        emit("rope_kv_store", name, us, gbytes=gb)
+        q = torch.randn(T, H, d, device=DEV, dtype=BF)
+        # (query, key) pairs / decode rows read: window, and with pooled blocks of 16
+        P = [p + 1 for s in P_sl for p in range(s)] if P_q else D_ctx
+        keys = sum(min(p, win) for p in P)
+        for kind in ("window", "rotated values", "pooled blocks"):
+            pool = 16 if kind == "pooled blocks" else 0
+            k2, v2 = kc, vc
+            if pool:
+                k2 = torch.randn(nb, G, bs + bs // pool, d, device=DEV, dtype=BF)
+                v2 = torch.randn(nb, G, bs + bs // pool, d, device=DEV, dtype=BF)
+            tot = keys + (sum(max(0, p - win) // pool for p in P) if pool else 0)
+            us = timed(lambda: ops.window_attention(q, k2, v2, pos, m, 0.09, win, 0, None, pool=pool,
+                                                    block_size=bs if pool else 0,
+                                                    v_table=tab if kind == "rotated values" else None), reps)
+            emit(f"window_attention ({kind})", name, us, gbytes=None if P_q else tot * G * 4 * d / 1e9,
+                 tflop=tot * H * 4 * d / 1e12 if P_q else None,
+                 like=None if kind == "window" else "window_attention (window)")
+
+
 if __name__ == "__main__":
     ap = argparse.ArgumentParser()
     ap.add_argument("--reps", type=int, default=20)
@@ -456,4 +558,4 @@ if __name__ == "__main__":
     ops.load_extension(strict=True)
     for part in a.only.split(","):
         {"attention": attention, "recurrent": recurrent, "rows": rows, "konovik": konovik,
-         "nolesun": nolesun, "lorenex": lorenex}[part](a.reps)
+         "nolesun": nolesun, "lorenex": lorenex, "generax": generax}[part](a.reps)
