@@ -1542,7 +1542,7 @@ void qk_norm_store(Tensor q_out, Tensor qkv, Tensor positions, Tensor qw, std::o
   check_gpu(qkv, "qkv");
   c10::hip::HIPGuardMasqueradingAsCUDA g(qkv.device());
   const bool kv = k_cache.has_value();
-  TORCH_CHECK(H >= 1 && G >= 1 && dk >= 1 && dv >= 1 && kgc::qk_norm_store_ok((int)H, (int)G, (int)dk, (int)dv),
+  TORCH_CHECK(H >= 1 && G >= 1 && dk >= 1 && dv >= 1 && (H + G) * dk + G * dv < (int64_t(1) << 24),
               "kgc.qk_norm_store: head sizes");
   TORCH_CHECK(qkv.dim() == 2 && qkv.stride(1) == 1 && act_dtype(qkv) &&
               qkv.size(1) >= H * dk + (kv ? G * (dk + dv) : 0),

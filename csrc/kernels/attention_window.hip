@@ -908,9 +908,9 @@ __device__ __forceinline__ void store_vec(T* p, const float (&v)[VEC]) {
 // the whole q row and the whole k row over their root mean squares times a weight per column,
 // rotation of q and k on the first `rot` dims (table: cos | sin) and of v on all dv (vtab);
 // q -> q_out [T, H, dk], k and v -> the cache row of the token's slot.  The row sits in LDS as
-// fp32 between the sums and the outputs.  VEC 8: a thread makes 8 adjacent outputs (head sizes,
+// fp32 between the sums and the outputs (STAGED), or is read again.  VEC 8: a thread makes 8 adjacent outputs (head sizes,
 // rotated parts and strides are multiples that keep them in one head and one half).
-template <typename T, int VEC>
+template <typename T, int VEC, bool STAGED>
 __global__ __launch_bounds__(256) void qk_norm_store_kernel(
     T* __restrict__ q_out, const T* __restrict__ qkv, int64_t qs, const int64_t* __restrict__ positions,
     const float* __restrict__ qw, const float* __restrict__ kw, const float* __restrict__ table,
@@ -932,7 +932,7 @@ __global__ __launch_bounds__(256) void qk_norm_store_kernel(
     float ss = 0.f;
 #pragma unroll
     for (int i = 0; i < VEC; ++i) {
-      lds[e + i] = v[i];
+      if constexpr (STAGED) lds[e + i] = v[i];
       ss += v[i] * v[i];
     }
     if (e < nq) sq += ss;
@@ -956,7 +956,12 @@ __global__ __launch_bounds__(256) void qk_norm_store_kernel(
     const float* rc = isv ? vcs : cs;
     const int rd = rc == nullptr ? 0 : isv ? dv : rot, half = rd >> 1;
     const int b0 = e - i0;                             // the head's first element
-    auto val = [&](int i) { return lds[b0 + i] * (isv ? 1.f : f * w[e0 - i0 + i]); };
+    auto val = [&](int i) {
+      float x;
+      if constexpr (STAGED) x = lds[b0 + i];
+      else x = to_f(row[b0 + i]);
+      return x * (isv ? 1.f : f * w[e0 - i0 + i]);
+    };
     float v[VEC];
 #pragma unroll
     for (int k = 0; k < VEC; ++k) {
@@ -1181,10 +1186,6 @@ void launch_norm_kv_store(int out_dtype, const float* qkv, int64_t qs, const int
       num_blocks, eps, qk_unit, v_unit, coef, every));
 }
 
-bool qk_norm_store_ok(int H, int G, int dk, int dv) {
-  return ((int64_t)(H + G) * dk + (int64_t)G * dv) * 4 <= 64 * 1024;
-}
-
 void launch_qk_norm_store(int dtype, void* q_out, const void* qkv, int64_t qs,
                           const int64_t* positions, const float* qw, const float* kw,
                           const float* table, int rot, int trows, const float* vtab, int vrows,
@@ -1193,7 +1194,9 @@ void launch_qk_norm_store(int dtype, void* q_out, const void* qkv, int64_t qs,
                           hipStream_t s) {
   if (T_ <= 0) return;
   const bool kv = k_cache != nullptr;
-  const size_t lds = sizeof(float) * (size_t)(H * dk + (kv ? G * (dk + dv) : 0));
+  const size_t row_lds = sizeof(float) * (size_t)(H * dk + (kv ? G * (dk + dv) : 0));
+  const bool staged = row_lds <= 64 * 1024;
+  const size_t lds = staged ? row_lds : 0;
   // eight adjacent elements of one head and one half of the rotated part, 16-byte aligned
   const bool vec = dk % 8 == 0 && (!kv || dv % 8 == 0) && qs % 8 == 0 &&
                    reinterpret_cast<uintptr_t>(qkv) % 16 == 0;
@@ -1210,11 +1213,13 @@ void launch_qk_norm_store(int dtype, void* q_out, const void* qkv, int64_t qs,
 #undef KGC_QKP
     return;
   }
-#define KGC_QKN(V)                                                                           \
-  KGC_DISPATCH_T(dtype, qk_norm_store_kernel<T, V><<<T_, 256, lds, s>>>(                     \
+#define KGC_QKN(V, ST)                                                                       \
+  KGC_DISPATCH_T(dtype, qk_norm_store_kernel<T, V, ST><<<T_, 256, lds, s>>>(                 \
       (T*)q_out, (const T*)qkv, qs, positions, qw, kw, table, rot, trows, vtab, vrows,       \
       (T*)k_cache, (T*)v_cache, slots, H, G, dk, dv, bs, prow, num_blocks, eps, inter))
-  if (vec) KGC_QKN(8); else KGC_QKN(1);
+  if (!staged) KGC_QKN(1, false);
+  else if (vec) KGC_QKN(8, true);
+  else KGC_QKN(1, true);
 #undef KGC_QKN
 }
 

@@ -289,8 +289,6 @@ struct WindowExtra {
   int vrows;
   bool vinter;
 };
-// whether a row of (H + G) dk + G dv fp32 values fits the store kernel's LDS
-bool qk_norm_store_ok(int H, int G, int dk, int dv);
 void launch_qk_norm_store(int dtype, void* q_out, const void* qkv, int64_t qs,
                           const int64_t* positions, const float* qw, const float* kw,
                           const float* table, int rot, int trows, const float* vtab, int vrows,

@@ -447,6 +447,34 @@ def test_preset_runs_through_sampling(device, dtype):
         llm.shutdown()
 
 
+@pytest.mark.parametrize("device,dtype", [CPU, GPU32])
+def test_cached_prefixes_of_a_model_without_recurrences(tmp_path, device, dtype):
+    """Only attention layers: everything a prefix leaves behind lies in its pages, so a second
+    prompt with the same beginning starts from them (keys and values turned by the same
+    positions, shared by the layers that read them)."""
+    if device == "cuda" and not torch.cuda.is_available():
+        pytest.skip("no GPU")
+    cfg = config([attl(att()), attl(att(kv_from=0, size=40)), attl(att(size=25, rot=12, vdim=6))])
+    wts = write_model(str(tmp_path), cfg, 61)
+    llm = LLM(model=str(tmp_path), dtype=dtype, device=device, block_size=8, max_num_seqs=2, max_model_len=96,
+              num_gpu_blocks_override=30, cuda_graph_max_bs=2)
+    try:
+        assert not llm.engine.mcfg.has_recurrent_state
+        head = tokens_for(cfg, 33, 5)
+        for tail in ([7, 9], [3], [11, 2, 5, 1]):
+            seq = head + tail
+            out = llm.generate([seq], SamplingParams(temperature=0.0, max_tokens=6, ignore_eos=True))[0]
+            for tok in out.output_token_ids:
+                lg = oracle.forward(cfg, wts, seq)[-1]
+                top2 = np.sort(lg)[-2:]
+                if top2[1] - top2[0] > 1e-3 * np.abs(lg).max():
+                    assert tok == int(np.argmax(lg))
+                seq = seq + [tok]
+        assert llm.engine.bm.hit_tokens >= 2 * 32
+    finally:
+        llm.shutdown()
+
+
 def test_config_reader(models):
     d, cfg, wts = models["mixed"]
     mc, wdir = resolve_model(d)

@@ -264,6 +264,30 @@ def test_rotated_values_cancel_in_a_window_of_one(dev, inter):
                                        rtol=1e-4, atol=1e-5)
 
 
+@pytest.mark.parametrize("dev", GPU)
+@pytest.mark.parametrize("H,G,dk,dv,inter", [(120, 8, 128, 64, True), (140, 4, 127, 30, False), (128, 8, 128, 128, False),
+                                             (32, 8, 128, 128, False), (32, 4, 64, 64, True)])
+def test_wide_rows_of_heads(dev, H, G, dk, dv, inter):
+    """Rows longer than the LDS staging and than one unit per thread, in both pair layouts,
+    against the reference op."""
+    dev = dev_of(dev)
+    n, page = 9, 4
+    q, k, v, qw, kw = qkv_for(n, H, G, dk, dv)
+    x = torch.tensor(np.concatenate([q, k, v], 1), dtype=torch.float32)
+    rot = dk // 2 // 16 * 16
+    tab, vtab = ops.ref.rope_table_linear(rot, n, 50.0, 2.0), ops.ref.rope_table_linear(dv, n, 50.0)
+    qw, kw = torch.tensor(qw, dtype=torch.float32), torch.tensor(kw, dtype=torch.float32)
+    slots = torch.tensor([4, 5, 6, 7, -1, 8, 9, 10, 11])
+    pos = torch.arange(n)
+    want = torch.zeros(4, G, page, dk), torch.zeros(4, G, page, dv)
+    wq = ops.ref.qk_norm_store(x, pos, qw, kw, 1e-6, tab, vtab, *want, slots, H, G, dk, dv, page, inter)
+    got = want[0].clone().zero_().to(dev), want[1].clone().zero_().to(dev)
+    gq = ops.qk_norm_store(x.to(dev), pos.to(dev), qw.to(dev), kw.to(dev), 1e-6, tab.to(dev), vtab.to(dev), *got,
+                           slots.to(dev), H, G, dk, dv, page, inter)
+    for a, b in ((gq, wq), (got[0], want[0]), (got[1], want[1])):
+        np.testing.assert_allclose(a.cpu().numpy(), b.numpy(), rtol=1e-4, atol=1e-5)
+
+
 @pytest.mark.parametrize("dev", DEV)
 def test_queries_on_another_layers_cache(dev):
     """A layer without keys and values of its own: q columns only, the cache left as it is."""
