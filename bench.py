@@ -644,8 +644,8 @@ def _compare_one(model: str, args) -> dict:
 
 def main_compare(args):
     """--mode compare: the hybrid presets (generax, lorenex, nolesun, dilavik, konovik) beside
-    the Llama-style decoders of equal size (models/configs.py), same requests, same engine settings, one JSON line per model and a
-    closing line with the ratios.  Random weights, synthetic prompts."""
+    the Llama-style decoders of equal size (models/configs.py), same requests, same engine
+    settings, one JSON line per model and a closing line with the ratios.  Random weights, synthetic prompts."""
     assert torch.cuda.is_available(), "bench.py --mode compare needs a GPU"
     rows = []
     for size in args.compare_sizes.split(","):

@@ -12,10 +12,13 @@ the bytes or FLOPs the call has to move or do at least, as GB/s or TFLOP/s.  Pre
 32 chunks of 512 tokens (16384 rows); decode shapes: 64 and 256 rows at context 544."""
 import argparse
 import json
+import os
+import sys
 import types
 
 import torch
 
+sys.path.insert(0, os.path.dirname(os.path.dirname(os.path.abspath(__file__))))
 from kubernetes_gpu_cluster_amd import ops
 from kubernetes_gpu_cluster_amd.ops import reference as ref
 from kubernetes_gpu_cluster_amd.ops.gemm import linear
