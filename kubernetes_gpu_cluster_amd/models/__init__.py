@@ -24,6 +24,7 @@ from .llama import LlamaForCausalLM
 from .lorenex import LorenexForCausalLM
 from .nolesun import NolesunForCausalLM
 from .opt import OPTForCausalLM
+from .ratizen import RatizenForCausalLM
 
 
 def build_model(cfg: ModelConfig, dtype=torch.bfloat16, device=None):
@@ -39,6 +40,8 @@ def build_model(cfg: ModelConfig, dtype=torch.bfloat16, device=None):
         return LorenexForCausalLM(cfg, dtype, device)
     if cfg.arch == "generax":
         return GeneraxForCausalLM(cfg, dtype, device)
+    if cfg.arch == "ratizen":
+        return RatizenForCausalLM(cfg, dtype, device)
     return LlamaForCausalLM(cfg, dtype, device)
 
 

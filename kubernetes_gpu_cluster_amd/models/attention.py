@@ -193,6 +193,69 @@ class LatentAttention(nn.Module):
         return self.o_proj(ops.gate_mul(o.transpose(0, 1), proj[:, self.n_q + self.n_kv:]))
 
 
+class LatentQueryAttention(nn.Module):
+    """Latent attention (see ``LatentAttention``) whose queries pass a normed latent of their own
+    (``q_rank``) and whose heads are gated by one sigmoid each, computed from the layer's input:
+
+      [dq | c | k_r | g] = W h     (one merged projection)
+      q = W_uq (RMSNorm(dq));   cache row [RMSNorm(c) | rotated k_r];   gate = sigmoid(g)
+      attention of [W_uk^T q_u | rotated q_r] over the cache rows, times gate
+      result W_o (W_uv per head)
+
+    Both per-head matrices run as ``head_gemm``; the first one's launch also rotates the
+    queries, and the gate rides in the attention kernels' epilogue."""
+
+    def __init__(self, hidden: int, spec, eps: float, dtype, device):
+        super().__init__()
+        from ..parallel.layers import ReplicatedLinear
+        self.spec, self.eps = spec, eps
+        H, d, r, dv, rank, qr = (spec.heads, spec.dim, spec.rot_dims, spec.vdim, spec.kv_rank,
+                                 spec.q_rank)
+        assert r % 2 == 0 and qr > 0 and spec.head_gate
+        # checkpoint names -> rows of the merged projection
+        self.rows = {"dq": (0, qr), "dkv": (qr, rank + r), "g": (qr + rank + r, H)}
+        n = -(-(qr + rank + r + H) // 64) * 64
+        self.proj = ReplicatedLinear(hidden, n, dtype=dtype, device=device)
+        self.proj.weight.data.zero_()                       # padding rows stay zero
+        self.uq_proj = ReplicatedLinear(qr, H * (d + r), dtype=dtype, device=device)
+        self.o_proj = ReplicatedLinear(H * dv, hidden, dtype=dtype, device=device)
+        z = lambda *s: nn.Parameter(torch.zeros(*s, dtype=dtype, device=device),   # noqa: E731
+                                    requires_grad=False)
+        one = lambda k: nn.Parameter(torch.ones(k, dtype=torch.float32, device=device),  # noqa: E731
+                                     requires_grad=False)
+        self.w_uk = z(H, rank, d)          # [head, latent, unrotated dim]
+        self.w_uv = z(H, dv, rank)         # [head, value dim, latent]
+        self.q_norm, self.kv_norm = one(qr), one(rank)
+        self.scale = (d + r) ** -0.5 if spec.scale is None else spec.scale
+        self.rope = None
+
+    prepare = LatentAttention.prepare
+
+    def cache_shape(self) -> tuple:
+        """One group whose rows hold the latent and the rotary key part; values are read from
+        the latent columns."""
+        return (1, self.spec.kv_rank + self.spec.rot_dims, 0)
+
+    def forward(self, h: torch.Tensor, positions: torch.Tensor, ctx: ForwardContext,
+                cache_idx: int) -> torch.Tensor:
+        sp = self.spec
+        H, d, r, dv, rank = sp.heads, sp.dim, sp.rot_dims, sp.vdim, sp.kv_rank
+        T = h.shape[0]
+        cache = ctx.kv_caches[cache_idx][0]                 # [nb, 1, bs, rank + r]
+        cq, gate = ops.latent_down_store(self.proj(h), positions, self.rope, self.q_norm,
+                                         self.kv_norm, self.eps, cache, ctx.attn.slot_mapping, r, H)
+        qf = self.uq_proj(cq).view(T, H, d + r)
+        q = torch.empty(T, H, rank + r, dtype=h.dtype, device=h.device)
+        ops.head_gemm(qf[:, :, :d], self.w_uk, q, qf[:, :, d:] if r else None, positions, self.rope)
+        w = sp.window
+        o = ops.window_attention(q, cache, cache[..., :rank], positions, ctx.attn, self.scale,
+                                 w.size if w else 0, 0, gate,
+                                 chunked=bool(w and w.chunked), sink=sp.sink)
+        y = torch.empty(T, H, dv, dtype=h.dtype, device=h.device)
+        ops.head_gemm(o.view(T, H, rank), self.w_uv, y)
+        return self.o_proj(y.view(T, H * dv))
+
+
 class AttentionCore(nn.Module):
     """The part of a softmax attention mixer between its projections, for mixers whose
     projections are merged with a neighbour's (a parallel mixer): reads q | k | v (| the
@@ -211,7 +274,9 @@ class AttentionCore(nn.Module):
     1 + coef * ln(floor((p + 1) / every) + 1); these take the place of the rotation.
 
     ``spec.qk_norm`` RMS-norms the whole q and the whole k row (all heads at once) with one
-    weight per column before rotation; a learned factor per query head on the scores
+    weight per column before rotation; ``spec.head_norm`` RMS-norms every head's q and k with one
+    weight per dimension, without rotation; ``spec.sink`` is a score without a value that joins
+    every softmax; ``spec.window.chunked`` limits a query to its own chunk; a learned factor per query head on the scores
     (``spec.head_temp``) is part of the q weight.  ``spec.rotary.values`` turns the cached
     values by their positions and each head's output back by the row's.  With
     ``spec.window.pool`` the cache pages also hold the mean rows of blocks that have left the
@@ -234,11 +299,13 @@ class AttentionCore(nn.Module):
         one = lambda n: nn.Parameter(torch.ones(n, dtype=torch.float32, device=device),  # noqa: E731
                                      requires_grad=False)
         # the q weight carries the heads' score factors; the k weight only where there are keys
-        self.q_norm = one(H * dk) if spec.qk_norm else None
-        self.k_norm = one(G * dk) if spec.qk_norm and self.own_kv else None
+        self.q_norm = one(H * dk) if spec.qk_norm else one(dk) if spec.head_norm else None
+        self.k_norm = (one(G * dk) if spec.qk_norm and self.own_kv else
+                       one(dk) if spec.head_norm else None)
+        assert not (spec.qk_norm and spec.head_norm)
         self.pool = spec.window.pool if spec.window else 0
         assert not self.pool or spec.window.size > 0
-        self.unit = bool(spec.qk_unit or spec.v_unit or spec.q_temp)
+        self.unit = bool(spec.qk_unit or spec.v_unit or spec.q_temp or spec.head_norm)
         assert not (self.unit and spec.rot_dims), "unit-RMS inputs take the rotation's place"
         self.conv_w = (nn.Parameter(torch.zeros(self.n_qkv, spec.conv, dtype=torch.float32,
                                                 device=device), requires_grad=False)
@@ -289,9 +356,10 @@ class AttentionCore(nn.Module):
                                   sp.kv_heads, sp.dim, sp.vdim, bs,
                                   bool(rotary and rotary.interleaved))
         elif self.unit:
-            q = ops.norm_kv_store(qkv.float(), positions, kc, vc, ctx.attn.slot_mapping, sp.heads,
-                                  sp.kv_heads, sp.dim, sp.vdim, self.eps, sp.qk_unit, sp.v_unit,
-                                  sp.q_temp, proj.dtype)
+            q = ops.norm_kv_store(qkv, positions, kc, vc, ctx.attn.slot_mapping, sp.heads,
+                                  sp.kv_heads, sp.dim, sp.vdim, self.eps,
+                                  sp.qk_unit or sp.head_norm, sp.v_unit, sp.q_temp, proj.dtype,
+                                  self.q_norm, self.k_norm)
         else:
             q = ops.rope_kv_store(qkv.to(proj.dtype), positions, self.rope, kc, vc,
                                   ctx.attn.slot_mapping, sp.heads, sp.kv_heads, sp.dim, sp.vdim,
@@ -301,4 +369,5 @@ class AttentionCore(nn.Module):
         ops.window_attention(q, kc, vc, positions, ctx.attn, self.scale, w.size if w else 0,
                              w.keep_first if w else 0, None, sp.softcap, self.out_scale, out=out,
                              elem_gate=g, pool=self.pool, block_size=bs, v_table=self.v_rope,
-                             interleaved=bool(rotary and rotary.interleaved))
+                             interleaved=bool(rotary and rotary.interleaved),
+                             chunked=bool(w and w.chunked), sink=sp.sink)

@@ -22,10 +22,13 @@ from typing import Optional
 class WindowSpec:
     """Sliding-window visibility with kept first tokens: query i sees key j when
     j <= i and (i - j < size or j < keep_first).  ``pool`` > 0: query i also sees one mean
-    key and value for every block of ``pool`` tokens whose last token j has i - j >= size."""
+    key and value for every block of ``pool`` tokens whose last token j has i - j >= size.
+    ``chunked``: query i sees key j <= i of its own chunk of ``size`` positions instead
+    (i // size == j // size, counted from the sequence's position 0)."""
     size: int
     keep_first: int = 0
     pool: int = 0
+    chunked: bool = False
 
 
 @dataclasses.dataclass(frozen=True)
@@ -67,8 +70,13 @@ class FeedForwardSpec:
     # "sigmoid": the routing described above; "softmax": logits W_r h + b_r, the ``top``
     # largest chosen, their weights the softmax over the chosen logits only; "softmax_all":
     # scores = softmax over all router outputs, the choice made on score + a per-output
+    # correction, the weights the chosen scores as they are; "sigmoid_raw": sigmoid scores, no
     # correction, the weights the chosen scores as they are
     router: str = "sigmoid"
+    # the routing weight multiplies the expert's input instead of its output
+    weight_input: bool = False
+    # the shared expert is scaled by a per-token sigmoid gate
+    shared_gate: bool = True
     # act "polynorm" (dense, not gated): a N(z) + b N(z^2) + c N(z^3) + e with N = division
     # by the row's root mean square and four learned numbers.  act "swiglu_clamp" (gated):
     # g = min(gate h, limit), u = clamp(up h, -limit, limit), g sigmoid(1.702 g) (u + 1)
@@ -91,6 +99,7 @@ class MixerSpec:
     of one ``kv_rank``-wide normed latent per token; a head's query / key has ``dim``
     unrotated dimensions plus ``rot_dims`` rotated ones, the rotated key part shared by
     all heads.  The paged cache holds the latent and the rotated key part only.
+    ``q_rank`` > 0: the queries pass a normed latent of that width of their own.
     kind "mingru": an element-wise gated recurrence of ``width`` channels (one fp32 state
     vector per sequence) with a SiLU output gate.
     kind "parallel": two mixers side by side on the same input, ``left`` (an "attention"
@@ -158,6 +167,12 @@ class MixerSpec:
     qk_norm: bool = False
     head_temp: bool = False
     kv_from: Optional[int] = None
+    # latent_attention: width of the normed latent the queries pass (0: none)
+    q_rank: int = 0
+    # attention: an RMS norm per head on q and on k, one weight of the head's size shared by all
+    # heads; a score without a value that joins every softmax's denominator (None: none)
+    head_norm: bool = False
+    sink: Optional[float] = None
     left: Optional["MixerSpec"] = None      # parallel
     right: Optional["MixerSpec"] = None
     left_scale: float = 1.0
@@ -223,6 +238,11 @@ class ModelConfig:
     # arch "generax": mixer and feed-forward of a layer read one norm's output and join the
     # stream together; the logits pass cap * tanh(. / cap) when ``logit_softcap`` > 0
     logit_softcap: float = 0.0
+    # arch "ratizen": hyper-connections -- the residual stream is ``streams`` copies that every
+    # sublayer reads through and writes back into by learned weights; the logits are multiplied
+    # by ``logit_scale``
+    streams: int = 1
+    logit_scale: float = 1.0
 
     @property
     def q_size(self) -> int:
@@ -261,8 +281,11 @@ class ModelConfig:
                 if self.weights_of and self.weights_of[li] != li:
                     continue                # a layer that runs with another layer's tensors
                 if sp.kind == "latent_attention":
-                    n += h * (sp.heads * (sp.dim + sp.rot_dims) + sp.kv_rank + sp.rot_dims)
-                    n += sp.kv_rank * sp.heads * (sp.dim + sp.vdim) + 2 * h * sp.heads * sp.vdim
+                    nq = sp.heads * (sp.dim + sp.rot_dims)
+                    n += sp.q_rank * (h + nq) if sp.q_rank else h * nq
+                    n += h * (sp.kv_rank + sp.rot_dims)
+                    n += sp.kv_rank * sp.heads * (sp.dim + sp.vdim) + h * sp.heads * sp.vdim
+                    n += h * (sp.heads if sp.head_gate else sp.heads * sp.vdim)
                 elif sp.kind == "mingru":
                     n += 4 * h * sp.width
                 elif sp.kind == "parallel":
@@ -294,8 +317,8 @@ class ModelConfig:
                 elif f.kind == "dense":
                     n += (2 if f.gated is False else 3) * h * f.ff
                 else:
-                    n += ((3 if f.gated else 2) * h * f.experts * f.ff + 2 * h * f.shared_ff
-                          + h * (f.experts + f.identity + 1))
+                    n += ((3 if f.gated else 2) * h * (f.experts * f.ff + f.shared_ff)
+                          + h * (f.experts + f.identity + (1 if f.shared_gate else 0)))
                 n += 2 * h * self.side_dim
             return n + self.vocab_size * self.side_dim * len(self.layer_specs)
         attn = h * (self.q_size + 2 * self.kv_size) + self.q_size * h
@@ -627,6 +650,53 @@ PRESETS.update({
     "tiny-generax": _generax("tiny-generax", 128, "paps",
                              dict(heads=4, kv=2, dim=32, vdim=16, rot=16, window=24, pool=4),
                              dict(heads=4, kv=2, dim=16, vdim=16, rank=8, conv=3), 192, vocab=1024),
+})
+
+
+def _ratizen(name: str, width: int, pattern: str, att: dict, lat: dict, expert_ff: int,
+             shared_ff: int, experts: int = 8, top: int = 2, streams: int = 4,
+             vocab: int = 32000) -> ModelConfig:
+    """A Ratizen-architecture preset: ``pattern`` is one letter per layer ("c": chunked
+    attention with a sink, "l": windowed latent attention); every layer has routed experts
+    and a shared one."""
+    mlp = FeedForwardSpec("moe", expert_ff, act="silu", gated=True, experts=experts, top=top,
+                          router="sigmoid_raw", weight_input=True, shared_ff=shared_ff,
+                          shared_gate=False)
+    rs = RotarySpec(lat["rot"], lat.get("base", 1e4), interleaved=True,
+                    yarn=(8.0, 4096.0, 32.0, 1.0))
+    specs = tuple(
+        MixerSpec("attention", att["heads"], att["dim"], att["vdim"], kv_heads=att["kv"],
+                  scale=att["dim"] ** -0.5, window=WindowSpec(att["chunk"], chunked=True),
+                  head_norm=True, sink=0.0, ff=expert_ff, mlp=mlp)
+        if c == "c" else
+        MixerSpec("latent_attention", lat["heads"], lat["dim"], lat["vdim"], kv_heads=1,
+                  scale=(lat["dim"] + lat["rot"]) ** -0.5, rot_dims=rs.dims, rot_base=rs.base,
+                  rotary=rs, window=WindowSpec(lat["window"]), kv_rank=lat["rank"],
+                  q_rank=lat["q_rank"], head_gate=True, ff=expert_ff, mlp=mlp)
+        for c in pattern)
+    return ModelConfig(name, "ratizen", len(specs), width, att["heads"], att["kv"], att["dim"],
+                       expert_ff, vocab, max_position=8192, rms_eps=1e-6, layer_specs=specs,
+                       embed_scale=width ** 0.5, residual_mult=0.5, streams=streams,
+                       bos_token_id=1, eos_token_id=2)
+
+
+# Ratizen presets beside the equal-width hybrid / Llama presets above: the same number of
+# layers, 16 / 32 heads of 128, experts whose active parameters per token (two of eight and the
+# shared one) are those of the Llama preset's feed-forward, the latent rows of the Konovik
+# presets (192 + 64).
+PRESETS.update({
+    "ratizen-w2048": _ratizen("ratizen-w2048", 2048, "ccl" * 4,
+                              dict(heads=16, kv=4, dim=128, vdim=128, chunk=1024),
+                              dict(heads=16, dim=128, rot=64, vdim=128, rank=192, q_rank=768,
+                                   window=1024), 1792, 1920),
+    "ratizen-w4096": _ratizen("ratizen-w4096", 4096, "clcl" * 2,
+                              dict(heads=32, kv=8, dim=128, vdim=128, chunk=2048),
+                              dict(heads=32, dim=128, rot=64, vdim=128, rank=192, q_rank=1536,
+                                   window=2048), 4608, 5120),
+    "tiny-ratizen": _ratizen("tiny-ratizen", 128, "ccl",
+                             dict(heads=4, kv=2, dim=32, vdim=16, chunk=24),
+                             dict(heads=4, dim=16, rot=8, vdim=16, rank=24, q_rank=48, window=20),
+                             64, 96, experts=4, streams=3, vocab=1024),
 })
 
 
@@ -976,6 +1046,73 @@ def generax_config(d: dict, name: str, shapes: Optional[dict] = None) -> ModelCo
         bos_token_id=int(d.get("bos_token_id", 0)), eos_token_id=int(d.get("eos_token_id", -1)))
 
 
+def _ratizen_ff(mlp: Optional[dict]) -> Optional[FeedForwardSpec]:
+    if not mlp:
+        return None
+    kind = mlp.get("kind", "moe")
+    if kind != "moe":
+        raise ValueError(f"unsupported feed-forward kind {kind!r}")
+    rt, sh = mlp["router"], mlp.get("shared")
+    E, top = int(rt["experts"]), int(rt["top"])
+    if not 1 <= top <= E:
+        raise ValueError(f"{top} of {E} experts")
+    return FeedForwardSpec("moe", int(mlp["expert"]["ff"]), act="silu", gated=True, experts=E,
+                           top=top, router="sigmoid_raw", weight_input=True,
+                           shared_ff=int(sh["ff"]) if sh else 0, shared_gate=False)
+
+
+def _ratizen_spec(entry: dict) -> MixerSpec:
+    """One entry of a Ratizen ``layers`` list.  Type "attention": unrotated grouped-query
+    attention inside chunks, q / k normed per head, a sink of score 0; type
+    "latent_attention": latent queries and keys, YaRN rotation, a sliding window, a gate per
+    head.  A mixer without ``mask`` is plain causal."""
+    kind, m = entry["type"], entry["mixer"]
+    mlp = _ratizen_ff(entry.get("mlp"))
+    ff, mask, H = mlp.ff if mlp else 0, m.get("mask"), int(m["heads"])
+    if kind == "attention":
+        sp = MixerSpec("attention", H, int(m["dim"]), int(m["vdim"]),
+                       kv_heads=int(m.get("kv_heads", H)), scale=float(m["scale"]),
+                       window=WindowSpec(int(mask["size"]), chunked=True) if mask else None,
+                       head_norm=True, sink=0.0, ff=ff, mlp=mlp)
+        if sp.heads % sp.kv_heads:
+            raise ValueError("heads must be a multiple of the key/value heads")
+        return sp
+    if kind != "latent_attention":
+        raise ValueError(f"unknown mixer type {kind!r}")
+    r, rs = int(m.get("rot_dim", 0)), None
+    if r:
+        rot = m["rot"]
+        if r % 2 or int(rot.get("dims", r)) != r:
+            raise ValueError("rot.dims must be the (even) rotated part of a head")
+        sc = rot.get("scaling")
+        rs = RotarySpec(r, float(rot["base"]), interleaved=True,
+                        yarn=(float(sc["factor"]), float(sc["original"]), float(sc["fast"]),
+                              float(sc["slow"])) if sc else None)
+    return MixerSpec("latent_attention", H, int(m["dim"]), int(m["vdim"]), kv_heads=1,
+                     scale=float(m["scale"]), rot_dims=r, rot_base=rs.base if rs else 10000.0,
+                     rotary=rs, window=WindowSpec(int(mask["size"])) if mask else None,
+                     kv_rank=int(m["kv_rank"]), q_rank=int(m["q_rank"]), head_gate=True, ff=ff,
+                     mlp=mlp)
+
+
+def ratizen_config(d: dict, name: str) -> ModelConfig:
+    """A Ratizen config.json (``architecture``, ``width``, ``vocab``, ``layers``, ``streams``,
+    ``norm``, ``embedding``, ``residual_mult``, ``logit_scale``) -> ModelConfig."""
+    specs = tuple(_ratizen_spec(e) for e in d["layers"])
+    a = next((sp for sp in specs if sp.kind == "attention"), specs[0])
+    streams = int(d["streams"])
+    if streams < 1:
+        raise ValueError("streams must be at least 1")
+    return ModelConfig(
+        name, "ratizen", len(specs), int(d["width"]), a.heads, a.kv_heads, a.dim,
+        max((sp.ff for sp in specs), default=0), int(d["vocab"]),
+        max_position=int(d.get("max_position", 8192)), rms_eps=float(d["norm"]["eps"]),
+        layer_specs=specs, embed_scale=float(d.get("embedding", {}).get("scale", 1.0)),
+        residual_mult=float(d.get("residual_mult", 1.0)), streams=streams,
+        logit_scale=float(d.get("logit_scale", 1.0)),
+        bos_token_id=int(d.get("bos_token_id", 0)), eos_token_id=int(d.get("eos_token_id", -1)))
+
+
 def _tensor_shapes(path: str) -> dict:
     """Tensor name -> shape from the headers of the safetensors files in ``path``."""
     import glob
@@ -992,6 +1129,8 @@ def _tensor_shapes(path: str) -> dict:
 
 def _from_hf_config(d: dict, name: str, path: Optional[str] = None) -> ModelConfig:
     """Map an HF config.json dict onto ModelConfig."""
+    if d.get("architecture") == "Ratizen":
+        return ratizen_config(d, name)
     if d.get("architecture") == "Generax":
         return generax_config(d, name, _tensor_shapes(path) if path else None)
     if d.get("architecture") == "Lorenex":

@@ -412,3 +412,70 @@ class SoftmaxAllRoutedExperts(nn.Module):
         if sp.identity:
             return ops.moe_finish(routed, dense, topk_w, topk_ids, x, idw)
         return ops.moe_finish(None, dense, topk_w, topk_ids, None, None)
+
+
+class InputScaledExperts(nn.Module):
+    """Mixture of gated experts whose input carries the routing weight: sigmoid scores
+    s = sigmoid(W_r h) in fp32, the ``top`` largest chosen, and the result
+    sum_e down_e(silu(s_e gate_e h) * (s_e up_e h)) over the chosen ones, the scores as they are;
+    an optional shared expert of the same form (weight 1) joins the sum.
+
+    One parameter ``w_in`` [(E 2 ff + 2 shared), hidden] holds every expert's gate rows, then its
+    up rows, the shared expert's last; ``w_down`` [hidden, E ff + shared] the down projections side
+    by side.  Two ways to run, both without host synchronisation:
+
+    * dense: ONE GEMM with all of ``w_in``, an activation kernel that multiplies by the token's
+      weight of each expert (0: not chosen), ONE GEMM with all of ``w_down``, which also sums
+      the experts.  Decode-size steps that touch most experts anyway read every weight once
+      this way; it takes any sizes and fp32.
+    * grouped: the MFMA GEMM over expert-sorted rows (16-bit activations, ff % 64 == 0,
+      hidden % 128 == 0), the shared expert as a dense feed-forward beside it.
+
+    Returns the addends [(rows, rows per token)] of the result, which the consumer sums."""
+
+    DENSE_MAX_T = 128          # tokens up to which a step's GEMMs are bound by the weights
+
+    def __init__(self, hidden: int, spec, dtype, device):
+        super().__init__()
+        assert spec.act == "silu" and spec.gated and spec.router == "sigmoid_raw"
+        assert spec.weight_input and not spec.shared_gate
+        self.spec = spec
+        E, I, Is = spec.experts, spec.ff, spec.shared_ff
+        self.in_proj = ReplicatedLinear(hidden, 2 * (E * I + Is), dtype=dtype, device=device)
+        self.down_proj = ReplicatedLinear(E * I + Is, hidden, dtype=dtype, device=device)
+        self.router = nn.Parameter(torch.zeros(E, hidden, dtype=dtype, device=device),
+                                   requires_grad=False)
+        self.native = (torch.device(device).type == "cuda" and dtype != torch.float32 and E <= 256 and
+                       ops.moe_supported(2 * I, hidden) and ops.moe_supported(hidden, I) and
+                       Is % 8 == 0)
+
+    def expert_in(self, e: int) -> torch.Tensor:
+        """Rows [gate | up] of expert e (e = experts: the shared one)."""
+        E, I, Is = self.spec.experts, self.spec.ff, self.spec.shared_ff
+        return self.in_proj.weight.data.narrow(0, e * 2 * I, 2 * (I if e < E else Is))
+
+    def expert_down(self, e: int) -> torch.Tensor:
+        E, I, Is = self.spec.experts, self.spec.ff, self.spec.shared_ff
+        return self.down_proj.weight.data.narrow(1, e * I, I if e < E else Is)
+
+    def route(self, x: torch.Tensor) -> tuple:
+        scores = ops.gate_proj(x, self.router, None, ops.GATE_SIGMOID)      # fp32 [T, E]
+        return ops.moe_route_sigmoid(scores, None, self.spec.top, 1.0, False)
+
+    def dense_step(self, T: int) -> bool:
+        return not self.native or (T <= self.DENSE_MAX_T and T * self.spec.top >= self.spec.experts)
+
+    def forward(self, x: torch.Tensor) -> list:
+        sp = self.spec
+        E, I, Is, T = sp.experts, sp.ff, sp.shared_ff, x.shape[0]
+        topk_w, topk_ids = self.route(x)
+        if self.dense_step(T):
+            a = ops.expert_silu_all(self.in_proj(x), topk_w, topk_ids, E, I, Is)
+            return [(self.down_proj(a), 1)]
+        w_in = self.in_proj.weight[: E * 2 * I].view(E, 2 * I, x.shape[1])
+        w_down = self.down_proj.weight[:, : E * I].view(x.shape[1], E, I).transpose(0, 1)
+        adds = [(ops.grouped_experts_scaled(x, w_in, w_down, topk_w, topk_ids), sp.top)]
+        if Is:
+            a = ops.silu_mul(F.linear(x, self.expert_in(E)))
+            adds.append((F.linear(a, self.expert_down(E)), 1))
+        return adds

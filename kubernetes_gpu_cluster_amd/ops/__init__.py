@@ -723,7 +723,8 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
                      out_scale: float = 1.0, out: Optional[torch.Tensor] = None,
                      elem_gate: Optional[torch.Tensor] = None, pool: int = 0,
                      block_size: int = 0, v_table: Optional[torch.Tensor] = None,
-                     interleaved: bool = False) -> torch.Tensor:
+                     interleaved: bool = False, chunked: bool = False,
+                     sink: Optional[float] = None) -> torch.Tensor:
     """Prefill chunks and decode rows of one step alike: row t sees the cached keys
     j <= p with p - j < window or j < keep_first (p = positions[t]; window <= 0: plain
     causal).  Decode padding rows (context length 0) give zeros.  ``softcap`` > 0: the
@@ -736,7 +737,9 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
     ceil(block_size / pool) pooled rows; the call first writes the rows of the blocks that
     the step's tokens complete.  ``v_table`` (fp32 [max_pos, dv], cos | sin): the cached
     values were turned by their positions, each head's output is turned back by the row's
-    (pairs (m, m + dv/2), or (2m, 2m + 1) when ``interleaved``)."""
+    (pairs (m, m + dv/2), or (2m, 2m + 1) when ``interleaved``).  ``chunked``: the row sees the
+    keys j <= p of its own chunk of ``window`` positions (j // window == p // window) instead.
+    ``sink``: a score without a value that joins every row's softmax."""
     T, H, _ = q.shape
     dv = v_cache.shape[3]
     if not _gpu(q):
@@ -749,7 +752,7 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
             ref.pool_kv_rows(k_cache, v_cache, pos, meta.slot_mapping, rt, pool, block_size)
         r = ref.window_attention(q, k_cache, v_cache, pos, rt, scale, window, keep_first, gate,
                                  softcap, out_scale, elem_gate, pool, block_size, v_table,
-                                 interleaved)
+                                 interleaved, chunked, sink)
         if out is not None:
             out.copy_(r)
             return out
@@ -770,7 +773,8 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
                           scale, window, keep_first, gate, window_attention_fast(),
                           float(softcap), float(out_scale), elem_gate, int(pool),
                           int(block_size), v_table, interleaved,
-                          meta.slot_mapping if pool > 0 else None)
+                          meta.slot_mapping if pool > 0 else None, chunked,
+                          float("-inf") if sink is None else float(sink))
     return out
 
 
@@ -910,14 +914,16 @@ def relu_sq(z: torch.Tensor) -> torch.Tensor:
     return out
 
 
-def moe_route_sigmoid(scores: torch.Tensor, correction: torch.Tensor, k: int, scale: float):
-    """(weights fp32 [T, k], expert ids int32 [T, k]) from sigmoid scores fp32 [T, >= E]."""
+def moe_route_sigmoid(scores: torch.Tensor, correction: Optional[torch.Tensor], k: int,
+                      scale: float, renormalize: bool = True):
+    """(weights fp32 [T, k], expert ids int32 [T, k]) from sigmoid scores fp32 [T, >= E]; see
+    ``ref.moe_route_sigmoid``."""
     if not _gpu(scores):
-        return ref.moe_route_sigmoid(scores, correction, k, scale)
+        return ref.moe_route_sigmoid(scores, correction, k, scale, renormalize)
     T = scores.shape[0]
     w = torch.empty(T, k, dtype=torch.float32, device=scores.device)
     ids = torch.empty(T, k, dtype=torch.int32, device=scores.device)
-    _k().moe_route_sigmoid(w, ids, scores, correction, float(scale))
+    _k().moe_route_sigmoid(w, ids, scores, correction, float(scale), renormalize)
     return w, ids
 
 
@@ -1128,17 +1134,19 @@ def selective_scan(x: torch.Tensor, dt: torch.Tensor, bc: torch.Tensor, At: torc
 def norm_kv_store(qkv: torch.Tensor, positions: torch.Tensor, k_cache: torch.Tensor,
                   v_cache: torch.Tensor, slot_mapping: torch.Tensor, H: int, G: int, dk: int,
                   dv: int, eps: float, qk_unit: bool, v_unit: bool, q_temp,
-                  out_dtype: torch.dtype) -> torch.Tensor:
-    """q [T, H, dk] in ``out_dtype`` from qkv fp32 [T, H dk + G dk + G dv], k and v into the
-    paged cache: head vectors divided by their root mean square (``qk_unit``, ``v_unit``),
+                  out_dtype: torch.dtype, q_w: Optional[torch.Tensor] = None,
+                  k_w: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """q [T, H, dk] in ``out_dtype`` from qkv [T, H dk + G dk + G dv] (fp32, or ``out_dtype``; a
+    column slice), k and v into the paged cache: head vectors divided by their root mean square
+    (``qk_unit``, ``v_unit``), q and k times ``q_w`` / ``k_w`` (fp32 [dk], all heads alike),
     q times 1 + coef * ln(floor((p + 1) / every) + 1) (``q_temp`` = (coef, every) or None)."""
     if not _gpu(qkv):
         return ref.norm_kv_store(qkv, positions, k_cache, v_cache, slot_mapping, H, G, dk, dv,
-                                 eps, qk_unit, v_unit, q_temp, out_dtype)
+                                 eps, qk_unit, v_unit, q_temp, out_dtype, q_w, k_w)
     q = torch.empty(qkv.shape[0], H, dk, dtype=out_dtype, device=qkv.device)
     coef, every = q_temp if q_temp is not None else (0.0, 1)
     _k().norm_kv_store(qkv, positions, q, k_cache, v_cache, slot_mapping, H, G, dk, dv,
-                       float(eps), qk_unit, v_unit, float(coef), int(every))
+                       float(eps), qk_unit, v_unit, float(coef), int(every), q_w, k_w)
     return q
 
 
@@ -1246,3 +1254,99 @@ def logit_softcap(logits: torch.Tensor, cap: float) -> torch.Tensor:
     out = torch.empty(logits.shape, dtype=torch.float32, device=logits.device)
     _k().logit_softcap(out, logits, float(cap))
     return out
+
+
+# ------------------------------------------------------------------ Ratizen-style decoders
+# Hyper-connections (several residual streams mixed around every sublayer), latent queries beside
+# the latent keys of the Konovik-style decoders, one small matrix per head, experts whose input
+# carries the routing weight.  Per-head norms: ``norm_kv_store`` with weights; chunks and sinks:
+# ``window_attention``.
+def hyper_norm(src: torch.Tensor, dst: Optional[torch.Tensor], adds: list,
+               mix: Optional[torch.Tensor], out_w: Optional[torch.Tensor], in_w: torch.Tensor,
+               w: Optional[torch.Tensor], eps: float, out_dtype: Optional[torch.dtype]
+               ) -> Optional[torch.Tensor]:
+    """One pass over the residual streams src fp32 [T, S, W] (or [T, 1, W] expanded to S): with
+    ``mix`` the sublayer result y = sum of up to two ``adds`` joins them, x_t = sum_s mix[s, t]
+    src_s + out_w[t] y, written to ``dst`` (may be src) when given; returns RMSNorm(u) * w (w
+    None: u) in out_dtype, u = sum_s in_w[s] x_s.  See ``ref.hyper_norm``."""
+    if not _gpu(src):
+        return ref.hyper_norm(src, dst, adds, mix, out_w, in_w, w, eps, out_dtype)
+    T, S, W = src.shape
+    out = torch.empty(T, W, dtype=out_dtype, device=src.device) if out_dtype is not None else None
+    a = list(adds) + [(None, 1)] * (2 - len(adds))
+    _k().hyper_norm(out, src, dst, a[0][0], a[0][1], a[1][0], a[1][1], mix, out_w, in_w, w,
+                    float(eps))
+    return out
+
+
+def latent_down_store(proj: torch.Tensor, positions: torch.Tensor, table: Optional[torch.Tensor],
+                      q_w: torch.Tensor, kv_w: torch.Tensor, eps: float, cache: torch.Tensor,
+                      slot_mapping: torch.Tensor, r: int, gates: int) -> tuple:
+    """From the merged down projection [T, q_rank | rank | r | gates ...]: the cache row, and
+    (normed query latent [T, q_rank], sigmoid gates fp32 [T, gates]); see
+    ``ref.latent_down_store``."""
+    if not _gpu(proj):
+        return ref.latent_down_store(proj, positions, table, q_w, kv_w, eps, cache, slot_mapping,
+                                     r, gates)
+    T = proj.shape[0]
+    cq = torch.empty(T, q_w.numel(), dtype=proj.dtype, device=proj.device)
+    g = torch.empty(T, gates, dtype=torch.float32, device=proj.device)
+    _k().latent_down_store(cq, g, proj, positions, table, q_w, kv_w, float(eps), cache,
+                           slot_mapping, r)
+    return cq, g
+
+
+def head_gemm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor,
+              rot: Optional[torch.Tensor] = None, positions: Optional[torch.Tensor] = None,
+              table: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """out[t, h, :N] = w[h] x[t, h] (x [T, H, K], w [H, N, K], out [T, H, N + r]: token and head
+    strides are free), and in the same launch out[t, h, N:] = ``rot`` [T, H, r] rotated by the
+    row's position; see ``ref.head_gemm``."""
+    if not _gpu(x):
+        return ref.head_gemm(x, w, out, rot, positions, table)
+    _k().head_gemm(out, x, w, rot, positions, table)
+    return out
+
+
+def expert_silu_all(x: torch.Tensor, topk_w: torch.Tensor, topk_ids: torch.Tensor, experts: int,
+                    ff: int, shared_ff: int) -> torch.Tensor:
+    """[T, experts * ff + shared_ff]: silu(w gate) * (w up) of every expert for every token, w its
+    routing weight there (0: not chosen; 1: the shared expert); see ``ref.expert_silu_all``."""
+    if not _gpu(x):
+        return ref.expert_silu_all(x, topk_w, topk_ids, experts, ff, shared_ff, x.dtype)
+    out = torch.empty(x.shape[0], experts * ff + shared_ff, dtype=x.dtype, device=x.device)
+    _k().expert_silu_all(out, x, topk_w, topk_ids, experts, ff, shared_ff)
+    return out
+
+
+def grouped_experts_scaled(x: torch.Tensor, w_in: torch.Tensor, w_down: torch.Tensor,
+                           topk_w: torch.Tensor, topk_ids: torch.Tensor) -> torch.Tensor:
+    """Down projections of the chosen experts on inputs scaled by their routing weights, per
+    (token, choice) pair: down_e(silu(w gate_e x) * (w up_e x)) as [T k, H] in x's dtype, or its
+    fp32 split-K slices [S, T k, H]; the consumer sums a token's pairs.  w_in [E, 2 I, H] (gate
+    rows, then up rows); w_down [E, H, I], any expert and row strides.  The grouped MFMA GEMM of
+    ``grouped_experts`` with the weights in the activation kernel; no host synchronisation."""
+    k = _k()
+    T, H = x.shape
+    E, I2 = w_in.shape[0], w_in.shape[1]
+    topk = topk_ids.shape[1]
+    npairs = T * topk
+    bm = 64 if npairs <= 40 * E else 128
+    rows = (npairs + E * (bm - 1) + bm - 1) // bm * bm
+    dev = x.device
+    sorted_ids = torch.empty(rows, dtype=torch.int32, device=dev)
+    block_expert = torch.empty(rows // bm, dtype=torch.int32, device=dev)
+    meta = torch.empty(1, dtype=torch.int32, device=dev)
+    k.moe_align(sorted_ids, block_expert, meta, topk_ids.contiguous(), 0, E, bm)
+    inter = torch.empty(rows, I2, dtype=x.dtype, device=dev)
+    k.moe_gemm(inter, x.contiguous(), w_in, sorted_ids, block_expert, meta, npairs, topk, bm,
+               True, False)
+    a = torch.empty(rows, I2 // 2, dtype=x.dtype, device=dev)
+    k.expert_silu_rows(a, inter, topk_w, sorted_ids)
+    S = moe_splitk(npairs, E, H, I2 // 2, bm)
+    if S > 1:
+        y = torch.empty(S, npairs, H, dtype=torch.float32, device=dev)
+    else:
+        y = torch.empty(npairs, H, dtype=x.dtype, device=dev)
+    k.moe_gemm(y, a, w_down, sorted_ids, block_expert, meta, npairs, topk, bm, False, True, S)
+    return y

@@ -458,7 +458,8 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
                      out_scale: float = 1.0,
                      elem_gate: Optional[torch.Tensor] = None, pool: int = 0,
                      block_size: int = 0, v_table: Optional[torch.Tensor] = None,
-                     interleaved: bool = False) -> torch.Tensor:
+                     interleaved: bool = False, chunked: bool = False,
+                     sink: Optional[float] = None) -> torch.Tensor:
     """q [T, H, dk] (rotated; the step's k / v already stored) -> [T, H*dv].  Row t at
     position p = positions[t] attends the cached keys j <= p with p - j < window or
     j < keep_first (window <= 0: all of them) of the sequence whose block table is
@@ -469,7 +470,9 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
     row (``pool_kv_rows``) of every block of ``pool`` tokens that lies wholly before its
     window; pages then hold ``block_size`` token rows followed by the pooled rows.
     ``v_table`` [max_pos, dv] (cos | sin): each head's output is turned back by the row's
-    position (the cached values were turned by theirs)."""
+    position (the cached values were turned by theirs).  ``chunked``: the visible keys are
+    those j <= p with j // window == p // window instead.  ``sink``: a score without a value
+    that joins every row's softmax."""
     T, H, dk = q.shape
     G, bs, dv = k_cache.shape[1], block_size or k_cache.shape[2], v_cache.shape[3]
     out = torch.zeros(T, H, dv, dtype=torch.float32)
@@ -479,7 +482,8 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
             continue
         j = torch.arange(p + 1)
         if window > 0:
-            j = j[(p - j < window) | (j < keep_first)]
+            lo = p - p % window if chunked else p - window + 1
+            j = j[(j >= lo) | (j < keep_first)]
         page, row = j // bs, j % bs
         if pool > 0:
             b = torch.arange(max(0, (p - window + 1) // pool))
@@ -492,7 +496,9 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
         s = torch.einsum("ghd,ngd->ghn", qt, k) * scale
         if softcap > 0:
             s = softcap * torch.tanh(s / softcap)
-        pr = torch.softmax(s, dim=-1)
+        if sink is not None:
+            s = torch.cat([s, torch.full_like(s[..., :1], sink)], -1)
+        pr = torch.softmax(s, dim=-1)[..., : k.shape[0]]
         out[t] = torch.einsum("ghn,ngv->ghv", pr, v).reshape(H, dv)
     if v_table is not None:
         cs = v_table[positions.long().clamp(0, v_table.shape[0] - 1)]
@@ -558,12 +564,12 @@ def head_norm_gate(o: torch.Tensor, g: torch.Tensor, w: torch.Tensor, H: int, ep
 # YaRN / interleaved rotary, sigmoid routing with a choice correction, squared-ReLU
 # experts, per-token side input)
 def rope_table_yarn(rot_dims: int, max_pos: int, base: float, yarn=None) -> torch.Tensor:
-    """[max_pos, rot_dims] fp32: cos | sin of p * f_i, i < rot_dims/2.  ``yarn`` =
-    (factor, original, fast, slow): f_i = base^(-2i/dims) is slowed by ``factor`` for the
-    pairs past the ramp between the dimensions that make ``fast`` and ``slow`` turns over
+    """[max_pos, rot_dims] fp32: cos | sin of p * f_i, i < rot_dims/2, evaluated in fp64.
+    ``yarn`` = (factor, original, fast, slow): f_i = base^(-2i/dims) is slowed by ``factor`` for
+    the pairs past the ramp between the dimensions that make ``fast`` and ``slow`` turns over
     ``original`` positions, and cos / sin are scaled by 0.1 ln(factor) + 1."""
-    i = torch.arange(rot_dims // 2, dtype=torch.float32)
-    f = torch.tensor(base, dtype=torch.float32) ** (-2.0 * i / rot_dims)
+    i = torch.arange(rot_dims // 2, dtype=torch.float64)
+    f = torch.tensor(base, dtype=torch.float64) ** (-2.0 * i / rot_dims)
     mag = 1.0
     if yarn is not None:
         factor, orig, fast, slow = yarn
@@ -575,8 +581,8 @@ def rope_table_yarn(rot_dims: int, max_pos: int, base: float, yarn=None) -> torc
         ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
         f = f / factor * ramp + f * (1 - ramp)
         mag = 0.1 * math.log(factor) + 1.0
-    a = torch.arange(max_pos, dtype=torch.float32)[:, None] * f[None]
-    return torch.cat([a.cos() * mag, a.sin() * mag], dim=-1)
+    a = torch.arange(max_pos, dtype=torch.float64)[:, None] * f[None]
+    return torch.cat([a.cos() * mag, a.sin() * mag], dim=-1).float()
 
 
 def residual_norm(x: torch.Tensor, add: Optional[torch.Tensor], mult: float,
@@ -701,15 +707,19 @@ def relu_sq(z: torch.Tensor) -> torch.Tensor:
     return torch.relu(z.float()).pow(2).to(z.dtype)
 
 
-def moe_route_sigmoid(scores: torch.Tensor, correction: torch.Tensor, k: int, scale: float):
-    """scores fp32 [T, >= E]: sigmoid router scores in the first E = len(correction)
-    columns.  The k experts with the largest score + correction (lowest index first among
-    equals); weights = their scores / (sum + 1e-20) * scale.  -> (fp32 [T, k], int32 [T, k])."""
-    E = correction.numel()
-    s = scores[:, :E].float()
-    ids = torch.topk(s + correction.float(), k, dim=-1).indices
+def moe_route_sigmoid(scores: torch.Tensor, correction: Optional[torch.Tensor], k: int,
+                      scale: float, renormalize: bool = True):
+    """scores fp32 [T, >= E]: sigmoid router scores in the first E = len(correction) columns
+    (all without a correction).  The k experts with the largest score + correction (lowest
+    index first among equals); weights = their scores / (sum + 1e-20) * scale, or just their
+    scores * scale.  -> (fp32 [T, k], int32 [T, k])."""
+    s = scores.float() if correction is None else scores[:, : correction.numel()].float()
+    pick = s if correction is None else s + correction.float()
+    ids = torch.sort(pick, dim=-1, descending=True, stable=True).indices[:, :k]
     w = torch.gather(s, 1, ids)
-    return w / (w.sum(-1, keepdim=True) + 1e-20) * scale, ids.to(torch.int32)
+    if renormalize:
+        w = w / (w.sum(-1, keepdim=True) + 1e-20)
+    return w * scale, ids.to(torch.int32)
 
 
 def moe_finish(routed: Optional[torch.Tensor], dense: Optional[torch.Tensor],
@@ -913,10 +923,12 @@ def selective_scan(x: torch.Tensor, dt: torch.Tensor, bc: torch.Tensor, At: torc
 def norm_kv_store(qkv: torch.Tensor, positions: torch.Tensor, k_cache: torch.Tensor,
                   v_cache: torch.Tensor, slot_mapping: torch.Tensor, H: int, G: int, dk: int,
                   dv: int, eps: float, qk_unit: bool, v_unit: bool, q_temp,
-                  out_dtype: torch.dtype) -> torch.Tensor:
-    """qkv fp32 [T, H dk + G dk + G dv] -> q [T, H, dk] in out_dtype; k and v go to the
+                  out_dtype: torch.dtype, q_w: Optional[torch.Tensor] = None,
+                  k_w: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """qkv [T, H dk + G dk + G dv] -> q [T, H, dk] in out_dtype; k and v go to the
     plain-layout paged cache at ``slot_mapping`` (< 0: no write).  ``qk_unit`` / ``v_unit``:
-    each head's vector is divided by sqrt(mean(x^2) + eps).  ``q_temp`` = (coef, every): q at
+    each head's vector is divided by sqrt(mean(x^2) + eps); q and k are then multiplied by
+    ``q_w`` / ``k_w`` [dk] where given.  ``q_temp`` = (coef, every): q at
     position p times 1 + coef * ln(floor((p + 1) / every) + 1).  fp32 math."""
     T = qkv.shape[0]
     q = qkv[:, : H * dk].float().view(T, H, dk)
@@ -927,6 +939,10 @@ def norm_kv_store(qkv: torch.Tensor, positions: torch.Tensor, k_cache: torch.Ten
         return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
     if qk_unit:
         q, k = unit(q), unit(k)
+    if q_w is not None:
+        q = q * q_w.float()
+    if k_w is not None:
+        k = k * k_w.float()
     if v_unit:
         v = unit(v)
     if q_temp is not None:
@@ -1119,3 +1135,87 @@ def channel_delta_scan(qkv: torch.Tensor, b: torch.Tensor, decay: torch.Tensor,
 def logit_softcap(logits: torch.Tensor, cap: float) -> torch.Tensor:
     """fp32 cap * tanh(logits / cap)."""
     return cap * torch.tanh(logits.float() / cap)
+
+
+# ------------------------------------------------------------------ Ratizen-style decoders
+def hyper_norm(src: torch.Tensor, dst: Optional[torch.Tensor], adds: list,
+               mix: Optional[torch.Tensor], out_w: Optional[torch.Tensor], in_w: torch.Tensor,
+               w: Optional[torch.Tensor], eps: float, out_dtype: Optional[torch.dtype]
+               ) -> Optional[torch.Tensor]:
+    """Hyper-connections over S residual streams src fp32 [T, S, W] (S rows may be one row
+    expanded).  With ``mix`` fp32 [from, to] and ``out_w`` fp32 [S]:
+        x_t = sum_s mix[s, t] src_s + out_w[t] y,   y the sum of ``adds``
+    (else x = src), written to ``dst`` [T, S, W] when given.  Returns u / rms(u) * w (w None: u)
+    in out_dtype (None: nothing), u = sum_s in_w[s] x_s.  An addend is (a, k): a [T k, W] holds k
+    rows per token that are summed; a fp32 [n, T k, W] holds n partial sums of them."""
+    T, S, W = src.shape
+    x = src.float()
+    if mix is not None:
+        y = torch.zeros(T, W, dtype=torch.float32)
+        for a, k in adds:
+            a = a.float().sum(0) if a.dim() == 3 else a.float()
+            y = y + a.reshape(T, k, W).sum(1)
+        x = torch.einsum("st,nsw->ntw", mix.float(), x) + out_w.float()[:, None] * y[:, None, :]
+        if dst is not None:
+            dst.copy_(x)
+    if out_dtype is None:
+        return None
+    u = torch.einsum("s,nsw->nw", in_w.float(), x)
+    if w is not None:
+        u = u * torch.rsqrt(u.pow(2).mean(-1, keepdim=True) + eps) * w.float()
+    return u.to(out_dtype)
+
+
+def latent_down_store(proj: torch.Tensor, positions: torch.Tensor, table: Optional[torch.Tensor],
+                      q_w: torch.Tensor, kv_w: torch.Tensor, eps: float, cache: torch.Tensor,
+                      slot_mapping: torch.Tensor, r: int, gates: int) -> tuple:
+    """proj [T, q_rank + rank + r + gates ...]: query latent | key/value latent | rotary key part
+    | gate pre-activations (q_rank, rank: the weights' lengths).  Writes the cache row
+    [normed key/value latent * kv_w | rotated key part] at slot_mapping (< 0: none) into cache
+    [nb, 1, bs, rank + r]; returns (normed query latent * q_w [T, q_rank] in proj's dtype,
+    sigmoid(gates) fp32 [T, gates]).  Pairs are (2i, 2i+1)."""
+    qr, rank = q_w.numel(), kv_w.numel()
+
+    def norm(x, w):
+        return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w.float()
+    p = proj.float()
+    cq = norm(p[:, :qr], q_w)
+    c, kr = norm(p[:, qr: qr + rank], kv_w), p[:, qr + rank: qr + rank + r]
+    if r:
+        kr = _rot_pairs(kr, table[positions.long()])
+    bs = cache.shape[2]
+    ok = slot_mapping >= 0
+    sl = slot_mapping[ok].long()
+    cache[sl // bs, 0, sl % bs] = torch.cat([c, kr], -1)[ok].to(cache.dtype)
+    g = torch.sigmoid(p[:, qr + rank + r: qr + rank + r + gates])
+    return cq.to(proj.dtype), g
+
+
+def head_gemm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor,
+              rot: Optional[torch.Tensor] = None, positions: Optional[torch.Tensor] = None,
+              table: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """One matrix per head: out[t, h, n] = sum_k x[t, h, k] w[h, n, k] for n < N; x [T, H, K],
+    w [H, N, K], out [T, H, N + r] (any token and head strides).  ``rot`` [T, H, r] fills the
+    columns behind N, rotated by the row's position (pairs (2i, 2i+1), table cos | sin)."""
+    N = w.shape[1]
+    out[..., :N] = torch.einsum("thk,hnk->thn", x.float(), w.float()).to(out.dtype)
+    if rot is not None and rot.shape[-1]:
+        out[..., N:] = _rot_pairs(rot.float(), table[positions.long()][:, None, :]).to(out.dtype)
+    return out
+
+
+def expert_silu_all(x: torch.Tensor, topk_w: torch.Tensor, topk_ids: torch.Tensor, experts: int,
+                    ff: int, shared_ff: int, out_dtype: torch.dtype) -> torch.Tensor:
+    """Activations of every expert for every token, zero where an expert was not chosen: x [T,
+    experts * 2 ff + 2 shared_ff] = per expert gate | up columns, then the shared expert's;
+    -> [T, experts * ff + shared_ff] with silu(w gate) * (w up), w the token's weight of the
+    expert (its input is scaled; 1 for the shared one)."""
+    T = x.shape[0]
+    w = torch.zeros(T, experts, dtype=torch.float32)
+    w.scatter_(1, topk_ids.long(), topk_w.float())
+    g = x[:, : experts * 2 * ff].float().view(T, experts, 2 * ff) * w[:, :, None]
+    parts = [(torch.nn.functional.silu(g[..., :ff]) * g[..., ff:]).reshape(T, experts * ff)]
+    if shared_ff:
+        s = x[:, experts * 2 * ff:].float()
+        parts.append(torch.nn.functional.silu(s[:, :shared_ff]) * s[:, shared_ff: 2 * shared_ff])
+    return torch.cat(parts, 1).to(out_dtype)
