@@ -487,7 +487,10 @@ void moe_gemm(Tensor C, Tensor A, Tensor W, Tensor sorted_ids, Tensor block_expe
   check_gpu(A, "A");
   c10::hip::HIPGuardMasqueradingAsCUDA g(A.device());
   TORCH_CHECK(bm == 64 || bm == 128, "row block 64 or 128");
-  TORCH_CHECK(W.dim() == 3 && W.is_contiguous(), "W [E, N, K] contiguous");
+  TORCH_CHECK(W.dim() == 3 && W.stride(2) == 1 && W.stride(0) % 8 == 0 && W.stride(1) % 8 == 0 &&
+              W.stride(0) >= 0 && W.stride(1) >= W.size(2) &&
+              reinterpret_cast<uintptr_t>(W.data_ptr()) % 16 == 0,
+              "W [E, N, K]: 16-byte rows at any expert and row strides");
   TORCH_CHECK(splitk >= 1 && splitk <= 16, "1 <= splitk <= 16");
   TORCH_CHECK(splitk == 1 || (scatter && !gather), "split-K only for the scattering second GEMM");
   TORCH_CHECK(A.scalar_type() == W.scalar_type() &&
@@ -520,7 +523,7 @@ void moe_gemm(Tensor C, Tensor A, Tensor W, Tensor sorted_ids, Tensor block_expe
                        sorted_ids.data_ptr<int>(), block_expert.data_ptr<int>(), meta.data_ptr<int>(),
                        (int)npairs, (int)topk, (int)N, (int)K, A.stride(0), C2.stride(0),
                        (int)(rows / bm), gather, scatter, (int)splitk,
-                       splitk > 1 ? C.stride(0) : 0, stream());
+                       splitk > 1 ? C.stride(0) : 0, W.stride(0), W.stride(1), stream());
 }
 
 // K14m: the grouped MoE projections on the K9m LDS-DMA pipeline over per-expert packed
@@ -1400,7 +1403,7 @@ void window_attention(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
                       std::optional<Tensor> gate, bool fast, double softcap, double out_scale,
                       std::optional<Tensor> elem_gate, int64_t pool, int64_t block_size,
                       std::optional<Tensor> v_table, bool interleaved,
-                      std::optional<Tensor> slots) {
+                      std::optional<Tensor> slots, bool chunked, double sink) {
   check_gpu(q, "q");
   c10::hip::HIPGuardMasqueradingAsCUDA g(q.device());
   TORCH_CHECK(q.dim() == 3 && q.is_contiguous() && act_dtype(q), "kgc.window_attention: q [T, H, dk]");
@@ -1465,7 +1468,10 @@ void window_attention(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
     vrows = v_table->size(0);
   }
   const kgc::WindowExtra ex{T > 1 ? out.stride(0) : H * dv, (float)softcap, (float)out_scale, egp,
-                            egs, (int)pool, prow, vtp, (int)vrows, interleaved};
+                            egs, (int)pool, prow, vtp, (int)vrows, interleaved, chunked,
+                            (float)sink};
+  TORCH_CHECK(!chunked || (window > 0 && keep_first == 0 && pool == 0),
+              "kgc.window_attention: chunks need a size, no kept first tokens, no pooled blocks");
   // the matrix-core kernel stores 8-byte pieces of a row
   const bool out_vec = reinterpret_cast<uintptr_t>(out.data_ptr()) % 8 == 0 &&
                        ex.ors * out.element_size() % 8 == 0;
@@ -1823,14 +1829,16 @@ void selective_scan(Tensor out, Tensor x, Tensor dt, Tensor bc, Tensor At, Tenso
 
 void norm_kv_store(Tensor qkv, Tensor positions, Tensor q_out, Tensor k_cache, Tensor v_cache,
                    Tensor slots, int64_t H, int64_t G, int64_t dk, int64_t dv, double eps,
-                   bool qk_unit, bool v_unit, double coef, int64_t every) {
+                   bool qk_unit, bool v_unit, double coef, int64_t every,
+                   std::optional<Tensor> q_w, std::optional<Tensor> k_w) {
   check_gpu(qkv, "qkv");
   c10::hip::HIPGuardMasqueradingAsCUDA g(qkv.device());
-  // rows may be a column slice of a wider fp32 matrix: the kernel walks them by their stride
-  TORCH_CHECK(qkv.scalar_type() == at::kFloat && qkv.dim() == 2 && qkv.stride(1) == 1 &&
+  // rows may be a column slice of a wider matrix: the kernel walks them by their stride
+  TORCH_CHECK((qkv.scalar_type() == at::kFloat || qkv.scalar_type() == q_out.scalar_type()) &&
+              qkv.dim() == 2 && qkv.stride(1) == 1 &&
               qkv.size(1) >= (H + G) * dk + G * dv &&
               H >= 1 && G >= 1 && dk >= 1 && dv >= 1 && every >= 1,
-              "kgc.norm_kv_store: qkv fp32 [T, H dk + G dk + G dv]");
+              "kgc.norm_kv_store: qkv [T, H dk + G dk + G dv], fp32 or of q's dtype");
   const int64_t T = qkv.size(0);
   TORCH_CHECK(q_out.is_cuda() && q_out.device() == qkv.device() && act_dtype(q_out) &&
               q_out.is_contiguous() && q_out.numel() == T * H * dk, "kgc.norm_kv_store: q_out");
@@ -1839,11 +1847,12 @@ void norm_kv_store(Tensor qkv, Tensor positions, Tensor q_out, Tensor k_cache, T
               positions.is_contiguous() && slots.scalar_type() == at::kLong &&
               slots.numel() == T && slots.is_contiguous() && positions.is_cuda() && slots.is_cuda(),
               "kgc.norm_kv_store: positions / slots int64 [T]");
-  kgc::launch_norm_kv_store(dt_code(q_out), qkv.data_ptr<float>(), qkv.stride(0),
+  kgc::launch_norm_kv_store(dt_code(qkv), dt_code(q_out), qkv.data_ptr(), qkv.stride(0),
                             positions.data_ptr<int64_t>(), q_out.data_ptr(), k_cache.data_ptr(),
                             v_cache.data_ptr(), slots.data_ptr<int64_t>(), (int)T, (int)H, (int)G,
                             (int)dk, (int)dv, (int)k_cache.size(2), (int)k_cache.size(0),
-                            (float)eps, qk_unit, v_unit, (float)coef, (int)every, stream());
+                            (float)eps, qk_unit, v_unit, (float)coef, (int)every,
+                            f32_opt(q_w, dk, "q_w"), f32_opt(k_w, dk, "k_w"), stream());
 }
 
 void polynorm(Tensor out, Tensor z, Tensor coef, double eps) {
@@ -2135,13 +2144,13 @@ bool side_input_rows(std::optional<Tensor> out, Tensor x, std::optional<Tensor> 
   return true;
 }
 
-void moe_route_sigmoid(Tensor w, Tensor ids, Tensor scores, Tensor correction, double scale) {
+void moe_route_sigmoid(Tensor w, Tensor ids, Tensor scores, std::optional<Tensor> correction,
+                       double scale, bool renorm) {
   check_f32(w, "w");
-  check_f32(correction, "correction");
   c10::hip::HIPGuardMasqueradingAsCUDA g(w.device());
   TORCH_CHECK(scores.is_cuda() && scores.scalar_type() == at::kFloat && scores.dim() == 2 &&
               scores.stride(1) == 1 && scores.device() == w.device(), "kgc.moe_route_sigmoid: scores fp32 [T, >= E]");
-  const int64_t T = scores.size(0), E = correction.numel();
+  const int64_t T = scores.size(0), E = correction ? correction->numel() : scores.size(1);
   TORCH_CHECK(w.dim() == 2 && w.size(0) == T, "kgc.moe_route_sigmoid: w [T, k]");
   const int64_t k = w.size(1);
   TORCH_CHECK(E >= 1 && E <= scores.size(1) && E <= kgc::moe_route_sigmoid_max_experts() &&
@@ -2149,8 +2158,8 @@ void moe_route_sigmoid(Tensor w, Tensor ids, Tensor scores, Tensor correction, d
   TORCH_CHECK(ids.is_cuda() && ids.scalar_type() == at::kInt && ids.is_contiguous() &&
               ids.numel() == T * k && ids.device() == w.device(), "kgc.moe_route_sigmoid: ids int32 [T, k]");
   kgc::launch_moe_route_sigmoid(w.data_ptr<float>(), ids.data_ptr<int>(), scores.data_ptr<float>(),
-                                scores.stride(0), correction.data_ptr<float>(), (int)T, (int)E,
-                                (int)k, (float)scale, stream());
+                                scores.stride(0), f32_opt(correction, E, "correction"), (int)T,
+                                (int)E, (int)k, (float)scale, renorm, stream());
 }
 
 void moe_finish(Tensor out, std::optional<Tensor> routed, std::optional<Tensor> dense,
@@ -2303,9 +2312,214 @@ void logit_softcap(Tensor out, Tensor x, double cap) {
                             (int)x.size(1), (float)cap, stream());
 }
 
+// ---- Ratizen-style decoders: hyper-connections, latent queries, input-scaled experts ----------
+void hyper_norm(std::optional<Tensor> out, Tensor src, std::optional<Tensor> dst,
+                std::optional<Tensor> a0, int64_t k0, std::optional<Tensor> a1, int64_t k1,
+                std::optional<Tensor> mix, std::optional<Tensor> out_w, Tensor in_w,
+                std::optional<Tensor> w, double eps) {
+  check_gpu(src, "src");
+  c10::hip::HIPGuardMasqueradingAsCUDA g(src.device());
+  TORCH_CHECK(src.scalar_type() == at::kFloat && src.dim() == 3 && src.stride(2) == 1,
+              "kgc.hyper_norm: src fp32 [rows, S, W]");
+  const int64_t rows = src.size(0), S = src.size(1), W = src.size(2);
+  TORCH_CHECK(S >= 1 && S <= kgc::hyper_max_streams() && W >= 1 && W <= 16384,
+              "kgc.hyper_norm: streams / width");
+  TORCH_CHECK(mix.has_value() == out_w.has_value() && (mix.has_value() || (!dst && !a0 && !a1)),
+              "kgc.hyper_norm: addends and dst come with mix and out_w");
+  if (dst.has_value())
+    TORCH_CHECK(dst->is_cuda() && dst->scalar_type() == at::kFloat && dst->is_contiguous() &&
+                dst->sizes() == src.sizes() && dst->device() == src.device(),
+                "kgc.hyper_norm: dst fp32 [rows, S, W]");
+  int dt = kgc::DT_F32, odt = kgc::DT_F32;
+  bool typed = false;
+  kgc::HyperAdds ad{};
+  const std::optional<Tensor>* as[2] = {&a0, &a1};
+  const int64_t ks[2] = {k0, k1};
+  for (int j = 0; j < 2; ++j) {
+    const auto& a = *as[j];
+    if (!a.has_value()) continue;
+    const bool sl = a->dim() == 3;
+    TORCH_CHECK(a->is_cuda() && a->is_contiguous() && a->device() == src.device() && ks[j] >= 1 &&
+                (sl ? a->scalar_type() == at::kFloat : a->dim() == 2 && act_dtype(*a)) &&
+                a->size(-1) == W && a->size(-2) == rows * ks[j],
+                "kgc.hyper_norm: addend [rows k, W], or fp32 [slices, rows k, W]");
+    ad.a[j] = a->data_ptr();
+    ad.k[j] = (int)ks[j];
+    ad.slices[j] = sl ? (int)a->size(0) : 0;
+    ad.ss[j] = sl ? a->stride(0) : 0;
+    if (!sl) {
+      TORCH_CHECK(!typed || dt_code(*a) == dt, "kgc.hyper_norm: addends of one dtype");
+      dt = dt_code(*a);
+      typed = true;
+    }
+  }
+  void* op = nullptr;
+  if (out.has_value()) {
+    TORCH_CHECK(out->is_cuda() && out->is_contiguous() && out->dim() == 2 && out->size(0) == rows &&
+                out->size(1) == W && act_dtype(*out) && out->device() == src.device(),
+                "kgc.hyper_norm: out [rows, W]");
+    odt = dt_code(*out);
+    if (!typed) dt = odt;
+    TORCH_CHECK(odt == kgc::DT_F32 || odt == dt,
+                "kgc.hyper_norm: out is fp32 or of the addends' dtype");
+    op = out->data_ptr();
+  }
+  kgc::launch_hyper_norm(dt, odt, op, src.data_ptr<float>(), src.stride(0), src.stride(1),
+                         dst ? dst->data_ptr<float>() : nullptr, ad, f32_opt(mix, S * S, "mix"),
+                         f32_opt(out_w, S, "out_w"), f32_opt(in_w, S, "in_w"), f32_opt(w, W, "w"),
+                         (int)rows, (int)S, (int)W, (float)eps, stream());
+}
+
+void latent_down_store(Tensor cq, Tensor gate, Tensor proj, Tensor positions,
+                       std::optional<Tensor> table, Tensor q_w, Tensor kv_w, double eps,
+                       Tensor cache, Tensor slots, int64_t r) {
+  check_gpu(proj, "proj");
+  check_f32(gate, "gate");
+  check_f32(q_w, "q_w");
+  check_f32(kv_w, "kv_w");
+  c10::hip::HIPGuardMasqueradingAsCUDA g(proj.device());
+  const int64_t T = proj.size(0), qr = q_w.numel(), rank = kv_w.numel();
+  TORCH_CHECK(gate.dim() == 2 && gate.size(0) == T && gate.is_contiguous() &&
+              gate.device() == proj.device(), "kgc.latent_down_store: gate fp32 [T, gates]");
+  const int64_t gates = gate.size(1);
+  TORCH_CHECK(r >= 0 && r % 2 == 0 && qr >= 1 && rank >= 1 && proj.dim() == 2 &&
+              proj.stride(1) == 1 && act_dtype(proj) && proj.size(1) >= qr + rank + r + gates,
+              "kgc.latent_down_store: proj [T, q_rank + rank + r + gates ...]");
+  TORCH_CHECK(q_w.device() == proj.device() && kv_w.device() == proj.device(),
+              "kgc.latent_down_store: weights on proj's device");
+  TORCH_CHECK(cq.is_cuda() && cq.is_contiguous() && cq.numel() == T * qr &&
+              cq.scalar_type() == proj.scalar_type() && cq.device() == proj.device(),
+              "kgc.latent_down_store: cq [T, q_rank]");
+  TORCH_CHECK(cache.is_cuda() && cache.dim() == 4 && cache.is_contiguous() && cache.size(1) == 1 &&
+              cache.size(3) == rank + r && cache.scalar_type() == proj.scalar_type() &&
+              cache.device() == proj.device(), "kgc.latent_down_store: cache [nb, 1, bs, rank + r]");
+  TORCH_CHECK(positions.scalar_type() == at::kLong && positions.numel() == T &&
+              positions.is_contiguous() && slots.scalar_type() == at::kLong &&
+              slots.numel() == T && slots.is_contiguous() && positions.is_cuda() && slots.is_cuda(),
+              "kgc.latent_down_store: positions / slots int64 [T]");
+  const float* tp = nullptr;
+  int64_t rows = 0;
+  if (r > 0) {
+    TORCH_CHECK(table.has_value(), "kgc.latent_down_store: rotary table missing");
+    check_f32(*table, "table");
+    TORCH_CHECK(table->dim() == 2 && table->size(1) == r && table->size(0) >= 1 &&
+                table->is_contiguous() && table->device() == proj.device(),
+                "kgc.latent_down_store: table [max_pos, r]");
+    tp = table->data_ptr<float>();
+    rows = table->size(0);
+  }
+  kgc::launch_latent_down_store(dt_code(proj), cq.data_ptr(), gate.data_ptr<float>(),
+                                proj.data_ptr(), proj.stride(0), positions.data_ptr<int64_t>(), tp,
+                                (int)rows, q_w.data_ptr<float>(), kv_w.data_ptr<float>(),
+                                (float)eps, cache.data_ptr(), slots.data_ptr<int64_t>(),
+                                cache.size(0) * cache.size(2), (int)T, (int)qr, (int)rank, (int)r,
+                                (int)gates, stream());
+}
+
+void head_gemm(Tensor out, Tensor x, Tensor w, std::optional<Tensor> rot,
+               std::optional<Tensor> positions, std::optional<Tensor> table) {
+  check_gpu(x, "x");
+  c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
+  TORCH_CHECK(x.dim() == 3 && x.stride(2) == 1 && act_dtype(x) && w.is_cuda() && w.dim() == 3 &&
+              w.is_contiguous() && w.size(0) == x.size(1) && w.size(2) == x.size(2) &&
+              w.scalar_type() == x.scalar_type() && w.device() == x.device(),
+              "kgc.head_gemm: x [T, H, K], w [H, N, K]");
+  kgc::HeadGemm a{};
+  a.T = (int)x.size(0);
+  a.H = (int)x.size(1);
+  a.K = (int)x.size(2);
+  a.N = (int)w.size(1);
+  TORCH_CHECK(a.K >= 1 && a.K <= 16384 && a.N >= 1 && a.H >= 1 && a.H <= 65535, "kgc.head_gemm: sizes");
+  a.r = rot ? (int)rot->size(-1) : 0;
+  TORCH_CHECK(out.is_cuda() && out.dim() == 3 && out.size(0) == a.T && out.size(1) == a.H &&
+              out.size(2) == a.N + a.r && out.stride(2) == 1 && out.stride(1) >= out.size(2) &&
+              (a.T <= 1 || out.stride(0) >= a.H * out.stride(1)) &&
+              out.scalar_type() == x.scalar_type() && out.device() == x.device(),
+              "kgc.head_gemm: out [T, H, N + r]");
+  a.out = out.data_ptr();
+  a.os = out.stride(0);
+  a.oh = out.stride(1);
+  a.x = x.data_ptr();
+  a.xs = x.stride(0);
+  a.xh = x.stride(1);
+  a.w = w.data_ptr();
+  if (a.r > 0) {
+    TORCH_CHECK(rot->is_cuda() && rot->dim() == 3 && rot->size(0) == a.T && rot->size(1) == a.H &&
+                rot->stride(2) == 1 && a.r % 2 == 0 && rot->scalar_type() == x.scalar_type() &&
+                rot->device() == x.device() && positions.has_value() && table.has_value(),
+                "kgc.head_gemm: rot [T, H, r] with positions and a table");
+    check_f32(*table, "table");
+    TORCH_CHECK(table->dim() == 2 && table->size(1) == a.r && table->size(0) >= 1 &&
+                table->is_contiguous() && table->device() == x.device(),
+                "kgc.head_gemm: table [max_pos, r]");
+    TORCH_CHECK(positions->is_cuda() && positions->scalar_type() == at::kLong &&
+                positions->is_contiguous() && positions->numel() == a.T, "kgc.head_gemm: positions");
+    TORCH_CHECK((int64_t)a.T * (a.r / 2) < (int64_t(1) << 31), "kgc.head_gemm: rows");
+    a.rot = rot->data_ptr();
+    a.rs = rot->stride(0);
+    a.rh = rot->stride(1);
+    a.positions = positions->data_ptr<int64_t>();
+    a.table = table->data_ptr<float>();
+    a.table_rows = (int)table->size(0);
+  }
+  kgc::launch_head_gemm(dt_code(x), a, stream());
+}
+
+void check_pairs(const Tensor& topk_w, int64_t T, int64_t k) {
+  TORCH_CHECK(topk_w.is_cuda() && topk_w.scalar_type() == at::kFloat && topk_w.is_contiguous() &&
+              topk_w.numel() == T * k, "kgc: routing weights fp32 [T, k]");
+}
+
+void expert_silu_all(Tensor out, Tensor x, Tensor topk_w, Tensor topk_ids, int64_t E, int64_t I,
+                     int64_t Is) {
+  check_gpu(x, "x");
+  c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
+  const int64_t T = x.size(0), n = E * I + Is;
+  TORCH_CHECK(E >= 1 && I >= 1 && Is >= 0 && n < (int64_t(1) << 30) && x.dim() == 2 &&
+              x.is_contiguous() && act_dtype(x) && x.size(1) == 2 * n,
+              "kgc.expert_silu_all: x [T, 2 (E I + Is)]");
+  TORCH_CHECK(out.is_cuda() && out.is_contiguous() && out.dim() == 2 && out.size(0) == T &&
+              out.size(1) == n && out.scalar_type() == x.scalar_type() && out.device() == x.device(),
+              "kgc.expert_silu_all: out [T, E I + Is]");
+  TORCH_CHECK(topk_ids.is_cuda() && topk_ids.dim() == 2 && topk_ids.size(0) == T &&
+              topk_ids.scalar_type() == at::kInt && topk_ids.is_contiguous() &&
+              topk_ids.device() == x.device() && topk_w.device() == x.device(),
+              "kgc.expert_silu_all: topk_ids int32 [T, k]");
+  check_pairs(topk_w, T, topk_ids.size(1));
+  kgc::launch_expert_silu_all(dt_code(x), out.data_ptr(), x.data_ptr(), topk_w.data_ptr<float>(),
+                              topk_ids.data_ptr<int>(), (int)T, (int)E, (int)topk_ids.size(1),
+                              (int)I, (int)Is, stream());
+}
+
+void expert_silu_rows(Tensor out, Tensor x, Tensor topk_w, Tensor sorted_ids) {
+  check_gpu(x, "x");
+  c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
+  TORCH_CHECK(x.dim() == 2 && x.is_contiguous() && act_dtype(x) && x.size(1) % 2 == 0 &&
+              out.is_cuda() && out.is_contiguous() && out.dim() == 2 && out.size(0) == x.size(0) &&
+              out.size(1) * 2 == x.size(1) && out.scalar_type() == x.scalar_type() &&
+              out.device() == x.device(), "kgc.expert_silu_rows: x [rows, 2 I], out [rows, I]");
+  TORCH_CHECK(sorted_ids.is_cuda() && sorted_ids.scalar_type() == at::kInt &&
+              sorted_ids.is_contiguous() && sorted_ids.numel() >= x.size(0) &&
+              sorted_ids.device() == x.device() && topk_w.device() == x.device(),
+              "kgc.expert_silu_rows: sorted_ids int32 [rows]");
+  check_pairs(topk_w, topk_w.numel(), 1);
+  kgc::launch_expert_silu_rows(dt_code(x), out.data_ptr(), x.data_ptr(), topk_w.data_ptr<float>(),
+                               sorted_ids.data_ptr<int>(), (int)topk_w.numel(), x.size(0),
+                               (int)out.size(1), stream());
+}
+
 }  // namespace
 
 TORCH_LIBRARY(kgc, m) {
+  m.def("hyper_norm(Tensor(a!)? out, Tensor src, Tensor(b!)? dst, Tensor? a0, int k0, Tensor? a1, "
+        "int k1, Tensor? mix, Tensor? out_w, Tensor in_w, Tensor? w, float eps) -> ()");
+  m.def("latent_down_store(Tensor(a!) cq, Tensor(b!) gate, Tensor proj, Tensor positions, "
+        "Tensor? table, Tensor q_w, Tensor kv_w, float eps, Tensor(c!) cache, Tensor slots, int r) -> ()");
+  m.def("head_gemm(Tensor(a!) out, Tensor x, Tensor w, Tensor? rot, Tensor? positions, Tensor? table) "
+        "-> ()");
+  m.def("expert_silu_all(Tensor(a!) out, Tensor x, Tensor topk_w, Tensor topk_ids, int E, int I, "
+        "int Is) -> ()");
+  m.def("expert_silu_rows(Tensor(a!) out, Tensor x, Tensor topk_w, Tensor sorted_ids) -> ()");
   m.def("residual_sum_norm(Tensor(a!)? out, Tensor(b!) x, Tensor? a0, Tensor? w0, Tensor? a1, "
         "Tensor? w1, Tensor? a2, Tensor? w2, Tensor? w, float eps) -> ()");
   m.def("qk_norm_store(Tensor(a!) q_out, Tensor qkv, Tensor positions, Tensor qw, Tensor? kw, "
@@ -2325,7 +2539,7 @@ TORCH_LIBRARY(kgc, m) {
         "Tensor slots, int P, int D, int Tp, float out_scale) -> ()");
   m.def("norm_kv_store(Tensor qkv, Tensor positions, Tensor(a!) q_out, Tensor(b!) k_cache, "
         "Tensor(c!) v_cache, Tensor slots, int H, int G, int dk, int dv, float eps, bool qk_unit, "
-        "bool v_unit, float coef, int every) -> ()");
+        "bool v_unit, float coef, int every, Tensor? q_w=None, Tensor? k_w=None) -> ()");
   m.def("polynorm(Tensor(a!) out, Tensor z, Tensor coef, float eps) -> ()");
   m.def("swiglu_clamp(Tensor(a!) out, Tensor x, float limit, float alpha) -> ()");
   m.def("embed_pos(Tensor(a!) out, Tensor ids, Tensor positions, Tensor table, Tensor? pos_table, "
@@ -2356,7 +2570,8 @@ TORCH_LIBRARY(kgc, m) {
   m.def("side_gate(Tensor(a!) out, Tensor pre, Tensor ids, Tensor table, int col0) -> ()");
   m.def("side_input_rows(Tensor(a!)? out, Tensor(b!) x, Tensor? y, Tensor wg, Tensor wp, Tensor ids, "
         "Tensor table, int col0, Tensor side_w, Tensor? w, float mult, float eps) -> bool");
-  m.def("moe_route_sigmoid(Tensor(a!) w, Tensor(b!) ids, Tensor scores, Tensor correction, float scale) -> ()");
+  m.def("moe_route_sigmoid(Tensor(a!) w, Tensor(b!) ids, Tensor scores, Tensor? correction, float scale, "
+        "bool renorm=True) -> ()");
   m.def("moe_finish(Tensor(a!) out, Tensor? routed, Tensor? dense, Tensor? topk_w, Tensor? topk_ids, "
         "Tensor? shared, Tensor? gate) -> ()");
   m.def("residual_group_norm(Tensor(a!) out, Tensor(b!) x, Tensor? y, Tensor w, int groups, float eps) -> ()");
@@ -2372,7 +2587,7 @@ TORCH_LIBRARY(kgc, m) {
         "Tensor? seq_lens, Tensor? pbt, Tensor? ctx_lens, Tensor? dbt, Tensor? work_seq, Tensor? work_blk, "
         "int P, int D, int Tp, float scale, int window, int keep_first, Tensor? gate, bool fast, "
         "float softcap, float out_scale, Tensor? elem_gate, int pool, int block_size, "
-        "Tensor? v_table, bool interleaved, Tensor? slots) -> ()");
+        "Tensor? v_table, bool interleaved, Tensor? slots, bool chunked, float sink) -> ()");
   m.def("mlstm_scan(Tensor(a!) out, Tensor qkvg, Tensor gates, Tensor(b!) S, Tensor(c!) n, Tensor(d!) m, "
         "Tensor? qsl, Tensor? seq_lens, Tensor? ctx_lens, Tensor slots, int P, int D, int Tp, int H, int d, "
         "int dv) -> ()");
@@ -2488,6 +2703,11 @@ TORCH_LIBRARY_IMPL(kgc, CUDA, m) {
   m.impl("selective_scan", &selective_scan);
   m.impl("norm_kv_store", &norm_kv_store);
   m.impl("residual_sum_norm", &residual_sum_norm);
+  m.impl("hyper_norm", &hyper_norm);
+  m.impl("latent_down_store", &latent_down_store);
+  m.impl("head_gemm", &head_gemm);
+  m.impl("expert_silu_all", &expert_silu_all);
+  m.impl("expert_silu_rows", &expert_silu_rows);
   m.impl("qk_norm_store", &qk_norm_store);
   m.impl("delta_gates", &delta_gates);
   m.impl("channel_delta_scan", &channel_delta_scan);

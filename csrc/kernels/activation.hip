@@ -1,6 +1,8 @@
 // K7 SiLU-and-mul: out[t, i] = silu(x[t, i]) * x[t, I + i] over the fused gate_up
 // projection output.  16-byte vector loads/stores (8 halves per lane), one vector
 // per thread on a 2-D grid (memory-bound; no index division).
+#include <algorithm>
+
 #include "common.h"
 #include "launch.h"
 
@@ -191,6 +193,62 @@ __global__ __launch_bounds__(256) void swiglu_clamp_kernel(T* __restrict__ out,
   }
 }
 
+// A gated pair of a scaled input: silu(w g) * (w u)
+__device__ __forceinline__ float scaled_silu(float g, float u, float w) {
+  const float gv = w * g;
+  return gv / (1.f + expf(-gv)) * (w * u);
+}
+
+// Every expert's activation for every token: x [T, E 2 I + 2 Is] = per expert gate | up, then the
+// shared expert's -> out [T, E I + Is]; w [T, k] / ids [T, k]: the token's experts and their
+// weights, zeros for the others, 1 for the shared one.  VEC adjacent columns lie in one expert.
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void expert_silu_all_kernel(
+    T* __restrict__ out, const T* __restrict__ x, const float* __restrict__ w,
+    const int* __restrict__ ids, int E, int k, int I, int Is) {
+  const int c = (blockIdx.x * 256 + threadIdx.x) * VEC, n = E * I + Is;
+  if (c >= n) return;
+  const int64_t t = blockIdx.y;
+  const int e = c < E * I ? c / I : E, i = c - e * I, len = e < E ? I : Is;
+  float we = e < E ? 0.f : 1.f;
+  for (int j = 0; j < k; ++j)
+    if (ids[t * k + j] == e) we = w[t * k + j];
+  float o[VEC];
+  if (we == 0.f) {
+#pragma unroll
+    for (int q = 0; q < VEC; ++q) o[q] = 0.f;
+  } else {
+    const T* xr = x + t * 2 * n + (int64_t)e * 2 * I + i;
+    float g[VEC], u[VEC];
+    load_row<T, VEC>(xr, g);
+    load_row<T, VEC>(xr + len, u);
+#pragma unroll
+    for (int q = 0; q < VEC; ++q) o[q] = scaled_silu(g[q], u[q], we);
+  }
+  store_row<T, VEC>(out + t * n + c, o);
+}
+
+// Expert-sorted rows: out [rows, I] from x [rows, 2 I] = gate | up, row r scaled by the weight of
+// its pair sorted_ids[r]; rows without a pair (>= npairs) are left as they are.
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void expert_silu_rows_kernel(
+    T* __restrict__ out, const T* __restrict__ x, const float* __restrict__ w,
+    const int* __restrict__ sorted_ids, int npairs, int64_t rows, int I) {
+  const int c = (blockIdx.x * 256 + threadIdx.x) * VEC;
+  if (c >= I) return;
+  for (int64_t r = blockIdx.y; r < rows; r += gridDim.y) {
+    const int p = sorted_ids[r];
+    if (p < 0 || p >= npairs) continue;
+    const float we = w[p];
+    float g[VEC], u[VEC];
+    load_row<T, VEC>(x + r * 2 * I + c, g);
+    load_row<T, VEC>(x + r * 2 * I + I + c, u);
+#pragma unroll
+    for (int q = 0; q < VEC; ++q) g[q] = scaled_silu(g[q], u[q], we);
+    store_row<T, VEC>(out + r * I + c, g);
+  }
+}
+
 // out fp32 [T, W] = table[ids[t]] * scale + pos[positions[t]]
 template <typename T>
 __global__ __launch_bounds__(256) void embed_pos_kernel(
@@ -239,6 +297,41 @@ void launch_swiglu_clamp(int dtype, void* out, const void* x, int64_t rows, int 
   else
     KGC_ACT_DISPATCH_T(dtype, swiglu_clamp_kernel<T, 1><<<grid, 256, 0, s>>>(
         (T*)out, (const T*)x, rows, I, limit, alpha));
+}
+
+void launch_expert_silu_all(int dtype, void* out, const void* x, const float* w, const int* ids,
+                            int T_, int E, int k, int I, int Is, hipStream_t s) {
+  const int n = E * I + Is;
+  if (T_ <= 0 || n <= 0) return;
+  const bool vec = dtype != DT_F32 && I % 8 == 0 && Is % 8 == 0 &&
+                   reinterpret_cast<uintptr_t>(x) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0;
+  const int per = 256 * (vec ? 8 : 1);
+  for (int t0 = 0; t0 < T_; t0 += 65535) {         // gridDim.y <= 65535
+    const dim3 grid((n + per - 1) / per, std::min(T_ - t0, 65535));
+    const float* wt = w + (int64_t)t0 * k;
+    const int* it = ids + (int64_t)t0 * k;
+#define KGC_ESA(V)                                                                             \
+  KGC_ACT_DISPATCH_T(dtype, expert_silu_all_kernel<T, V><<<grid, 256, 0, s>>>(                 \
+      (T*)out + (int64_t)t0 * n, (const T*)x + (int64_t)t0 * 2 * n, wt, it, E, k, I, Is))
+    if (vec) KGC_ESA(8); else KGC_ESA(1);
+#undef KGC_ESA
+  }
+}
+
+void launch_expert_silu_rows(int dtype, void* out, const void* x, const float* w,
+                             const int* sorted_ids, int npairs, int64_t rows, int I,
+                             hipStream_t s) {
+  if (rows <= 0 || I <= 0) return;
+  const bool vec = dtype != DT_F32 && I % 8 == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0 &&
+                   reinterpret_cast<uintptr_t>(out) % 16 == 0;
+  const int per = 256 * (vec ? 8 : 1);
+  const dim3 grid((I + per - 1) / per, (unsigned)std::min<int64_t>(rows, 65535));
+  if (vec)
+    KGC_ACT_DISPATCH_T(dtype, expert_silu_rows_kernel<T, 8><<<grid, 256, 0, s>>>(
+        (T*)out, (const T*)x, w, sorted_ids, npairs, rows, I));
+  else
+    KGC_ACT_DISPATCH_T(dtype, expert_silu_rows_kernel<T, 1><<<grid, 256, 0, s>>>(
+        (T*)out, (const T*)x, w, sorted_ids, npairs, rows, I));
 }
 
 void launch_embed_pos(int dtype, float* out, const int64_t* ids, const int64_t* positions,

@@ -2,7 +2,8 @@
 // (k [nb, G, bs, dk], v [nb, G, bs, dv]; dk != dv allowed, any sizes), for the hybrid
 // decoders.  Rows are addressed through their strides (krs, vrs elements per cache row), so
 // the values may be columns of the key rows (one latent cache row per token).  Query i sees key j when j <= i and (i - j < window or j < keep_first);
-// window <= 0 means plain causal attention.  With pooled blocks (pool > 0) a page holds
+// window <= 0 means plain causal attention; ex.chunked: i sees the keys of its own chunk of
+// ``window`` positions instead; ex.sink: a score without a value in every softmax.  With pooled blocks (pool > 0) a page holds
 // ceil(bs / pool) further rows after its bs token rows: the mean key (value) row of every block
 // of pool tokens whose last token lies in the page; query i also sees the blocks that end
 // before its window.  Values may be cached turned by their positions (pairs over all dv
@@ -20,6 +21,8 @@
 //   qk_norm_store     RMS norm over the whole q row and the whole k row, rotation of q, k and
 //                     v, write of q and into the cache
 //   pool_kv           mean rows of the blocks that a step's tokens complete
+#include <algorithm>
+
 #include "common.h"
 #include "launch.h"
 
@@ -74,18 +77,20 @@ __global__ __launch_bounds__(256) void rope_kv_store_kernel(
   }
 }
 
-// Attention inputs as unit-RMS vectors: qkv fp32 [T, H dk + G dk + G dv] (row stride qs).
-// Each head's q and k (qk_unit) and v (v_unit) is divided by sqrt(mean(x^2) + eps); q at
-// position p is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1); q goes to q_out
-// [T, H, dk], k and v into the cache.  One wave per head vector, fp32 math.
-template <typename T>
+// Attention inputs normed per head: qkv [T, H dk + G dk + G dv] of type TI (row stride qs).
+// Each head's q and k (qk_unit) and v (v_unit) is divided by sqrt(mean(x^2) + eps), q and k are
+// multiplied by qw / kw [dk] (null: none), q at position p by
+// 1 + coef * ln(floor((p + 1) / every) + 1); q goes to q_out [T, H, dk], k and v into the cache.
+// fp32 math.  One wave per head vector, any sizes.
+template <typename TI, typename T>
 __global__ __launch_bounds__(256) void norm_kv_store_kernel(
-    const float* __restrict__ qkv, int64_t qs, const int64_t* __restrict__ positions,
+    const TI* __restrict__ qkv, int64_t qs, const int64_t* __restrict__ positions,
     T* __restrict__ q_out, T* __restrict__ k_cache, T* __restrict__ v_cache,
     const int64_t* __restrict__ slots, int H, int G, int dk, int dv, int bs, int num_blocks,
-    float eps, bool qk_unit, bool v_unit, float coef, int every) {
+    float eps, bool qk_unit, bool v_unit, float coef, int every, const float* __restrict__ qw,
+    const float* __restrict__ kw) {
   const int64_t t = blockIdx.x;
-  const float* row = qkv + t * qs;
+  const TI* row = qkv + t * qs;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   int64_t pos = positions[t];
   if (pos < 0) pos = 0;
@@ -96,20 +101,31 @@ __global__ __launch_bounds__(256) void norm_kv_store_kernel(
   for (int hv = wave; hv < H + 2 * G; hv += 4) {
     const bool isq = hv < H, isk = !isq && hv < H + G;
     const int n = hv < H + G ? dk : dv;
-    const float* src = row + (hv < H + G ? hv * dk : (H + G) * dk + (hv - H - G) * dv);
+    const TI* src = row + (hv < H + G ? hv * dk : (H + G) * dk + (hv - H - G) * dv);
     if (!isq && !store) continue;
     float f = isq ? temp : 1.f;
     if (isq || isk ? qk_unit : v_unit) {
       float ss = 0.f;
-      for (int i = lane; i < n; i += 64) ss += src[i] * src[i];
+      for (int i = lane; i < n; i += 64) {
+        const float v = to_f(src[i]);
+        ss += v * v;
+      }
       ss = wave_sum(ss);
       f /= sqrtf(ss / (float)n + eps);
     }
+    const float* w = isq ? qw : isk ? kw : nullptr;
     T* dst = isq ? q_out + (t * H + hv) * dk
                  : isk ? k_cache + ((blk * G + (hv - H)) * bs + off) * dk
                        : v_cache + ((blk * G + (hv - H - G)) * bs + off) * dv;
-    for (int i = lane; i < n; i += 64) dst[i] = from_f<T>(src[i] * f);
+    for (int i = lane; i < n; i += 64)
+      dst[i] = from_f<T>(to_f(src[i]) * f * (w != nullptr ? w[i] : 1.f));
   }
+}
+
+// first position that a query at `pos` sees
+__device__ __forceinline__ int first_visible(int pos, int window, bool chunked) {
+  if (window <= 0) return 0;
+  return chunked ? pos - pos % window : max(0, pos - window + 1);
 }
 
 // whole blocks of `pool` tokens that end before the window of a query at `pos`
@@ -225,11 +241,11 @@ __global__ __launch_bounds__(64) void window_attention_kernel(
   const T* qrow = q + ((int64_t)t * H + h) * dk;
   for (int c = lane; c < dk; c += 64) qs[c] = to_f(qrow[c]);
   __syncthreads();
-  const int lo_w = window > 0 ? max(0, pos - window + 1) : 0;
+  const int lo_w = first_visible(pos, window, ex.chunked);
   // kept first tokens outside the window, or the pooled blocks before it
   const int ns = ex.pool > 0 ? pooled_count(pos, window, ex.pool) : min(keep_first, lo_w);
   const int total = ns + (pos - lo_w + 1);
-  float m = -INFINITY, l = 0.f;
+  float m = ex.sink, l = ex.sink > -INFINITY ? 1.f : 0.f;
   float acc[MAX_DV_PER_LANE];
 #pragma unroll
   for (int u = 0; u < MAX_DV_PER_LANE; ++u) acc[u] = 0.f;
@@ -392,7 +408,7 @@ __global__ __launch_bounds__(64 * NWV) void window_decode_kernel(
     qs[e] = to_f(q[((int64_t)t * H + h0) * dk + e]);
   for (int e = threadIdx.x; e < QH * dv; e += 64 * NWV) accs[e] = 0.f;
   __syncthreads();
-  const int lo_w = window > 0 ? max(0, pos - window + 1) : 0;
+  const int lo_w = first_visible(pos, window, ex.chunked);
   int ns = min(keep_first, lo_w);
   if constexpr (EXT) {
     if (ex.pool > 0) {
@@ -407,8 +423,8 @@ __global__ __launch_bounds__(64 * NWV) void window_decode_kernel(
   float m[QH], l[QH], acc[QH][DEC_UMAX][2];
 #pragma unroll
   for (int h = 0; h < QH; ++h) {
-    m[h] = -INFINITY;
-    l[h] = 0.f;
+    m[h] = wave == 0 ? ex.sink : -INFINITY;           // (the first wave always has keys)
+    l[h] = m[h] > -INFINITY ? 1.f : 0.f;
 #pragma unroll
     for (int u = 0; u < DEC_UMAX; ++u) acc[h][u][0] = acc[h][u][1] = 0.f;
   }
@@ -621,7 +637,7 @@ __global__ __launch_bounds__(64 * NWV) void window_decode_kernel(
 // (64 query rows of a chunk, query head); wave w owns rows 16 w .. 16 w + 15.  Keys come in
 // 64-key tiles -- first the kept first tokens that lie before the tile's earliest window,
 // then the span from that window's start to the last row -- gathered from the pages into
-// LDS as K [64][dk + 8] and V^T [dv][64 + 8].  Per tile and wave:
+// LDS as K [64][dk, padded to 32, + 8] and V^T [dv][64 + 8].  Per tile and wave:
 //   S^T = K . Q^T   (v_mfma_f32_16x16x32; the query is lane & 15 in every accumulator, so
 //                    the softmax statistics are lane-local up to two shuffles),
 //   visibility mask, online softmax in fp32,
@@ -644,8 +660,9 @@ __global__ __launch_bounds__(256, KSM <= 4 ? 3 : 2) void window_prefill_mfma_ker
     WindowExtra ex) {
   typedef typename Vec8<T>::type V8;
   extern __shared__ float lds_f[];
-  T* Ks = reinterpret_cast<T*>(lds_f);                 // [64][dk + 8]
-  const int kst = dk + PFW_KPAD, vst = PFW_BN + PFW_VPAD;
+  T* Ks = reinterpret_cast<T*>(lds_f);                 // [64][kp + 8]
+  const int kp = (dk + 31) & ~31;                      // key rows padded with zeros in LDS
+  const int kst = kp + PFW_KPAD, vst = PFW_BN + PFW_VPAD;
   T* Vt = Ks + PFW_BN * kst;                           // [dv][64 + 8]
   const int item = blockIdx.x / (blk_rows / PFW_BM), sub = blockIdx.x % (blk_rows / PFW_BM);
   const int seq = work_seq[item], h = blockIdx.y, g = h / (H / G);
@@ -654,7 +671,7 @@ __global__ __launch_bounds__(256, KSM <= 4 ? 3 : 2) void window_prefill_mfma_ker
   if (r0 >= qlen || ctx0 < 0) return;
   const int rows = min(PFW_BM, qlen - r0);
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r16 = lane & 15, qd = lane >> 4;
-  const int nks = dk >> 5, ndt = dv >> 4;
+  const int nks = kp >> 5, ndt = dv >> 4;
   const int* bt = pbt + (int64_t)seq * bt_stride;
   const int myrow = r0 + 16 * wave + r16;
   const bool rowok = myrow < qlen;
@@ -667,16 +684,17 @@ __global__ __launch_bounds__(256, KSM <= 4 ? 3 : 2) void window_prefill_mfma_ker
     for (int s2 = 0; s2 < KSM; ++s2) {
       Pack8<T> tq;
       tq.u = u32x4{0u, 0u, 0u, 0u};
-      if (s2 < nks && rowok) tq.u = *reinterpret_cast<const u32x4*>(qrow + 32 * s2 + 8 * qd);
+      if (32 * s2 + 8 * qd < dk && rowok) tq.u = *reinterpret_cast<const u32x4*>(qrow + 32 * s2 + 8 * qd);
       qf[s2] = tq.v;
     }
   }
   f32x4 o[DTM];
 #pragma unroll
   for (int t2 = 0; t2 < DTM; ++t2) o[t2] = f32x4{0.f, 0.f, 0.f, 0.f};
-  float m = -INFINITY, l = 0.f;
+  float m = ex.sink, l = qd == 0 && ex.sink > -INFINITY ? 1.f : 0.f;
   const int p_min = ctx0 + r0, p_max = ctx0 + r0 + rows - 1;
-  const int lo_min = window > 0 ? max(0, p_min - window + 1) : 0;
+  const int lo_min = first_visible(p_min, window, ex.chunked);
+  const int row_lo = first_visible(qpos, window, ex.chunked);
   int ns = window > 0 ? min(keep_first, lo_min) : 0;
   const bool pooled = EXT && ex.pool > 0;
   if (pooled) ns = pooled_count(p_max, window, ex.pool);     // what the last row sees
@@ -685,9 +703,10 @@ __global__ __launch_bounds__(256, KSM <= 4 ? 3 : 2) void window_prefill_mfma_ker
   const int nmain = (p_max - lo_min + PFW_BN) / PFW_BN;
   // the wave's own span of visible keys (tiles outside it are staged but not computed)
   const int wp_lo = ctx0 + r0 + 16 * wave, wp_hi = min(wp_lo + 15, p_max);
-  const int w_lo = window > 0 ? max(0, wp_lo - window + 1) : 0;
+  const int w_lo = first_visible(wp_lo, window, ex.chunked);
+  const int w_lo_hi = first_visible(wp_hi, window, ex.chunked);
   const int keyA = 8 * (r16 >> 2) + (r16 & 3);
-  const int kchunks = dk >> 3, vchunks = dv >> 3;
+  const int kchunks = kp >> 3, vchunks = dv >> 3;
   const int bs_shift = (bs & (bs - 1)) == 0 ? __builtin_ctz(bs) : -1;
   auto page_row = [&](int key) -> int64_t {
     const int pg = bs_shift >= 0 ? key >> bs_shift : key / bs;
@@ -715,7 +734,7 @@ __global__ __launch_bounds__(256, KSM <= 4 ? 3 : 2) void window_prefill_mfma_ker
       const T* src = key < hi ? k_cache + (ptile ? block_row(key) : page_row(key)) * krs : nullptr;
       for (int c = sc; c < kchunks; c += 16) {
         u32x4 val = u32x4{0u, 0u, 0u, 0u};
-        if (src != nullptr) val = *reinterpret_cast<const u32x4*>(src + 8 * c);
+        if (src != nullptr && 8 * c < dk) val = *reinterpret_cast<const u32x4*>(src + 8 * c);
         *reinterpret_cast<u32x4*>(Ks + ks * kst + 8 * c) = val;
       }
     }
@@ -766,7 +785,7 @@ __global__ __launch_bounds__(256, KSM <= 4 ? 3 : 2) void window_prefill_mfma_ker
     const int nblk = ptile ? pooled_count(qpos, window, ex.pool) : 0;
     const bool full = ptile ? kb + PFW_BN <= pooled_count(wp_lo, window, ex.pool) && wp_lo + 15 == wp_hi
                             : hi == kb + PFW_BN && kb + PFW_BN - 1 <= wp_lo &&
-                                  (window <= 0 || wp_hi - kb < window) && wp_lo + 15 == wp_hi;
+                                  kb >= w_lo_hi && wp_lo + 15 == wp_hi;
     float tmax = -INFINITY;
     if (full) {
 #pragma unroll
@@ -784,7 +803,7 @@ __global__ __launch_bounds__(256, KSM <= 4 ? 3 : 2) void window_prefill_mfma_ker
           const int key = kb + (j >> 1) * 32 + 8 * qd + 4 * (j & 1) + i;
           const bool vis = ptile ? rowok && key < nblk
                                  : rowok && key < hi && key <= qpos &&
-                                       (window <= 0 || qpos - key < window || key < keep_first);
+                                       (key >= row_lo || key < keep_first);
           s[j][i] = vis ? cap_score(s[j][i] * scale, ex.softcap) : -INFINITY;
           tmax = fmaxf(tmax, s[j][i]);
         }
@@ -901,6 +920,57 @@ __device__ __forceinline__ void store_vec(T* p, const float (&v)[VEC]) {
 #pragma unroll
     for (int e = 0; e < 8; ++e) t.h[e] = from_f<T>(v[e]);
     *reinterpret_cast<u32x4*>(p) = t.u;
+  }
+}
+
+// norm_kv_store for head sizes that are multiples of 8 (<= 512) and 16-byte rows: 2^lsh lanes take
+// one head vector, 8 adjacent elements each, and sum over themselves.
+template <typename TI, typename T>
+__global__ __launch_bounds__(256) void norm_kv_store_vec_kernel(
+    const TI* __restrict__ qkv, int64_t qs, const int64_t* __restrict__ positions,
+    T* __restrict__ q_out, T* __restrict__ k_cache, T* __restrict__ v_cache,
+    const int64_t* __restrict__ slots, int H, int G, int dk, int dv, int bs, int num_blocks,
+    float eps, bool qk_unit, bool v_unit, float coef, int every, const float* __restrict__ qw,
+    const float* __restrict__ kw, int lsh) {
+  const int64_t t = blockIdx.x;
+  const TI* row = qkv + t * qs;
+  int64_t pos = positions[t];
+  if (pos < 0) pos = 0;
+  const float temp = coef != 0.f ? 1.f + coef * logf((float)((pos + 1) / every) + 1.f) : 1.f;
+  const int64_t slot = slots[t];
+  const bool store = slot >= 0 && slot < (int64_t)num_blocks * bs;
+  const int64_t blk = store ? slot / bs : 0, off = store ? slot % bs : 0;
+  const int c = (threadIdx.x & ((1 << lsh) - 1)) * 8;
+  const int nv = store ? H + 2 * G : H;
+  for (int hv = threadIdx.x >> lsh; hv < nv; hv += 256 >> lsh) {
+    const bool isq = hv < H, isk = !isq && hv < H + G;
+    const int n = hv < H + G ? dk : dv;
+    const TI* src = row + (hv < H + G ? hv * dk : (H + G) * dk + (hv - H - G) * dv);
+    float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    if (c < n) load8(src + c, v);
+    float f = isq ? temp : 1.f;
+    if (isq || isk ? qk_unit : v_unit) {
+      float ss = 0.f;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) ss += v[e] * v[e];
+      for (int o = 1; o < (1 << lsh); o <<= 1) ss += __shfl_xor(ss, o, 64);
+      f /= sqrtf(ss / (float)n + eps);
+    }
+    if (c < n) {
+      const float* w = isq ? qw : isk ? kw : nullptr;
+      float wv[8];
+      if (w != nullptr) {
+        load8(w + c, wv);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] *= wv[e];
+      }
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] *= f;
+      T* dst = isq ? q_out + (t * H + hv) * dk
+                   : isk ? k_cache + ((blk * G + (hv - H)) * bs + off) * dk
+                         : v_cache + ((blk * G + (hv - H - G)) * bs + off) * dv;
+      store_vec<T, 8>(dst + c, v);
+    }
   }
 }
 
@@ -1176,14 +1246,32 @@ void launch_rope_kv_store(int dtype, const void* qkv, int64_t qkv_stride,
       (T*)v_cache, slots, H, G, dk, dv, bs, num_blocks, interleaved));
 }
 
-void launch_norm_kv_store(int out_dtype, const float* qkv, int64_t qs, const int64_t* positions,
-                          void* q_out, void* k_cache, void* v_cache, const int64_t* slots, int T_,
-                          int H, int G, int dk, int dv, int bs, int num_blocks, float eps,
-                          bool qk_unit, bool v_unit, float coef, int every, hipStream_t s) {
+void launch_norm_kv_store(int dtype, int out_dtype, const void* qkv, int64_t qs,
+                          const int64_t* positions, void* q_out, void* k_cache, void* v_cache,
+                          const int64_t* slots, int T_, int H, int G, int dk, int dv, int bs,
+                          int num_blocks, float eps, bool qk_unit, bool v_unit, float coef,
+                          int every, const float* qw, const float* kw, hipStream_t s) {
   if (T_ <= 0) return;
-  KGC_DISPATCH_T(out_dtype, norm_kv_store_kernel<T><<<T_, 256, 0, s>>>(
-      qkv, qs, positions, (T*)q_out, (T*)k_cache, (T*)v_cache, slots, H, G, dk, dv, bs,
-      num_blocks, eps, qk_unit, v_unit, coef, every));
+  auto al = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
+  const bool vec = dk % 8 == 0 && dv % 8 == 0 && dk <= 512 && dv <= 512 &&
+                   qs % (dtype == DT_F32 ? 4 : 8) == 0 && al(qkv) && al(q_out) && al(k_cache) &&
+                   al(v_cache) && al(qw) && al(kw);
+  int lsh = 0;
+  while ((8 << lsh) < std::max(dk, dv)) ++lsh;
+#define KGC_NKV(TI)                                                                             \
+  do {                                                                                          \
+    if (vec)                                                                                    \
+      norm_kv_store_vec_kernel<TI, T><<<T_, 256, 0, s>>>(                                       \
+          (const TI*)qkv, qs, positions, (T*)q_out, (T*)k_cache, (T*)v_cache, slots, H, G, dk, dv, \
+          bs, num_blocks, eps, qk_unit, v_unit, coef, every, qw, kw, lsh);                      \
+    else                                                                                        \
+      norm_kv_store_kernel<TI, T><<<T_, 256, 0, s>>>(                                           \
+          (const TI*)qkv, qs, positions, (T*)q_out, (T*)k_cache, (T*)v_cache, slots, H, G, dk, dv, \
+          bs, num_blocks, eps, qk_unit, v_unit, coef, every, qw, kw);                           \
+  } while (0)
+  if (dtype == DT_F32) KGC_DISPATCH_T(out_dtype, KGC_NKV(float));
+  else KGC_DISPATCH_T(out_dtype, KGC_NKV(T));
+#undef KGC_NKV
 }
 
 void launch_qk_norm_store(int dtype, void* q_out, const void* qkv, int64_t qs,
@@ -1328,13 +1416,13 @@ void launch_window_decode(int dtype, void* out, const void* q, const void* k_cac
 }
 
 size_t window_prefill_mfma_lds(int dk, int dv) {
-  return 2 * ((size_t)PFW_BN * (dk + PFW_KPAD) + (size_t)dv * (PFW_BN + PFW_VPAD));
+  return 2 * ((size_t)PFW_BN * (((dk + 31) & ~31) + PFW_KPAD) + (size_t)dv * (PFW_BN + PFW_VPAD));
 }
 
-// the matrix-core prefill path: 16-bit activations, dk a multiple of 32 (<= 256), dv a
+// the matrix-core prefill path: 16-bit activations, dk a multiple of 8 (<= 256), dv a
 // multiple of 16 (<= 256), both tiles within 64 KB of LDS
 bool window_prefill_mfma_ok(int dtype, int dk, int dv) {
-  return (dtype == DT_BF16 || dtype == DT_F16) && dk % 32 == 0 && dk <= 256 && dv % 16 == 0 &&
+  return (dtype == DT_BF16 || dtype == DT_F16) && dk % 8 == 0 && dk <= 256 && dv % 16 == 0 &&
          dv <= 256 && window_prefill_mfma_lds(dk, dv) <= 64 * 1024;
 }
 

@@ -126,7 +126,7 @@ void launch_moe_align(const int* topk_ids, int npairs, int e0, int E_local, int 
 void launch_moe_gemm(int dtype, int bm, void* C, const void* A, const void* W,
                      const int* sorted_ids, const int* block_expert, const int* meta, int npairs,
                      int topk, int N, int K, int64_t lda, int64_t ldc, int max_mblocks,
-                     bool gather, bool scatter, int splitk, int64_t slice_stride, hipStream_t s);
+                     bool gather, bool scatter, int splitk, int64_t slice_stride, int64_t wes, int64_t wrs, hipStream_t s);
 // dense split-K decode GEMM: Cs [splitk, M, N] fp32 = A [M, K] x W [N, K]^T, XCD-mapped slices
 void launch_dense_gemm_splitk(int dtype, int bm, float* Cs, const void* A, const void* W, int M,
                               int N, int K, int64_t lda, int splitk, hipStream_t s);
@@ -288,6 +288,10 @@ struct WindowExtra {
   const float* vtab;
   int vrows;
   bool vinter;
+  // window counts chunks instead: position p sees the keys j <= p with j / window == p / window
+  bool chunked;
+  // a score without a value that joins every softmax (-infinity: none)
+  float sink;
 };
 void launch_qk_norm_store(int dtype, void* q_out, const void* qkv, int64_t qs,
                           const int64_t* positions, const float* qw, const float* kw,
@@ -368,7 +372,7 @@ void launch_latent_rope_store(int dtype, void* q_out, const void* proj, int64_t 
                               int r, int rank, hipStream_t s);
 int moe_route_sigmoid_max_experts();
 void launch_moe_route_sigmoid(float* w, int* ids, const float* scores, int64_t stride,
-                              const float* corr, int ntok, int E, int k, float scale,
+                              const float* corr, int ntok, int E, int k, float scale, bool renorm,
                               hipStream_t s);
 void launch_moe_finish(int dtype, void* out, const void* routed, const void* dense,
                        const float* w, const int* ids, const void* shared, const float* gate,
@@ -412,10 +416,12 @@ void launch_selective_scan(int dtype, void* out, int64_t os, const void* x, cons
                            const int* qsl, const int* seq_lens, const int* ctx_lens,
                            const int* slots, int P, int D, int Tp, int I, int N,
                            float out_scale, int num_slots, hipStream_t s);
-void launch_norm_kv_store(int out_dtype, const float* qkv, int64_t qs, const int64_t* positions,
-                          void* q_out, void* k_cache, void* v_cache, const int64_t* slots, int T_,
-                          int H, int G, int dk, int dv, int bs, int num_blocks, float eps,
-                          bool qk_unit, bool v_unit, float coef, int every, hipStream_t s);
+// dtype: of qkv (fp32 or out_dtype); qw / kw fp32 [dk] multiply every head's q / k (null: none)
+void launch_norm_kv_store(int dtype, int out_dtype, const void* qkv, int64_t qs,
+                          const int64_t* positions, void* q_out, void* k_cache, void* v_cache,
+                          const int64_t* slots, int T, int H, int G, int dk, int dv, int bs,
+                          int num_blocks, float eps, bool qk_unit, bool v_unit, float coef,
+                          int every, const float* qw, const float* kw, hipStream_t s);
 void launch_polynorm(int dtype, void* out, const void* z, const float* coef, int64_t rows, int F,
                      float eps, hipStream_t s);
 void launch_swiglu_clamp(int dtype, void* out, const void* x, int64_t rows, int I, float limit,
@@ -444,6 +450,49 @@ struct ResidualAdds {
 };
 void launch_residual_sum_norm(int dtype, int out_dtype, void* out, float* x, ResidualAdds adds,
                               const float* w, int rows, int W, float eps, hipStream_t s);
+// ---- hyper-connected streams, latent queries, input-scaled experts ---------------------------
+// a sublayer's result: up to two addends, each the sum of k rows per token -- of the activation
+// dtype (slices = 0), or fp32 partial sums [slices] (stride ss elements) of such rows
+struct HyperAdds {
+  const void* a[2];
+  int k[2];
+  int slices[2];
+  int64_t ss[2];
+};
+int hyper_max_streams();
+// streams of src at src + row * srow + stream * sstream; dst [rows, S, W] (may be src; null: not
+// written); mix null: the streams stay as they are
+void launch_hyper_norm(int dtype, int out_dtype, void* out, const float* src, int64_t srow,
+                       int64_t sstream, float* dst, HyperAdds ad, const float* mix,
+                       const float* ow, const float* iw, const float* w, int rows, int S, int W,
+                       float eps, hipStream_t s);
+void launch_latent_down_store(int dtype, void* cq, float* gate, const void* proj, int64_t ps,
+                              const int64_t* positions, const float* table, int table_rows,
+                              const float* qw, const float* kw, float eps, void* cache,
+                              const int64_t* slots, int64_t cache_rows, int T, int qr, int rank,
+                              int r, int gates, hipStream_t s);
+// out[t, h, n] = sum_k x[t, h, k] w[h, n, k] (token strides xs / os, head strides xh / oh; w
+// [H, N, K]); with rot, out[t, h, N ..] = its r columns (strides rs / rh) turned by the position
+struct HeadGemm {
+  void* out;
+  int64_t os, oh;
+  const void* x;
+  int64_t xs, xh;
+  const void* w;
+  int T, H, N, K;
+  const void* rot;
+  int64_t rs, rh;
+  int r;
+  const int64_t* positions;
+  const float* table;
+  int table_rows;
+};
+void launch_head_gemm(int dtype, HeadGemm a, hipStream_t s);
+void launch_expert_silu_all(int dtype, void* out, const void* x, const float* w, const int* ids,
+                            int T, int E, int k, int I, int Is, hipStream_t s);
+void launch_expert_silu_rows(int dtype, void* out, const void* x, const float* w,
+                             const int* sorted_ids, int npairs, int64_t rows, int I,
+                             hipStream_t s);
 void launch_logit_softcap(int dtype, float* out, const void* x, int64_t xs, int64_t rows, int V,
                           float cap, hipStream_t s);
 

@@ -11,7 +11,8 @@
 //                 BM rows of one expert by a MG_BN-column slice of that expert's
 //                 weight [N, K] on MFMA 16x16x32; A rows are gathered from the token
 //                 matrix (first GEMM) or read contiguously (second GEMM); the second
-//                 GEMM scatters rows back to pair order.  M-blocks run fastest in the
+//                 GEMM scatters rows back to pair order.  Experts and weight rows may lie
+//                 at any stride.  M-blocks run fastest in the
 //                 grid so the blocks sharing a weight slice run together (L2/MALL reuse).
 //   moe_combine : out[t] = sum_j w[t, j] * y[t*k + j]   (fp32 accumulation).
 #include "common.h"
@@ -203,7 +204,7 @@ __global__ __launch_bounds__(MG_THREADS, 2) void moe_gemm_kernel(
     void* __restrict__ Cv, const T* __restrict__ A, const T* __restrict__ W,
     const int* __restrict__ sorted_ids, const int* __restrict__ block_expert,
     const int* __restrict__ meta, int npairs, int topk, int N, int K, int64_t lda,
-    int64_t ldc, int64_t slice_stride, int dense_m) {
+    int64_t ldc, int64_t slice_stride, int dense_m, int64_t wes, int64_t wrs) {
   int mb, nb, z, S, e;
   if constexpr (DENSE) {
     // npairs = number of M-blocks, topk = number of K-slices (reused scalar args);
@@ -249,7 +250,7 @@ __global__ __launch_bounds__(MG_THREADS, 2) void moe_gemm_kernel(
     }
     a_ptr[i] = A + arow * lda + chunk * 8;
   }
-  const T* w_ptr = W + ((int64_t)e * N + (int64_t)nb * MG_BN + (tid >> 3)) * K + chunk * 8;
+  const T* w_ptr = W + e * wes + ((int64_t)nb * MG_BN + (tid >> 3)) * wrs + chunk * 8;
   u32x4 ra[AC], rb[4];
   auto gload = [&](int kb) {
     const int ko = kb * MG_BK;
@@ -257,7 +258,7 @@ __global__ __launch_bounds__(MG_THREADS, 2) void moe_gemm_kernel(
     for (int i = 0; i < AC; ++i) ra[i] = *reinterpret_cast<const u32x4*>(a_ptr[i] + ko);
 #pragma unroll
     for (int i = 0; i < 4; ++i)
-      rb[i] = *reinterpret_cast<const u32x4*>(w_ptr + (int64_t)32 * i * K + ko);
+      rb[i] = *reinterpret_cast<const u32x4*>(w_ptr + 32 * i * wrs + ko);
   };
   auto lstore = [&](int buf) {
 #pragma unroll
@@ -488,13 +489,14 @@ template <typename T, int BM>
 static void moe_gemm_bm(void* C, const void* A, const void* W, const int* sorted_ids,
                         const int* block_expert, const int* meta, int npairs, int topk, int N,
                         int K, int64_t lda, int64_t ldc, int max_mblocks, bool gather,
-                        bool scatter, int splitk, int64_t slice_stride, hipStream_t s) {
+                        bool scatter, int splitk, int64_t slice_stride, int64_t wes,
+                        int64_t wrs, hipStream_t s) {
   const dim3 grid(max_mblocks, N / MG_BN, splitk);
 #define MG_LAUNCH(G, S, P)                                                                   \
   moe_gemm_kernel<T, BM, G, S, P><<<grid, MG_THREADS, 0, s>>>(C, (const T*)A, (const T*)W,   \
                                                               sorted_ids, block_expert, meta, \
                                                               npairs, topk, N, K, lda, ldc,   \
-                                                              slice_stride, 0)
+                                                              slice_stride, 0, wes, wrs)
   if (splitk > 1) MG_LAUNCH(false, true, true);          // host-checked: scatter, !gather
   else if (gather && !scatter) MG_LAUNCH(true, false, false);
   else if (!gather && scatter) MG_LAUNCH(false, true, false);
@@ -507,25 +509,27 @@ template <typename T>
 static void moe_gemm_t(int bm, void* C, const void* A, const void* W, const int* sorted_ids,
                        const int* block_expert, const int* meta, int npairs, int topk, int N,
                        int K, int64_t lda, int64_t ldc, int max_mblocks, bool gather,
-                       bool scatter, int splitk, int64_t slice_stride, hipStream_t s) {
+                       bool scatter, int splitk, int64_t slice_stride, int64_t wes,
+                        int64_t wrs, hipStream_t s) {
   if (bm == 128)
     moe_gemm_bm<T, 128>(C, A, W, sorted_ids, block_expert, meta, npairs, topk, N, K, lda, ldc,
-                        max_mblocks, gather, scatter, splitk, slice_stride, s);
+                        max_mblocks, gather, scatter, splitk, slice_stride, wes, wrs, s);
   else
     moe_gemm_bm<T, 64>(C, A, W, sorted_ids, block_expert, meta, npairs, topk, N, K, lda, ldc,
-                       max_mblocks, gather, scatter, splitk, slice_stride, s);
+                       max_mblocks, gather, scatter, splitk, slice_stride, wes, wrs, s);
 }
 
 void launch_moe_gemm(int dtype, int bm, void* C, const void* A, const void* W,
                      const int* sorted_ids, const int* block_expert, const int* meta, int npairs,
                      int topk, int N, int K, int64_t lda, int64_t ldc, int max_mblocks,
-                     bool gather, bool scatter, int splitk, int64_t slice_stride, hipStream_t s) {
+                     bool gather, bool scatter, int splitk, int64_t slice_stride, int64_t wes,
+                        int64_t wrs, hipStream_t s) {
   if (dtype == DT_BF16)
     moe_gemm_t<bf16>(bm, C, A, W, sorted_ids, block_expert, meta, npairs, topk, N, K, lda, ldc,
-                     max_mblocks, gather, scatter, splitk, slice_stride, s);
+                     max_mblocks, gather, scatter, splitk, slice_stride, wes, wrs, s);
   else
     moe_gemm_t<f16>(bm, C, A, W, sorted_ids, block_expert, meta, npairs, topk, N, K, lda, ldc,
-                    max_mblocks, gather, scatter, splitk, slice_stride, s);
+                    max_mblocks, gather, scatter, splitk, slice_stride, wes, wrs, s);
 }
 
 void launch_dense_gemm_splitk(int dtype, int bm, float* Cs, const void* A, const void* W, int M,
@@ -535,7 +539,7 @@ void launch_dense_gemm_splitk(int dtype, int bm, float* Cs, const void* A, const
   const int64_t ss = (int64_t)M * N;
 #define DG_LAUNCH(T, BMV)                                                                     \
   moe_gemm_kernel<T, BMV, false, false, true, true><<<grid, MG_THREADS, 0, s>>>(             \
-      Cs, (const T*)A, (const T*)W, nullptr, nullptr, nullptr, MB, splitk, N, K, lda, N, ss, M)
+      Cs, (const T*)A, (const T*)W, nullptr, nullptr, nullptr, MB, splitk, N, K, lda, N, ss, M, 0, K)
   if (dtype == DT_BF16) {
     if (bm == 128) DG_LAUNCH(bf16, 128);
     else DG_LAUNCH(bf16, 64);
@@ -626,13 +630,15 @@ namespace {
 
 // One wave per token.  scores fp32 [T, stride]: sigmoid router scores in the first E
 // columns.  k rounds of a wave-wide arg-max over score + correction (the lowest index
-// wins among equals); weights = the chosen scores / (their sum + 1e-20) * scale.
+// wins among equals; corr null: over the score itself); weights = the chosen scores
+// (renorm: / (their sum + 1e-20)) * scale.
 constexpr int RS_MAX_PER_LANE = 16;          // E <= 1024
 
 template <int RS_PER_LANE>                   // experts per lane: E <= 64 * RS_PER_LANE
 __global__ __launch_bounds__(256) void moe_route_sigmoid_kernel(
     float* __restrict__ w, int* __restrict__ ids, const float* __restrict__ scores,
-    int64_t stride, const float* __restrict__ corr, int ntok, int E, int k, float scale) {
+    int64_t stride, const float* __restrict__ corr, int ntok, int E, int k, float scale,
+    bool renorm) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (t >= ntok) return;
   const float* sr = scores + (int64_t)t * stride;
@@ -641,7 +647,7 @@ __global__ __launch_bounds__(256) void moe_route_sigmoid_kernel(
   for (int u = 0; u < RS_PER_LANE; ++u) {
     const int e = lane + 64 * u;
     sc[u] = e < E ? sr[e] : 0.f;
-    ch[u] = e < E ? sc[u] + corr[e] : -INFINITY;
+    ch[u] = e < E ? sc[u] + (corr != nullptr ? corr[e] : 0.f) : -INFINITY;
   }
   float mine = 0.f, sum = 0.f;          // lane j keeps the j-th chosen score
   int mine_id = 0;
@@ -676,7 +682,7 @@ __global__ __launch_bounds__(256) void moe_route_sigmoid_kernel(
     }
   }
   if (lane < k) {
-    w[(int64_t)t * k + lane] = mine / (sum + 1e-20f) * scale;
+    w[(int64_t)t * k + lane] = (renorm ? mine / (sum + 1e-20f) : mine) * scale;
     ids[(int64_t)t * k + lane] = mine_id;
   }
 }
@@ -711,17 +717,17 @@ __global__ __launch_bounds__(256) void moe_finish_kernel(
 int moe_route_sigmoid_max_experts() { return 64 * RS_MAX_PER_LANE; }
 
 void launch_moe_route_sigmoid(float* w, int* ids, const float* scores, int64_t stride,
-                              const float* corr, int ntok, int E, int k, float scale,
+                              const float* corr, int ntok, int E, int k, float scale, bool renorm,
                               hipStream_t s) {
   if (ntok <= 0) return;
   const int grid = (ntok + 3) / 4;
   if (E <= 64)
-    moe_route_sigmoid_kernel<1><<<grid, 256, 0, s>>>(w, ids, scores, stride, corr, ntok, E, k, scale);
+    moe_route_sigmoid_kernel<1><<<grid, 256, 0, s>>>(w, ids, scores, stride, corr, ntok, E, k, scale, renorm);
   else if (E <= 256)
-    moe_route_sigmoid_kernel<4><<<grid, 256, 0, s>>>(w, ids, scores, stride, corr, ntok, E, k, scale);
+    moe_route_sigmoid_kernel<4><<<grid, 256, 0, s>>>(w, ids, scores, stride, corr, ntok, E, k, scale, renorm);
   else
     moe_route_sigmoid_kernel<RS_MAX_PER_LANE><<<grid, 256, 0, s>>>(w, ids, scores, stride, corr,
-                                                                   ntok, E, k, scale);
+                                                                   ntok, E, k, scale, renorm);
 }
 
 void launch_moe_finish(int dtype, void* out, const void* routed, const void* dense,
