@@ -445,7 +445,7 @@ class InputScaledExperts(nn.Module):
         self.down_proj = ReplicatedLinear(E * I + Is, hidden, dtype=dtype, device=device)
         self.router = nn.Parameter(torch.zeros(E, hidden, dtype=dtype, device=device),
                                    requires_grad=False)
-        self.native = (torch.device(device).type == "cuda" and dtype != torch.float32 and E <= 256 and
+        self.native = (self.router.is_cuda and dtype != torch.float32 and E <= 256 and
                        ops.moe_supported(2 * I, hidden) and ops.moe_supported(hidden, I) and
                        Is % 8 == 0)
 

@@ -141,12 +141,15 @@ def gated(h, wts, p):
 
 def route(h, router, top):
     """-> ids [T, top] of the largest scores (the lower index first among equals), scores
-    [T, top], and each token's gap between the last chosen and the first unchosen score."""
-    s = sigmoid(h @ router.T)
-    order = np.argsort(-s, axis=-1, kind="stable")
-    ranked = np.take_along_axis(s, order, -1)
-    gap = ranked[:, top - 1] - ranked[:, top] if top < s.shape[1] else np.full(len(s), np.inf)
-    return order[:, :top], ranked[:, :top], gap
+    [T, top], and how close each token's decision was: the gap between the last chosen and the
+    first unchosen logit over the largest logit."""
+    z = h @ router.T
+    order = np.argsort(-z, axis=-1, kind="stable")
+    ranked = np.take_along_axis(z, order, -1)
+    gap = np.full(len(z), np.inf)
+    if top < z.shape[1]:
+        gap = (ranked[:, top - 1] - ranked[:, top]) / np.abs(z).max(-1)
+    return order[:, :top], sigmoid(ranked[:, :top]), gap
 
 
 def experts(h, wts, P, mlp, gaps=None):
@@ -185,3 +188,78 @@ def forward(cfg, wts, tokens, taps=None, gaps=None):
         if taps is not None:
             taps.append(X.sum(0))
     return (rms(X.sum(0), eps) * (1.0 + wts["final.norm"])) @ wts["head"].T * cfg["logit_scale"]
+
+
+# ------------------------------------------------------------------ random checkpoints
+def tensor_shapes(cfg):
+    """Checkpoint names -> shapes."""
+    W, S = cfg["width"], cfg["streams"]
+    out = {"embed": (cfg["vocab"], W), "head": (cfg["vocab"], W), "final.norm": (W,)}
+    for i, lay in enumerate(cfg["layers"]):
+        L, m, f = "l%d." % i, lay["mixer"], lay.get("mlp")
+        for n in ("1", "2") if f else ("1",):
+            out.update({L + "norm" + n: (W,), L + "hc%s.in" % n: (S,), L + "hc%s.out" % n: (S,),
+                        L + "hc%s.mix" % n: (S, S)})
+        P, H = L + "mix.", m["heads"]
+        if lay["type"] == "attention":
+            G, d, dv = m["kv_heads"], m["dim"], m["vdim"]
+            out.update({P + "q": (H * d, W), P + "k": (G * d, W), P + "v": (G * dv, W),
+                        P + "q.norm": (d,), P + "k.norm": (d,), P + "o": (W, H * dv)})
+        else:
+            d, r, dv, rank, qr = m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"], m["q_rank"]
+            out.update({P + "dq": (qr, W), P + "dq.norm": (qr,), P + "uq": (H * (d + r), qr),
+                        P + "dkv": (rank + r, W), P + "dkv.norm": (rank,), P + "uk": (H * d, rank),
+                        P + "uv": (H * dv, rank), P + "g": (H, W), P + "o": (W, H * dv)})
+        if f:
+            P, E = L + "mlp.", f["router"]["experts"]
+            out[P + "router"] = (E, W)
+            ffs = [("e%d." % e, f["expert"]["ff"]) for e in range(E)]
+            if f.get("shared"):
+                ffs.append(("shared.", f["shared"]["ff"]))
+            for n, ff in ffs:
+                out.update({P + n + "gate": (ff, W), P + n + "up": (ff, W), P + n + "down": (W, ff)})
+    return out
+
+
+def bf16(a):
+    """Round-to-nearest-even bf16 values, as float64."""
+    b = np.ascontiguousarray(a, dtype=np.float32).view(np.uint32)
+    b = (b + 0x7FFF + ((b >> 16) & 1)) & np.uint32(0xFFFF0000)
+    return b.view(np.float32).astype(np.float64)
+
+
+def random_weights(cfg, seed):
+    """bf16-valued random weights.  The routers decide on a code of the token: the first
+    columns of the stream (as many as the largest router has outputs) hold a permutation of
+    spaced levels that no sublayer writes to, so no routing decision is close and rounding cannot
+    turn one; all other mechanisms see random data."""
+    rng = np.random.default_rng(seed)
+    S, V = cfg["streams"], cfg["vocab"]
+    C = max([lay["mlp"]["router"]["experts"] for lay in cfg["layers"] if lay.get("mlp")] or [0])
+    wts = {}
+    for name, shape in tensor_shapes(cfg).items():
+        leaf = name.split(".", 1)[-1]
+        z = rng.normal(size=shape)
+        if leaf in ("hc1.in", "hc2.in"):
+            w = rng.uniform(0.4, 1.6, shape) / S
+        elif leaf in ("hc1.out", "hc2.out"):
+            w = 1.0 + 0.4 * z
+        elif leaf in ("hc1.mix", "hc2.mix"):
+            w = 0.75 * np.eye(S) + rng.uniform(0.0, 0.5, shape) / S
+        elif leaf in ("norm1", "norm2") or name == "final.norm":
+            w = 0.2 * z
+            w[:C] = 0.0
+        elif len(shape) == 1:
+            w = 1.0 + 0.3 * z
+        elif name == "embed":
+            w = z
+            w[:, :C] = np.stack([rng.permutation(np.linspace(-2.0, 2.0, C)) for _ in range(V)]) if C else 0
+        elif leaf.endswith("router"):
+            w = np.zeros(shape)
+            w[np.arange(shape[0]), rng.permutation(C)[: shape[0]]] = 2.5
+        else:
+            w = 1.3 * z / np.sqrt(shape[1])
+            if C and shape[0] == cfg["width"] and (leaf.endswith(".o") or leaf.endswith("down")):
+                w[:C] = 0.0
+        wts[name] = bf16(w)
+    return wts
