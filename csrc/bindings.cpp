@@ -2162,6 +2162,30 @@ void moe_route_sigmoid(Tensor w, Tensor ids, Tensor scores, std::optional<Tensor
                                 (int)E, (int)k, (float)scale, renorm, stream());
 }
 
+void moe_gate_sigmoid(Tensor w, Tensor ids, Tensor x, Tensor wg, std::optional<Tensor> correction,
+                      double scale, bool renorm) {
+  check_gpu(x, "x");
+  check_f32(w, "w");
+  c10::hip::HIPGuardMasqueradingAsCUDA g(x.device());
+  TORCH_CHECK(x.dim() == 2 && x.stride(1) == 1 && x.stride(0) % 8 == 0 && x.size(1) % 8 == 0 &&
+              (x.scalar_type() == at::kBFloat16 || x.scalar_type() == at::kHalf) &&
+              reinterpret_cast<uintptr_t>(x.data_ptr()) % 16 == 0,
+              "kgc.moe_gate_sigmoid: x [T, H], 16-byte rows");
+  const int64_t T = x.size(0), H = x.size(1), E = wg.size(0);
+  TORCH_CHECK(wg.is_cuda() && wg.dim() == 2 && wg.is_contiguous() && wg.size(1) == H &&
+              wg.scalar_type() == x.scalar_type() && wg.device() == x.device() &&
+              reinterpret_cast<uintptr_t>(wg.data_ptr()) % 16 == 0, "kgc.moe_gate_sigmoid: wg [E, H]");
+  TORCH_CHECK(w.dim() == 2 && w.size(0) == T && w.is_contiguous() && w.device() == x.device(),
+              "kgc.moe_gate_sigmoid: w [T, k]");
+  const int64_t k = w.size(1);
+  TORCH_CHECK(E >= 1 && E <= 64 && k >= 1 && k <= E && k <= 16, "kgc.moe_gate_sigmoid: experts / top");
+  TORCH_CHECK(ids.is_cuda() && ids.scalar_type() == at::kInt && ids.is_contiguous() &&
+              ids.numel() == T * k && ids.device() == x.device(), "kgc.moe_gate_sigmoid: ids int32 [T, k]");
+  kgc::launch_moe_gate_sigmoid(dt_code(x), w.data_ptr<float>(), ids.data_ptr<int>(), x.data_ptr(),
+                               x.stride(0), wg.data_ptr(), f32_opt(correction, E, "correction"),
+                               (int)T, (int)H, (int)E, (int)k, (float)scale, renorm, stream());
+}
+
 void moe_finish(Tensor out, std::optional<Tensor> routed, std::optional<Tensor> dense,
                 std::optional<Tensor> topk_w, std::optional<Tensor> topk_ids,
                 std::optional<Tensor> shared, std::optional<Tensor> gate) {
@@ -2572,6 +2596,8 @@ TORCH_LIBRARY(kgc, m) {
         "Tensor table, int col0, Tensor side_w, Tensor? w, float mult, float eps) -> bool");
   m.def("moe_route_sigmoid(Tensor(a!) w, Tensor(b!) ids, Tensor scores, Tensor? correction, float scale, "
         "bool renorm=True) -> ()");
+  m.def("moe_gate_sigmoid(Tensor(a!) w, Tensor(b!) ids, Tensor x, Tensor wg, Tensor? correction, "
+        "float scale, bool renorm) -> ()");
   m.def("moe_finish(Tensor(a!) out, Tensor? routed, Tensor? dense, Tensor? topk_w, Tensor? topk_ids, "
         "Tensor? shared, Tensor? gate) -> ()");
   m.def("residual_group_norm(Tensor(a!) out, Tensor(b!) x, Tensor? y, Tensor w, int groups, float eps) -> ()");
@@ -2737,6 +2763,7 @@ TORCH_LIBRARY_IMPL(kgc, CUDA, m) {
   m.impl("side_gate", &side_gate);
   m.impl("side_input_rows", &side_input_rows);
   m.impl("moe_route_sigmoid", &moe_route_sigmoid);
+  m.impl("moe_gate_sigmoid", &moe_gate_sigmoid);
   m.impl("moe_finish", &moe_finish);
   m.impl("rms_norm", &rms_norm);
   m.impl("layer_norm", &layer_norm);

@@ -664,8 +664,10 @@ __global__ __launch_bounds__(256, KSM <= 4 ? 3 : 2) void window_prefill_mfma_ker
   const int kp = (dk + 31) & ~31;                      // key rows padded with zeros in LDS
   const int kst = kp + PFW_KPAD, vst = PFW_BN + PFW_VPAD;
   T* Vt = Ks + PFW_BN * kst;                           // [dv][64 + 8]
-  const int item = blockIdx.x / (blk_rows / PFW_BM), sub = blockIdx.x % (blk_rows / PFW_BM);
-  const int seq = work_seq[item], h = blockIdx.y, g = h / (H / G);
+  // heads run fastest: workgroups are dealt round-robin over the XCDs, so every XCD sees all row
+  // blocks of its heads (with chunks the cost of a block depends on its place)
+  const int item = blockIdx.y / (blk_rows / PFW_BM), sub = blockIdx.y % (blk_rows / PFW_BM);
+  const int seq = work_seq[item], h = blockIdx.x, g = h / (H / G);
   const int q0 = qsl[seq], qlen = qsl[seq + 1] - q0, ctx0 = seq_lens[seq] - qlen;
   const int r0 = work_blk[item] * blk_rows + sub * PFW_BM;
   if (r0 >= qlen || ctx0 < 0) return;
@@ -1433,7 +1435,7 @@ static void prefill_dispatch(T* out, const T* q, const T* kc, const T* vc, const
                              int H, int G, int dk, int dv, int krs, int vrs, int bs, int num_blocks,
                              float scale, int window, int keep_first, const float* gate,
                              WindowExtra ex, hipStream_t s) {
-  const dim3 grid(n_work * (blk_rows / PFW_BM), H);
+  const dim3 grid(H, n_work * (blk_rows / PFW_BM));
   const size_t lds = window_prefill_mfma_lds(dk, dv);
   const bool ext = ex.pool > 0 || ex.vtab != nullptr;
 #define KGC_PF_E(K, D, E)                                                                     \

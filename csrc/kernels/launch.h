@@ -374,6 +374,10 @@ int moe_route_sigmoid_max_experts();
 void launch_moe_route_sigmoid(float* w, int* ids, const float* scores, int64_t stride,
                               const float* corr, int ntok, int E, int k, float scale, bool renorm,
                               hipStream_t s);
+// 16-bit dtype, E <= 64, k <= 16, H % 8 == 0
+void launch_moe_gate_sigmoid(int dtype, float* w, int* ids, const void* x, int64_t xs,
+                             const void* wg, const float* corr, int ntok, int H, int E, int k,
+                             float scale, bool renorm, hipStream_t s);
 void launch_moe_finish(int dtype, void* out, const void* routed, const void* dense,
                        const float* w, const int* ids, const void* shared, const float* gate,
                        int64_t gs, int ntok, int E, int k, int W, hipStream_t s);

@@ -687,6 +687,95 @@ __global__ __launch_bounds__(256) void moe_route_sigmoid_kernel(
   }
 }
 
+// The router's product and the choice in one launch, for 16-bit activations: sigmoid(x . wg^T),
+// then as moe_route_sigmoid_kernel.  A workgroup takes 16 tokens; its four waves split the columns
+// (MFMA, A rows = experts, B columns = tokens, fp32 accumulation), the partial products meet in
+// LDS, and 16 lanes choose for each token.  E <= 16 NT, k <= 16, H % 8 == 0.
+template <typename T, int NT>
+__global__ __launch_bounds__(256) void moe_gate_sigmoid_kernel(
+    float* __restrict__ w, int* __restrict__ ids, const T* __restrict__ x, int64_t xs,
+    const T* __restrict__ wg, const float* __restrict__ corr, int ntok, int H, int E, int k,
+    float scale, bool renorm) {
+  constexpr int ES = NT * 16 + 1;
+  __shared__ float part[4][16][ES];
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r16 = lane & 15, qd = lane >> 4;
+  const int t0 = blockIdx.x * 16;
+  const T* xr = x + (int64_t)min(t0 + r16, ntok - 1) * xs + 8 * qd;
+  const T* wr[NT];
+#pragma unroll
+  for (int j = 0; j < NT; ++j) wr[j] = wg + (int64_t)min(16 * j + r16, E - 1) * H + 8 * qd;
+  f32x4 acc[NT];
+#pragma unroll
+  for (int j = 0; j < NT; ++j) acc[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+  const int steps = (H + 31) >> 5;
+  constexpr int U = NT == 1 ? 8 : NT == 2 ? 4 : 2;            // steps whose loads are in flight
+  for (int s0 = wave; s0 < steps; s0 += 4 * U) {
+    Pack8<T> xf[U], wf[U][NT];
+#pragma unroll
+    for (int q = 0; q < U; ++q) {
+      const int c = 32 * (s0 + 4 * q);
+      const bool ok = c + 8 * qd < H;
+      xf[q].u = ok ? *reinterpret_cast<const u32x4*>(xr + c) : u32x4{0u, 0u, 0u, 0u};
+#pragma unroll
+      for (int j = 0; j < NT; ++j)
+        wf[q][j].u = ok ? *reinterpret_cast<const u32x4*>(wr[j] + c) : u32x4{0u, 0u, 0u, 0u};
+    }
+#pragma unroll
+    for (int q = 0; q < U; ++q)
+#pragma unroll
+      for (int j = 0; j < NT; ++j) acc[j] = mfma16x16x32(wf[q][j].v, xf[q].v, acc[j]);
+  }
+#pragma unroll
+  for (int j = 0; j < NT; ++j)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) part[wave][r16][16 * j + 4 * qd + i] = acc[j][i];
+  __syncthreads();
+  const int tl = threadIdx.x >> 4, l = threadIdx.x & 15, t = t0 + tl;
+  float sc[NT], ch[NT];
+#pragma unroll
+  for (int j = 0; j < NT; ++j) {
+    const int e = 16 * j + l;
+    const float z = (part[0][tl][e] + part[1][tl][e]) + (part[2][tl][e] + part[3][tl][e]);
+    sc[j] = 1.f / (1.f + expf(-z));
+    ch[j] = e < E ? sc[j] + (corr != nullptr ? corr[e] : 0.f) : -INFINITY;
+  }
+  float mine = 0.f, sum = 0.f;
+  int mine_id = 0;
+  for (int n = 0; n < k; ++n) {
+    float best = -INFINITY, bs = 0.f;
+    int bi = 0x7fffffff;
+#pragma unroll
+    for (int j = 0; j < NT; ++j)
+      if (ch[j] > best) {                 // strict: the lowest index of a lane's equals
+        best = ch[j];
+        bi = 16 * j + l;
+        bs = sc[j];
+      }
+#pragma unroll
+    for (int o = 8; o > 0; o >>= 1) {     // within the token's 16 lanes
+      const float ob = __shfl_xor(best, o, 64), os = __shfl_xor(bs, o, 64);
+      const int oi = __shfl_xor(bi, o, 64);
+      if (ob > best || (ob == best && oi < bi)) {
+        best = ob;
+        bi = oi;
+        bs = os;
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < NT; ++j)
+      if (16 * j + l == bi) ch[j] = -INFINITY;
+    sum += bs;
+    if (n == l) {
+      mine = bs;
+      mine_id = bi < E ? bi : 0;
+    }
+  }
+  if (t < ntok && l < k) {
+    w[(int64_t)t * k + l] = (renorm ? mine / (sum + 1e-20f) : mine) * scale;
+    ids[(int64_t)t * k + l] = mine_id;
+  }
+}
+
 // out[t] = routed[t] (already combined), or sum_j w[t, j] * dense[ids[t, j], t];
 // + gate[t * gs] * shared[t] when a shared expert is given.  fp32 sums.
 template <typename T>
@@ -728,6 +817,25 @@ void launch_moe_route_sigmoid(float* w, int* ids, const float* scores, int64_t s
   else
     moe_route_sigmoid_kernel<RS_MAX_PER_LANE><<<grid, 256, 0, s>>>(w, ids, scores, stride, corr,
                                                                    ntok, E, k, scale, renorm);
+}
+
+void launch_moe_gate_sigmoid(int dtype, float* w, int* ids, const void* x, int64_t xs,
+                             const void* wg, const float* corr, int ntok, int H, int E, int k,
+                             float scale, bool renorm, hipStream_t s) {
+  if (ntok <= 0) return;
+  const int grid = (ntok + 15) / 16;
+#define KGC_MGS(TT, N)                                                                       \
+  moe_gate_sigmoid_kernel<TT, N><<<grid, 256, 0, s>>>(w, ids, (const TT*)x, xs, (const TT*)wg, \
+                                                      corr, ntok, H, E, k, scale, renorm)
+#define KGC_MGS_E(TT)                \
+  do {                               \
+    if (E <= 16) KGC_MGS(TT, 1);     \
+    else if (E <= 32) KGC_MGS(TT, 2); \
+    else KGC_MGS(TT, 4);             \
+  } while (0)
+  if (dtype == DT_BF16) KGC_MGS_E(bf16); else KGC_MGS_E(f16);
+#undef KGC_MGS_E
+#undef KGC_MGS
 }
 
 void launch_moe_finish(int dtype, void* out, const void* routed, const void* dense,

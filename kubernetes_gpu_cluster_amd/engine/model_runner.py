@@ -786,7 +786,10 @@ class ModelRunner:
                              silu_shapes=getattr(self.model, "silu_shapes", lambda: set())(),
                              tail_shapes=getattr(self.model, "tail_shapes", lambda: set())(),
                              qkv_dims=getattr(self.model, "qkv_dims", lambda: {})(),
-                             rs_shapes=getattr(self.model, "_rs_w", None) is not None)
+                             rs_shapes=getattr(self.model, "_rs_w", None) is not None,
+                             sum_shapes=getattr(self.model, "sum_shapes", lambda: set())(),
+                             sum_consumer=getattr(self.model, "sum_consumer", None),
+                             stream_shapes=getattr(self.model, "stream_shapes", lambda: set())())
         whole = self.model.first and self.model.last
         if (not self.use_graphs or not (whole or self.pp_link is not None)
                 or not getattr(self.model, "graph_safe", True)):

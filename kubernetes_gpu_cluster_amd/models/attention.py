@@ -15,6 +15,7 @@ import torch
 import torch.nn as nn
 
 from .. import ops
+from ..ops.gemm import linear_slices
 
 
 @dataclasses.dataclass
@@ -203,7 +204,8 @@ class LatentQueryAttention(nn.Module):
       result W_o (W_uv per head)
 
     Both per-head matrices run as ``head_gemm``; the first one's launch also rotates the
-    queries, and the gate rides in the attention kernels' epilogue."""
+    queries, and the gate rides in the attention kernels' epilogue.  The result may come as
+    K-slices (``linear_slices``) for a consumer that sums them."""
 
     def __init__(self, hidden: int, spec, eps: float, dtype, device):
         super().__init__()
@@ -253,7 +255,7 @@ class LatentQueryAttention(nn.Module):
                                  chunked=bool(w and w.chunked), sink=sp.sink)
         y = torch.empty(T, H, dv, dtype=h.dtype, device=h.device)
         ops.head_gemm(o.view(T, H, rank), self.w_uv, y)
-        return self.o_proj(y.view(T, H * dv))
+        return linear_slices(y.view(T, H * dv), self.o_proj.weight)
 
 
 class AttentionCore(nn.Module):

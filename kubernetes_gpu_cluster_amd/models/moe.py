@@ -28,6 +28,7 @@ import torch.nn as nn
 import torch.nn.functional as F
 
 from .. import ops
+from ..ops.gemm import linear_slices
 from ..parallel import comm
 from ..parallel.layers import ReplicatedLinear
 from ..parallel.state import get_state
@@ -431,9 +432,13 @@ class InputScaledExperts(nn.Module):
     * grouped: the MFMA GEMM over expert-sorted rows (16-bit activations, ff % 64 == 0,
       hidden % 128 == 0), the shared expert as a dense feed-forward beside it.
 
-    Returns the addends [(rows, rows per token)] of the result, which the consumer sums."""
+    Returns the addends [(rows or K-slices, rows per token)] of the result, which the consumer
+    sums."""
 
-    DENSE_MAX_T = 128          # tokens up to which a step's GEMMs are bound by the weights
+    DENSE_MAX_T = 256          # tokens up to which a step's GEMMs are bound by the weights
+    # what the grouped form costs beside its weights (sorting, short launches) in bytes of weight
+    # stream, and how much slower its kernels stream
+    GROUPED_EXTRA, GROUPED_RATE = 200e6, 1.7
 
     def __init__(self, hidden: int, spec, dtype, device):
         super().__init__()
@@ -459,11 +464,16 @@ class InputScaledExperts(nn.Module):
         return self.down_proj.weight.data.narrow(1, e * I, I if e < E else Is)
 
     def route(self, x: torch.Tensor) -> tuple:
-        scores = ops.gate_proj(x, self.router, None, ops.GATE_SIGMOID)      # fp32 [T, E]
-        return ops.moe_route_sigmoid(scores, None, self.spec.top, 1.0, False)
+        return ops.moe_gate_sigmoid(x, self.router, None, self.spec.top, 1.0, False)
 
     def dense_step(self, T: int) -> bool:
-        return not self.native or (T <= self.DENSE_MAX_T and T * self.spec.top >= self.spec.experts)
+        """Which form a step of T tokens takes: by the bytes either one streams."""
+        if not self.native:
+            return True
+        sp, per = self.spec, 3 * self.router.shape[1] * self.router.element_size()
+        touched = min(sp.experts, T * sp.top)
+        grouped = self.GROUPED_RATE * per * (touched * sp.ff + sp.shared_ff) + self.GROUPED_EXTRA
+        return T <= self.DENSE_MAX_T and per * (sp.experts * sp.ff + sp.shared_ff) <= grouped
 
     def forward(self, x: torch.Tensor) -> list:
         sp = self.spec
@@ -471,7 +481,7 @@ class InputScaledExperts(nn.Module):
         topk_w, topk_ids = self.route(x)
         if self.dense_step(T):
             a = ops.expert_silu_all(self.in_proj(x), topk_w, topk_ids, E, I, Is)
-            return [(self.down_proj(a), 1)]
+            return [(linear_slices(a, self.down_proj.weight), 1)]
         w_in = self.in_proj.weight[: E * 2 * I].view(E, 2 * I, x.shape[1])
         w_down = self.down_proj.weight[:, : E * I].view(x.shape[1], E, I).transpose(0, 1)
         adds = [(ops.grouped_experts_scaled(x, w_in, w_down, topk_w, topk_ids), sp.top)]

@@ -20,9 +20,9 @@ Kernel sequence per layer (ops/__init__.py, "Ratizen-style decoders"):
   attention:         q | k | v GEMM -> norm_kv_store -> window_attention -> output GEMM
   latent_attention:  merged GEMM -> latent_down_store -> query GEMM -> head_gemm (with the
                      rotation) -> window_attention (gate in its epilogue) -> head_gemm -> GEMM
-  -> hyper_norm -> gate_proj -> moe_route_sigmoid -> all experts as one GEMM pair around
-  expert_silu_all (decode sizes), or the grouped expert GEMMs beside the shared expert's; a
-  token's expert rows are summed by the next hyper_norm.
+  -> hyper_norm -> moe_gate_sigmoid -> all experts as one GEMM pair around expert_silu_all
+  (decode sizes), or the grouped expert GEMMs beside the shared expert's; K-slices of the
+  projections and a token's expert rows are summed by the next hyper_norm.
 One GPU per replica (TP = PP = 1).
 """
 from __future__ import annotations
@@ -34,6 +34,7 @@ import torch
 import torch.nn as nn
 
 from .. import ops
+from ..ops.gemm import linear_slices
 from ..parallel.layers import ParallelLMHead, ReplicatedLinear, VocabParallelEmbedding
 from ..parallel.state import get_state
 from .attention import AttentionCore, ForwardContext, LatentQueryAttention
@@ -47,7 +48,8 @@ def _f32(shape, device, fill=0.0):
 
 
 class CoreAttention(nn.Module):
-    """A mixer that is one attention core between its own projections."""
+    """A mixer that is one attention core between its own projections; the result may come as
+    K-slices (``linear_slices``)."""
 
     def __init__(self, hidden: int, spec, eps: float, dtype, device):
         super().__init__()
@@ -65,7 +67,7 @@ class CoreAttention(nn.Module):
                 cache_idx: int) -> torch.Tensor:
         o = torch.empty(h.shape[0], self.core.n_out, dtype=h.dtype, device=h.device)
         self.core(self.qkv_proj(h), 0, positions, ctx, cache_idx, o)
-        return self.o_proj(o)
+        return linear_slices(o, self.o_proj.weight)
 
 
 class HyperConnection(nn.Module):
@@ -120,6 +122,24 @@ class RatizenForCausalLM(nn.Module):
 
     def cache_layout(self) -> list:
         return [l.mix.cache_shape() for l in self.layers]
+
+    def sum_shapes(self) -> set:
+        """(N, K) of the projections whose results ``hyper_norm`` sums."""
+        ws = [l.mix.o_proj.weight for l in self.layers]
+        ws += [l.mlp.down_proj.weight for l in self.layers if l.mlp is not None]
+        return {tuple(w.shape) for w in ws}
+
+    def stream_shapes(self) -> set:
+        """(N, K) of all other projections."""
+        return {tuple(p.shape) for n, p in self.named_parameters()
+                if p.dim() == 2 and n.endswith("proj.weight")} - self.sum_shapes()
+
+    def sum_consumer(self, M: int, N: int):
+        """A ``hyper_norm`` over scratch rows, for timing a projection with what follows it."""
+        hc, dev = self.layers[0].hc1, self.final_norm.device
+        X = torch.zeros(M, self.cfg.streams, N, dtype=torch.float32, device=dev)
+        return lambda y: ops.hyper_norm(X, X, [(y, 1)], hc.mix, hc.w_out, hc.w_in, hc.norm,
+                                        self.cfg.rms_eps, self.dtype)
 
     def prepare(self, max_pos: int, max_tokens: int, device) -> None:
         """Rotary tables for ``max_pos`` positions and the step buffers for ``max_tokens`` rows

@@ -927,6 +927,22 @@ def moe_route_sigmoid(scores: torch.Tensor, correction: Optional[torch.Tensor], 
     return w, ids
 
 
+def moe_gate_sigmoid(x: torch.Tensor, wg: torch.Tensor, correction: Optional[torch.Tensor],
+                     k: int, scale: float, renormalize: bool = True):
+    """``moe_route_sigmoid`` of sigmoid(x . wg^T) (fp32), x [T, H], wg [E, H]: one launch for 16-bit
+    activations, E <= 64, k <= 16 and H % 8 == 0, ``gate_proj`` and the routing kernel otherwise."""
+    E = wg.shape[0]
+    if (not _gpu(x) or x.dtype == torch.float32 or E > 64 or k > 16 or x.shape[1] % 8
+            or x.stride(1) != 1 or x.stride(0) % 8):
+        return moe_route_sigmoid(gate_proj(x, wg, None, GATE_SIGMOID), correction, k, scale,
+                                 renormalize)
+    T = x.shape[0]
+    w = torch.empty(T, k, dtype=torch.float32, device=x.device)
+    ids = torch.empty(T, k, dtype=torch.int32, device=x.device)
+    _k().moe_gate_sigmoid(w, ids, x, wg, correction, float(scale), renormalize)
+    return w, ids
+
+
 def grouped_experts(x: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor,
                     topk_w: torch.Tensor, topk_ids: torch.Tensor, act,
                     all_local: bool = True) -> torch.Tensor:

@@ -56,7 +56,9 @@ _enabled = os.environ.get("KGC_SKINNY_GEMM", "1") != "0"
 # K9m mid-batch decode GEMM (csrc/kernels/gemm_decode.hip), M in (SKINNY_MAX_M, DG_MAX_M]:
 # (M, N, K, kind) -> (cfg, S) where it measured faster than hipBLASLt (+ the same consumer).
 # kind: "plain" (qkv / lm_head / any linear), "silu" (merged gate_up -> silu_mul),
-# "tail" (o / down -> residual add + RMSNorm).  S > 1: fp32 K-slices summed by the consumer.
+# "tail" (o / down -> residual add + RMSNorm), "sum" (any linear whose consumer adds rows or
+# K-slices itself: hyper-connected streams; also tried at M <= SKINNY_MAX_M, as "plain" is for
+# the shapes a model names).  S > 1: fp32 K-slices summed by the consumer.
 DG_MAX_M = 512
 _plan_dg: dict[tuple[int, int, int, str], tuple[int, int]] = {}
 _dg_enabled = os.environ.get("KGC_DGEMM", "1") != "0"
@@ -210,6 +212,17 @@ def linear_qkv(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
     if p is not None:
         cfg, S = p
         return dgemm(x, w, cfg, S)
+    return linear(x, w)
+
+
+def linear_slices(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """x W^T for a consumer that adds K-slices itself (``ops.hyper_norm``): [M, N] in x's dtype,
+    or fp32 slices [S, M, N] where the plan runs K9m split-K at this (M, N, K)."""
+    if x.dtype != torch.float32:
+        p = _dg_plan(x, w, "sum")
+        if p is not None:
+            cfg, S = p
+            return dgemm(x, w, cfg, S)
     return linear(x, w)
 
 
@@ -490,7 +503,7 @@ def save_dg_table(path: str, res: dict, meta: dict) -> int:
     import json
     ent = []
     for key, v in sorted(res.items()):
-        if len(key) != 4 or key[3] not in ("plain", "silu", "tail", "qkv"):
+        if len(key) != 4 or key[3] not in ("plain", "silu", "tail", "qkv", "sum"):
             continue
         M, N, K, kind = key
         chosen, lib_us, best_us, best = v
@@ -614,7 +627,8 @@ def _time_graphed(body, reps: int) -> float:
 @torch.inference_mode()
 def tune_skinny(weights: Iterable[torch.Tensor], ms: Iterable[int], margin: float = 0.97,
                 reps: int = 3, norm_shapes=(), norm_max_m: int = 16, silu_shapes=(),
-                tail_shapes=(), qkv_dims=None, rs_shapes: bool = False) -> dict:
+                tail_shapes=(), qkv_dims=None, rs_shapes: bool = False, sum_shapes=(),
+                sum_consumer=None, stream_shapes=()) -> dict:
     """Time hipBLASLt against every skinny configuration for each weight shape and
     batch size M (decode buckets <= SKINNY_MAX_M) and record the skinny kernel where it
     is faster by more than ``1 - margin``.  Each timing sweeps ALL weights of the shape
@@ -626,7 +640,9 @@ def tune_skinny(weights: Iterable[torch.Tensor], ms: Iterable[int], margin: floa
     ``tail_shapes``: (N, K) of row-parallel projections feeding a residual add + RMSNorm
     (``linear_add_rms``), timed with that norm on both sides.  ``rs_shapes``: also time the
     norm-free layer's epilogues at M <= 16 (tail -> SK_ACC_SS, norm -> SK_RSCALE, silu ->
-    SK_RSCALE_SILU) for ``rs_plan``."""
+    SK_RSCALE_SILU) for ``rs_plan``.  ``sum_shapes``: (N, K) whose consumer sums K-slices
+    (``linear_slices``), timed with ``sum_consumer(M)`` -> fn(y); ``stream_shapes``: (N, K) for
+    which K9m is also tried at M <= SKINNY_MAX_M."""
     if not _enabled:
         return {}
     by_shape: dict[tuple[int, int], list[torch.Tensor]] = {}
@@ -681,10 +697,11 @@ def tune_skinny(weights: Iterable[torch.Tensor], ms: Iterable[int], margin: floa
                      lib_t * 1e3 / n, sk_cfg, sk_t * 1e3 / n, "skinny" if best else "hipBLASLt")
         if _dg_enabled:
             qd = (qkv_dims or {}).get((N, K))
-            kind = ("silu" if (N, K) in silu_shapes else
+            kind = ("sum" if (N, K) in sum_shapes else "silu" if (N, K) in silu_shapes else
                     "tail" if (N, K) in tail_shapes else "qkv" if qd else "plain")
-            _tune_dgemm(ws, N, K, [m for m in ms if SKINNY_MAX_M < m <= DG_MAX_M], margin,
-                        reps, res, kind, qd)
+            lo = 0 if kind == "sum" or (N, K) in stream_shapes else SKINNY_MAX_M
+            _tune_dgemm(ws, N, K, [m for m in ms if lo < m <= DG_MAX_M], margin,
+                        reps, res, kind, qd, sum_consumer)
     log.info("GEMM tuning: %d shapes in %.1f s", len(res), time.time() - t0)
     return res
 
@@ -709,7 +726,8 @@ def _dg_candidates(M: int, N: int, K: int, kind: str, packed: bool):
     from . import _k
     # 11-14: packed 64 / 80 / 112-wide column tiles (gemm_decode.hip kCfg) for the narrow
     # shards of a TP = 8 rank
-    cfgs = [5, 7, 2, 14, 11] if M <= 128 else [6, 8, 4, 0, 10, 11, 12, 13, 14]
+    cfgs = ([5, 7, 10, 2, 14, 3] if M <= SKINNY_MAX_M or (kind == "sum" and M <= 128) else
+            [5, 7, 2, 14, 11] if M <= 128 else [6, 8, 4, 0, 10, 11, 12, 13, 14])
     out = []
     for c in range(_k().dgemm_num_cfgs()):
         if c not in cfgs:
@@ -737,17 +755,17 @@ def _dg_candidates(M: int, N: int, K: int, kind: str, packed: bool):
 
 
 def _tune_dgemm(ws, N: int, K: int, ms, margin: float, reps: int, res: dict,
-                kind: str, qkv_dims=None) -> None:
-    """hipBLASLt vs the K9m candidates at each M in ``ms``, over all weights of the shape
+                kind: str, qkv_dims=None, sum_consumer=None) -> None:
+    """hipBLASLt (at M <= SKINNY_MAX_M: what ``linear`` runs) vs the K9m candidates at each M in ``ms``, over all weights of the shape
     (HBM-resident, as in a decode step), each side timed WITH its consumer: "silu" the
     SiLU-and-mul, "tail" the residual add + RMSNorm, "qkv" the fused RoPE / KV-write /
-    decode-attention kernel (which sums the K-slices in its prologue), "plain" the split-K
-    reduction."""
+    decode-attention kernel (which sums the K-slices in its prologue), "sum" the consumer given,
+    "plain" the split-K reduction."""
     from . import (_k, decode_partials, fused_add_rms_norm, paged_attention_decode_rope,
                    silu_mul)
     packed = all(packed_weight(w, kind == "silu") is not None for w in ws)
     for M in sorted(set(ms)):
-        if not dgemm_ok(M, N, K) or (kind == "tail" and N > 8192):
+        if not dgemm_ok(max(M, SKINNY_MAX_M + 1), N, K) or (kind == "tail" and N > 8192):
             continue
         key = (M, N, K, kind)
         if key in _dg_table:
@@ -781,14 +799,17 @@ def _tune_dgemm(ws, N: int, K: int, ms, margin: float, reps: int, res: dict,
                 paged_attention_decode_rope(y, pos, cs, kc, vc, slots, nq, nkv, hd, bt, cl,
                                             hd ** -0.5, workspace=wsp, grid_z=1, dtype=dt)
 
+        if kind == "sum":
+            consume = sum_consumer(M, N)
+
         def lib():
             for w in ws:
-                y = F.linear(x, w)
+                y = linear(x, w) if M <= SKINNY_MAX_M else F.linear(x, w)
                 if kind == "silu":
                     silu_mul(y, act)
                 elif kind == "tail":
                     fused_add_rms_norm(y, res_t, gamma, 1e-6)
-                elif kind == "qkv":
+                elif kind in ("qkv", "sum"):
                     consume(y)
         lib_t = _time(lib, reps)
         best_t, best_cfg = float("inf"), None
@@ -807,11 +828,11 @@ def _tune_dgemm(ws, N: int, K: int, ms, margin: float, reps: int, res: dict,
                         _k().dgemm(buf, x, w, cfg, 2 if kind == "silu" else 1)
                         if kind == "tail":
                             fused_add_rms_norm(buf, res_t, gamma, 1e-6)
-                        elif kind == "qkv":
+                        elif kind in ("qkv", "sum"):
                             consume(buf)
                     else:
                         _k().dgemm(buf, x, w, cfg, 0)
-                        if kind == "qkv":
+                        if kind in ("qkv", "sum"):
                             consume(buf)
                         elif kind == "silu":
                             _k().splitk_reduce_silu(red, buf, il)
@@ -848,6 +869,8 @@ def _tune_dgemm(ws, N: int, K: int, ms, margin: float, reps: int, res: dict,
         chosen = best_cfg if best_t < lib_t * margin else None
         if chosen is not None:
             _plan_dg[(M, N, K, kind)] = chosen
+            if kind == "plain":
+                _plan.pop((M, N, K), None)
         res[(M, N, K, kind)] = (chosen, lib_t * 1e3 / n, best_t * 1e3 / n, best_cfg)
         log.info("gemm M=%d N=%d K=%d %s: hipBLASLt %.1f us, K9m %s %.1f us -> %s", M, N, K,
                  kind, lib_t * 1e3 / n, best_cfg, best_t * 1e3 / n,

@@ -390,7 +390,7 @@ def test_one_matrix_per_head(device, dtype, T, H, N, K, r):
 
 # ---------------------------------------------------------------- routing and experts
 @pytest.mark.parametrize("device", DEV)
-@pytest.mark.parametrize("E,top", [(5, 2), (12, 1), (3, 3), (70, 4), (300, 9)])
+@pytest.mark.parametrize("E,top", [(5, 2), (12, 1), (3, 3), (24, 6), (64, 16), (70, 4), (300, 9), (40, 20)])
 def test_raw_sigmoid_routing(device, E, top):
     dev, T, rng = dev_of(device), 40, np.random.default_rng(E)
     h, router = oracle.bf16(rng.normal(size=(T, 64))), oracle.bf16(0.3 * rng.normal(size=(E, 64)))
@@ -399,6 +399,17 @@ def test_raw_sigmoid_routing(device, E, top):
     gw, gi = ops.moe_route_sigmoid(s, None, top, 1.0, False)
     assert np.array_equal(gi.cpu().numpy(), ids)
     np.testing.assert_allclose(gw.cpu().numpy(), w, rtol=1e-5)
+    # the router's product and the choice in one launch (16-bit activations), or both ops
+    for dt in (torch.float32, torch.bfloat16):
+        for n in (T, 17, 1):
+            gw, gi = ops.moe_gate_sigmoid(f32(h[:n], dev).to(dt), f32(router, dev).to(dt), None, top, 1.0, False)
+            assert np.array_equal(gi.cpu().numpy(), ids[:n])
+            np.testing.assert_allclose(gw.cpu().numpy(), w[:n], rtol=1e-4)
+    corr = f32(rng.normal(size=E), dev)
+    want = ops.moe_route_sigmoid(s, corr, top, 2.5)
+    got = ops.moe_gate_sigmoid(f32(h, dev).to(torch.bfloat16), f32(router, dev).to(torch.bfloat16), corr, top, 2.5)
+    assert torch.equal(got[1], want[1])
+    np.testing.assert_allclose(got[0].cpu().numpy(), want[0].cpu().numpy(), rtol=1e-4)
     # equal scores: the lowest index; and the correction still only steers the choice
     flat = torch.full((3, E), 0.25, device=dev)
     gw, gi = ops.moe_route_sigmoid(flat, None, top, 1.0, False)
@@ -476,8 +487,13 @@ def test_grouped_experts_split_k(device):
 
 
 def test_which_form_a_step_takes():
-    m = InputScaledExperts(128, FeedForwardSpec("moe", 64, gated=True, experts=8, top=2, router="sigmoid_raw",
-                                                weight_input=True, shared_gate=False), torch.float32, "cpu")
-    assert m.dense_step(1) and m.dense_step(5000)              # sizes or types without tiles
-    m.native = True
-    assert [m.dense_step(t) for t in (1, 3, 4, 64, 5000)] == [False, False, True, True, False]
+    def form(E, top, ff, T, native=True):
+        spec = FeedForwardSpec("moe", ff, gated=True, experts=E, top=top, router="sigmoid_raw",
+                               weight_input=True, shared_gate=False)
+        m = InputScaledExperts(4096, spec, torch.bfloat16, "meta")
+        m.native = native
+        return ["grouped", "dense"][m.dense_step(T)]
+    assert form(8, 2, 1792, 5000, native=False) == "dense"     # sizes or types without tiles
+    assert [form(8, 2, 1792, t) for t in (2, 64, 256, 257)] == ["dense"] * 3 + ["grouped"]
+    # many large experts of which a step touches few
+    assert [form(64, 2, 4096, t) for t in (1, 4, 64, 5000)] == ["grouped", "grouped", "dense", "grouped"]

@@ -3,7 +3,8 @@ closest to, at the layer shapes of the dilavik-w2048 / konovik-w2048 / nolesun-w
 llama-w2048 presets (``--only nolesun``: the parallel mixers' kernels; ``--only lorenex``: gated
 linear attention, the selective scan, unit-RMS attention inputs, PolyNorm, clamped experts;
 ``--only generax``: the channel-wise delta rule, pooled blocks, rotated values, whole-row norms,
-each beside its like kernel on the same shapes).
+each beside its like kernel on the same shapes; ``--only ratizen``: hyper-connected streams, per-head
+norms, chunks with a sink, latent queries, experts on scaled inputs, likewise).
 
     python tools/hybrid_bench.py [--reps 20] > profiles/hybrid_kernels.jsonl
 
@@ -553,6 +554,146 @@ def generax(reps):
                  like=None if kind == "window" else "window_attention (window)")
 
 
+def ratizen(reps):
+    """The Ratizen kernels at the ratizen-w2048 layer shapes, each beside the closest kernel of the
+    other decoders at the same sizes."""
+    W, S = 2048, 4
+    for T in (16384, 64, 256):
+        X, x = torch.randn(T, S, W, device=DEV), torch.zeros(T, W, device=DEV)
+        y = torch.randn(T, W, device=DEV, dtype=BF)
+        w, mix = torch.ones(W, device=DEV), torch.eye(S, device=DEV)
+        one = torch.full((S,), 0.25, device=DEV)
+        us = timed(lambda: ops.hyper_norm(X, X, [(y, 1)], mix, one, one, w, 1e-6, BF), reps)
+        emit("hyper_norm (4 streams)", f"{T}x{W}", us, gbytes=T * W * (8 * S + 4) / 1e9, like="residual_norm")
+        pairs = torch.randn(2 * T, W, device=DEV, dtype=BF)
+        us = timed(lambda: ops.hyper_norm(X, X, [(pairs, 2), (y, 1)], mix, one, one, w, 1e-6, BF), reps)
+        emit("hyper_norm (4 streams, 2 expert rows + shared)", f"{T}x{W}", us,
+             gbytes=T * W * (8 * S + 8) / 1e9, like="residual_norm + moe_finish")
+        us = timed(lambda: ops.residual_norm(x, y, 0.5, w, 1e-6, BF), reps)
+        emit("residual_norm", f"{T}x{W}", us, gbytes=T * W * 12 / 1e9)
+        h = torch.randn(T, W, device=DEV, dtype=BF)
+        router = torch.randn(8, W, device=DEV, dtype=BF)
+        us = timed(lambda: ops.gate_proj(h, router, None, ops.GATE_SIGMOID), reps)
+        emit("gate_proj (8 experts)", f"{T}x{W}", us, gbytes=T * W * 2 / 1e9)
+        sc = torch.rand(T, 8, device=DEV)
+        us = timed(lambda: ops.moe_route_sigmoid(sc, None, 2, 1.0, False), reps)
+        emit("moe_route_sigmoid (raw scores)", f"{T}x8", us, like="moe_route_sigmoid")
+        corr = torch.zeros(8, device=DEV)
+        us = timed(lambda: ops.moe_route_sigmoid(sc, corr, 2, 1.0), reps)
+        emit("moe_route_sigmoid", f"{T}x8", us)
+    # experts: 8 of 1792 (two per token) and a shared one of 1920
+    E, I, Is, top = 8, 1792, 1920, 2
+    w_in = torch.randn(2 * (E * I + Is), W, device=DEV, dtype=BF) * 0.02
+    w_dn = torch.randn(W, E * I + Is, device=DEV, dtype=BF) * 0.02
+    up, dn = w_in[: 2 * E * I].view(E, 2 * I, W), w_dn[:, : E * I].view(W, E, I).transpose(0, 1)
+    dnc = dn.contiguous()
+    for T in (16384, 256, 64, 8):
+        h = torch.randn(T, W, device=DEV, dtype=BF)
+        tw, ti = ops.moe_route_sigmoid(torch.rand(T, E, device=DEV), None, top, 1.0, False)
+        fl = 2 * T * top * 3 * I * W / 1e12
+        gb = 3 * E * I * W * 2 / 1e9
+        us = timed(lambda: ops.grouped_experts_scaled(h, up, dn, tw, ti), reps)
+        emit("grouped_experts_scaled", f"{T}x{W}, 2 of 8 x {I}", us, tflop=fl, gbytes=gb, like="fused_moe")
+        us = timed(lambda: ops.fused_moe(h, up, dnc, tw, ti), reps)
+        emit("fused_moe (same shape)", f"{T}x{W}, 2 of 8 x {I}", us, tflop=fl, gbytes=gb)
+        if T <= 256:
+            def dense():
+                a = ops.expert_silu_all(torch.nn.functional.linear(h, w_in), tw, ti, E, I, Is)
+                return torch.nn.functional.linear(a, w_dn)
+            us = timed(dense, reps)
+            emit("all experts and the shared one as one GEMM pair (untuned)", f"{T}x{W}", us,
+                 gbytes=(w_in.numel() + w_dn.numel()) * 2 / 1e9, like="fused_moe")
+            g = torch.randn(T, 2 * (E * I + Is), device=DEV, dtype=BF)
+            us = timed(lambda: ops.expert_silu_all(g, tw, ti, E, I, Is), reps)
+            emit("expert_silu_all", f"{T}x{E * I + Is}", us,
+                 gbytes=T * ((E * I + Is) * 2 + 4 * (top * I + Is)) / 1e9, like="silu_mul")
+            us = timed(lambda: ops.silu_mul(g), reps)
+            emit("silu_mul (same shape)", f"{T}x{E * I + Is}", us, gbytes=T * (E * I + Is) * 6 / 1e9)
+        else:
+            rows = T * top
+            g, o = torch.randn(rows, 2 * I, device=DEV, dtype=BF), torch.empty(rows, I, device=DEV, dtype=BF)
+            ids = torch.arange(rows, device=DEV, dtype=torch.int32)
+            us = timed(lambda: torch.ops.kgc.expert_silu_rows(o, g, tw, ids), reps)
+            emit("expert_silu_rows", f"{rows}x{I}", us, gbytes=rows * I * 6 / 1e9, like="silu_mul")
+            us = timed(lambda: ops.silu_mul(g), reps)
+            emit("silu_mul (same shape)", f"{rows}x{I}", us, gbytes=rows * I * 6 / 1e9)
+    H, G, d, bs, win = 16, 4, 128, 32, 1024
+    r, rank, qr = 64, 192, 768
+    for name, P_q, P_sl, D_ctx in (("prefill 32x512", [512] * 32, [512] * 32, []),
+                                   ("prefill 8x2048", [2048] * 8, [2048] * 8, []),
+                                   ("prefill 2x8192", [8192] * 2, [8192] * 2, []),
+                                   ("decode 64 @544", [], [], [544] * 64),
+                                   ("decode 256 @544", [], [], [544] * 256),
+                                   ("decode 64 @8000", [], [], [8000] * 64)):
+        m, tables, nb = meta(P_q, P_sl, D_ctx, bs, DEV)
+        T = sum(P_q) + len(D_ctx)
+        pos = torch.cat([torch.arange(s) for s in P_sl]) if P_q else torch.tensor(D_ctx) - 1
+        pos = pos.to(DEV)
+        seq = torch.repeat_interleave(torch.arange(len(P_sl) + len(D_ctx)), torch.tensor(P_q or [1] * len(D_ctx)))
+        slots = tables[seq.to(DEV), pos // bs].long() * bs + pos % bs
+        m.slot_mapping = slots
+        qkv = torch.randn(T, (H + 2 * G) * d, device=DEV, dtype=BF)
+        kc = torch.randn(nb, G, bs, d, device=DEV, dtype=BF)
+        vc = torch.randn(nb, G, bs, d, device=DEV, dtype=BF)
+        one = torch.ones(H * d, device=DEV)
+        gb = T * (H + 2 * G) * d * 4 / 1e9
+        us = timed(lambda: ops.norm_kv_store(qkv, pos, kc, vc, slots, H, G, d, d, 1e-6, True, False, None, BF,
+                                             one[:d], one[:d]), reps)
+        emit("norm_kv_store (per-head norms)", name, us, gbytes=gb, like="qk_norm_store")
+        us = timed(lambda: ops.qk_norm_store(qkv, pos, one, one[: G * d], 1e-6, None, None, kc, vc, slots, H, G,
+                                             d, d), reps)
+        emit("qk_norm_store (whole-row norms)", name, us, gbytes=gb)
+        q = torch.randn(T, H, d, device=DEV, dtype=BF)
+        P = [p + 1 for s in P_sl for p in range(s)] if P_q else D_ctx
+        for kind in ("window", "chunks and a sink"):
+            ch = kind != "window"
+            keys = sum(((p - 1) % win + 1) if ch else min(p, win) for p in P)
+            us = timed(lambda: ops.window_attention(q, kc, vc, pos, m, 0.09, win, 0, chunked=ch,
+                                                    sink=0.0 if ch else None), reps)
+            emit(f"window_attention ({kind})", name, us, gbytes=None if P_q else keys * G * 4 * d / 1e9,
+                 tflop=keys * H * 4 * d / 1e12 if P_q else None,
+                 like="window_attention (window)" if ch else None)
+        # latent attention: rows into the cache, queries into latent space, results out of it
+        cache = torch.randn(nb, 1, bs, rank + r, device=DEV, dtype=BF)
+        tab = ops.ref.rope_table_yarn(r, 8192, 1e4).to(DEV)
+        n_in = -(-(qr + rank + r + H) // 64) * 64
+        proj = torch.randn(T, n_in, device=DEV, dtype=BF)
+        qw, kw = torch.ones(qr, device=DEV), torch.ones(rank, device=DEV)
+        qf = torch.randn(T, H, d + r, device=DEV, dtype=BF)
+        uk = torch.randn(H, rank, d, device=DEV, dtype=BF) * 0.1
+        uv = torch.randn(H, d, rank, device=DEV, dtype=BF) * 0.1
+        us = timed(lambda: ops.latent_down_store(proj, pos, tab, qw, kw, 1e-6, cache, slots, r, H), reps)
+        emit("latent_down_store", name, us, gbytes=T * (2 * qr + 2 * (rank + r) + 3 * H) * 2 / 1e9,
+             like="latent_rope_store")
+        qo = torch.empty(T, H, rank + r, device=DEV, dtype=BF)
+        us = timed(lambda: ops.head_gemm(qf[..., :d], uk, qo, qf[..., d:], pos, tab), reps)
+        gbq = T * H * (d + r + rank + r) * 2 / 1e9
+        emit("head_gemm (queries, with the rotation)", name, us, gbytes=gbq, tflop=2 * T * H * d * rank / 1e12,
+             like="bmm + latent_rope_store")
+        kpj = torch.randn(T, H * (d + r) + rank + r, device=DEV, dtype=BF)
+        ukb = uk.transpose(1, 2).contiguous()
+
+        def konovik_queries():
+            ql = torch.bmm(kpj[:, : H * (d + r)].view(T, H, d + r)[:, :, :d].transpose(0, 1), ukb)
+            return ops.latent_rope_store(kpj, ql, pos, tab, kw, 1e-6, cache, slots, H, d, r, rank)
+        us = timed(konovik_queries, reps)
+        emit("bmm + latent_rope_store (same sizes)", name, us, gbytes=gbq)
+        o, yo = torch.randn(T, H, rank, device=DEV, dtype=BF), torch.empty(T, H, d, device=DEV, dtype=BF)
+        us = timed(lambda: ops.head_gemm(o, uv, yo), reps)
+        gbv = T * H * (rank + d) * 2 / 1e9
+        emit("head_gemm (values)", name, us, gbytes=gbv, tflop=2 * T * H * d * rank / 1e12, like="bmm + gate_mul")
+        uvb, gm = uv.transpose(1, 2).contiguous(), torch.randn(T, H * d, device=DEV, dtype=BF)
+        us = timed(lambda: ops.gate_mul(torch.bmm(o.transpose(0, 1), uvb).transpose(0, 1), gm), reps)
+        emit("bmm + gate_mul (same sizes)", name, us, gbytes=gbv)
+        gate = torch.rand(T, H, device=DEV)
+        keys = sum(min(p, win) for p in P)
+        for kind, g in (("latent rows, head gates", gate), ("latent rows", None)):
+            us = timed(lambda: ops.window_attention(qo, cache, cache[..., :rank], pos, m, 0.07, win, 0, g), reps)
+            emit(f"window_attention ({kind})", name, us, gbytes=None if P_q else keys * (rank + r) * 2 / 1e9,
+                 tflop=keys * H * 2 * (2 * rank + r) / 1e12,
+                 like="window_attention (latent rows)" if g is not None else None)
+
+
 if __name__ == "__main__":
     ap = argparse.ArgumentParser()
     ap.add_argument("--reps", type=int, default=20)
@@ -561,4 +702,4 @@ if __name__ == "__main__":
     ops.load_extension(strict=True)
     for part in a.only.split(","):
         {"attention": attention, "recurrent": recurrent, "rows": rows, "konovik": konovik,
-         "nolesun": nolesun, "lorenex": lorenex, "generax": generax}[part](a.reps)
+         "nolesun": nolesun, "lorenex": lorenex, "generax": generax, "ratizen": ratizen}[part](a.reps)
