@@ -91,7 +91,7 @@ def parse():
     ap.add_argument("--compare-sizes", default="w2048,w4096",
                     help="--mode compare: size suffixes of the <family>-<size> presets")
     ap.add_argument("--compare-families", default="dilavik,llama",
-                    help="--mode compare: the preset families to run at each size (generax, lorenex, "
+                    help="--mode compare: the preset families to run at each size (ratizen, generax, lorenex, "
                          "nolesun, dilavik, konovik, llama); ratios are taken against the last one")
     ap.add_argument("--mode", default="service", choices=["service", "engine", "compare"],
                     help="service: HTTP/SSE through API server + router (headline); "
@@ -643,7 +643,7 @@ def _compare_one(model: str, args) -> dict:
 
 
 def main_compare(args):
-    """--mode compare: the hybrid presets (generax, lorenex, nolesun, dilavik, konovik) beside
+    """--mode compare: the hybrid presets (ratizen, generax, lorenex, nolesun, dilavik, konovik) beside
     the Llama-style decoders of equal size (models/configs.py), same requests, same engine
     settings, one JSON line per model and a closing line with the ratios.  Random weights, synthetic prompts."""
     assert torch.cuda.is_available(), "bench.py --mode compare needs a GPU"

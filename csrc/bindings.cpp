@@ -1517,6 +1517,7 @@ void window_attention(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
       kgc::window_prefill_mfma_ok(dt, (int)dk, (int)dv) &&
       (vtp == nullptr || interleaved || dv % 32 == 0)) {   // a pair within one lane
     const int64_t nw = work_seq->numel();
+    TORCH_CHECK(nw * (kgc::prefill_block_m() / 64) <= 65535, "kgc.window_attention: work items");
     kgc::launch_window_prefill_mfma(dt, out.data_ptr(), q.data_ptr(), k_cache.data_ptr(),
                                     v_cache.data_ptr(), qp, sp, pp, (int)bts,
                                     work_seq->data_ptr<int>(), work_blk->data_ptr<int>(), (int)nw,
@@ -1525,7 +1526,14 @@ void window_attention(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
                                     stream());
     rest &= ~1;
   }
-  if (decode_fast) {
+  if (fast && aligned && D > 0 &&
+      kgc::window_decode_mfma_ok(dt, (int)dk, (int)dv, (int)(H / G), ex)) {
+    kgc::launch_window_decode_mfma(dt, out.data_ptr(), q.data_ptr(), k_cache.data_ptr(),
+                                   v_cache.data_ptr(), cp, dp, (int)bts, (int)Tp, (int)D, (int)H,
+                                   (int)G, (int)dk, (int)dv, (int)krs, (int)vrs, bs, nb,
+                                   (float)scale, (int)window, (int)keep_first, gp, ex, stream());
+    rest &= ~2;
+  } else if (decode_fast) {
     kgc::launch_window_decode(dt, out.data_ptr(), q.data_ptr(), k_cache.data_ptr(),
                               v_cache.data_ptr(), cp, dp, (int)bts, (int)Tp, (int)D, (int)H,
                               (int)G, (int)dk, (int)dv, (int)krs, (int)vrs, bs, nb, (float)scale,

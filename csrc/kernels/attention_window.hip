@@ -633,6 +633,182 @@ __global__ __launch_bounds__(64 * NWV) void window_decode_kernel(
   }
 }
 
+// Decode rows on the matrix cores (16-bit activations): one workgroup of NWV waves per (row, kv
+// head, group of up to 16 query heads).  The visible keys are cut into 32-key chunks dealt
+// round-robin to the waves.  Per chunk and wave, with the heads as columns (lane & 15):
+//   S^T = K . Q^T   two 16-key tiles, A fragments straight from the cache rows (A row m is key
+//                   8 (m >> 2) + (m & 3), + 4 in the second tile),
+//   online softmax in fp32, statistics per head in the lane,
+//   O^T += V^T . P^T with P^T straight from the S^T accumulators as a pair of values (value +
+//                   remainder) and V^T through the wave's own piece of LDS; where the values are
+//                   columns of the key rows the key fragments are what is written there.
+// The waves' states meet in LDS at the end, in wave order.
+constexpr int DM_VST = 40;             // elements per V^T row: 32 keys + 8
+
+template <typename T, int KS, int DT, int NWV>
+__global__ __launch_bounds__(64 * NWV) void window_decode_mfma_kernel(
+    T* __restrict__ out, const T* __restrict__ q, const T* __restrict__ k_cache,
+    const T* __restrict__ v_cache, const int* __restrict__ ctx_lens, const int* __restrict__ dbt,
+    int bt_stride, int Tp, int H, int G, int dk, int dv, int krs, int vrs, int bs, int num_blocks,
+    float scale, int window, int keep_first, const float* __restrict__ gate, bool shared,
+    WindowExtra ex) {
+  typedef typename Vec8<T>::type V8;
+  constexpr int VBYTES = NWV * DT * 16 * DM_VST * 2, OBYTES = NWV * 16 * DT * 16 * 4;
+  __shared__ __attribute__((aligned(16))) char smem[VBYTES > OBYTES ? VBYTES : OBYTES];
+  __shared__ float mm[NWV][16], ml[NWV][16];
+  const int dd = blockIdx.x, g = blockIdx.y, qpg = H / G, hq0 = blockIdx.z * 16;
+  const int nh = min(16, qpg - hq0), h0 = g * qpg + hq0, t = Tp + dd;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r16 = lane & 15, qd = lane >> 4;
+  const int pos = ctx_lens[dd] - 1;
+  const int* bt = dbt + (int64_t)dd * bt_stride;
+  if (pos < 0 || pos >= bt_stride * bs) {             // a padding row: zeros
+    for (int e = threadIdx.x; e < nh * dv; e += 64 * NWV)
+      out[(int64_t)t * ex.ors + h0 * dv + e] = from_f<T>(0.f);
+    return;
+  }
+  V8 qf[KS];
+  {
+    const T* qrow = q + ((int64_t)t * H + h0 + min(r16, nh - 1)) * dk;
+#pragma unroll
+    for (int s = 0; s < KS; ++s) {
+      Pack8<T> p;
+      p.u = u32x4{0u, 0u, 0u, 0u};
+      if (32 * s + 8 * qd < dk) p.u = *reinterpret_cast<const u32x4*>(qrow + 32 * s + 8 * qd);
+      qf[s] = p.v;
+    }
+  }
+  const int lo_w = first_visible(pos, window, ex.chunked), ns = min(keep_first, lo_w);
+  const int total = ns + (pos - lo_w + 1), nch = (total + 31) >> 5;
+  const int keyA = 8 * (r16 >> 2) + (r16 & 3);
+  T* vt = reinterpret_cast<T*>(smem) + wave * DT * 16 * DM_VST;
+  float m = wave == 0 ? ex.sink : -INFINITY;          // (the first wave always has keys)
+  float l = qd == 0 && m > -INFINITY ? 1.f : 0.f;
+  f32x4 o[DT];
+#pragma unroll
+  for (int d = 0; d < DT; ++d) o[d] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int ch = wave; ch < nch; ch += NWV) {
+    Pack8<T> kf[2][KS];
+    int64_t row[2];
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+      const int idx = min(32 * ch + keyA + 4 * j, total - 1);      // clamped: weight 0 below
+      const int key = idx < ns ? idx : lo_w + (idx - ns);
+      int b = bt[key / bs];
+      if (b < 0 || b >= num_blocks) b = 0;
+      row[j] = (int64_t)(b * G + g) * bs + key % bs;
+      const T* kr = k_cache + row[j] * krs + 8 * qd;
+#pragma unroll
+      for (int s = 0; s < KS; ++s) {
+        kf[j][s].u = u32x4{0u, 0u, 0u, 0u};
+        if (32 * s + 8 * qd < dk) kf[j][s].u = *reinterpret_cast<const u32x4*>(kr + 32 * s);
+      }
+    }
+    Pack8<T> vf[2][DT / 2];
+    if (!shared) {
+#pragma unroll
+      for (int j = 0; j < 2; ++j) {
+        const T* vr = v_cache + row[j] * vrs + 8 * qd;
+#pragma unroll
+        for (int s = 0; s < DT / 2; ++s) {
+          vf[j][s].u = u32x4{0u, 0u, 0u, 0u};
+          if (32 * s + 8 * qd < dv) vf[j][s].u = *reinterpret_cast<const u32x4*>(vr + 32 * s);
+        }
+      }
+    }
+    f32x4 sc[2];
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+      f32x4 a = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int s = 0; s < KS; ++s) a = mfma16x16x32(kf[j][s].v, qf[s], a);
+      sc[j] = a;
+    }
+    // V^T of the chunk, while the products are under way
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");    // (the last chunk's fragments were read)
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int s = 0; s < DT / 2; ++s) {
+      if (32 * s + 8 * qd < dv) {
+#pragma unroll
+        for (int j = 0; j < 2; ++j)
+#pragma unroll
+          for (int e = 0; e < 8; ++e)
+            vt[(32 * s + 8 * qd + e) * DM_VST + keyA + 4 * j] =
+                shared ? kf[j][s < KS ? s : 0].h[e] : vf[j][s].h[e];
+      }
+    }
+    float tmax = -INFINITY;
+#pragma unroll
+    for (int j = 0; j < 2; ++j)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const bool ok = 32 * ch + 8 * qd + 4 * j + i < total;
+        sc[j][i] = ok ? cap_score(sc[j][i] * scale, ex.softcap) : -INFINITY;
+        tmax = fmaxf(tmax, sc[j][i]);
+      }
+    tmax = fmaxf(tmax, __shfl_xor(tmax, 16, 64));
+    tmax = fmaxf(tmax, __shfl_xor(tmax, 32, 64));
+    const float mn = fmaxf(m, tmax);
+    const float alpha = m == -INFINITY ? 0.f : __expf(m - mn);
+    m = mn;
+    l *= alpha;
+    Pack8<T> ph, pl;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const float pa = sc[0][i] == -INFINITY ? 0.f : __expf(sc[0][i] - mn);
+      const float pb = sc[1][i] == -INFINITY ? 0.f : __expf(sc[1][i] - mn);
+      l += pa + pb;
+      ph.h[i] = from_f<T>(pa);
+      ph.h[4 + i] = from_f<T>(pb);
+      pl.h[i] = from_f<T>(pa - to_f(ph.h[i]));
+      pl.h[4 + i] = from_f<T>(pb - to_f(ph.h[4 + i]));
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int d = 0; d < DT; ++d) {
+      if (16 * d < dv) {
+        Pack8<T> fr;
+        fr.u = *reinterpret_cast<const u32x4*>(vt + (16 * d + r16) * DM_VST + 8 * qd);
+        f32x4 a = o[d] * alpha;
+        a = mfma16x16x32(fr.v, ph.v, a);
+        o[d] = mfma16x16x32(fr.v, pl.v, a);
+      }
+    }
+  }
+  l += __shfl_xor(l, 16, 64);
+  l += __shfl_xor(l, 32, 64);
+  if (qd == 0) {
+    mm[wave][r16] = m;
+    ml[wave][r16] = l;
+  }
+  __syncthreads();
+  float M = -INFINITY;
+#pragma unroll
+  for (int w = 0; w < NWV; ++w) M = fmaxf(M, mm[w][r16]);
+  const float f = m == -INFINITY ? 0.f : __expf(m - M);
+  float* ob = reinterpret_cast<float*>(smem);         // [NWV][16][DT * 16]
+#pragma unroll
+  for (int d = 0; d < DT; ++d)
+    *reinterpret_cast<f32x4*>(ob + (wave * 16 + r16) * DT * 16 + 16 * d + 4 * qd) = o[d] * f;
+  __syncthreads();
+  for (int e = threadIdx.x; e < nh * dv; e += 64 * NWV) {
+    const int h = e / dv, c = e - h * dv;
+    float Mh = -INFINITY, L = 0.f, a = 0.f;
+#pragma unroll
+    for (int w = 0; w < NWV; ++w) Mh = fmaxf(Mh, mm[w][h]);
+#pragma unroll
+    for (int w = 0; w < NWV; ++w) {
+      const float mw = mm[w][h];
+      if (mw != -INFINITY) L += ml[w][h] * __expf(mw - Mh);
+      a += ob[(w * 16 + h) * DT * 16 + c];
+    }
+    const float gt = (gate != nullptr ? gate[(int64_t)t * H + h0 + h] : 1.f) * ex.out_scale;
+    out[(int64_t)t * ex.ors + h0 * dv + e] =
+        from_f<T>(a * gt / L * elem_gate<T>(ex, t, h0 * dv + e));
+  }
+}
+
 // Prefill chunks on the matrix cores (16-bit activations).  One workgroup of 4 waves per
 // (64 query rows of a chunk, query head); wave w owns rows 16 w .. 16 w + 15.  Keys come in
 // 64-key tiles -- first the kept first tokens that lie before the tile's earliest window,
@@ -1415,6 +1591,52 @@ void launch_window_decode(int dtype, void* out, const void* q, const void* k_cac
                                            (const T*)v_cache, ctx_lens, dbt, bt_stride, Tp, D, H,
                                            G, dk, dv, krs, vrs, bs, num_blocks, scale, window, keep_first,
                                            gate, ex, s));
+}
+
+// (with one or two query heads per key/value head the vector kernel is as fast)
+bool window_decode_mfma_ok(int dtype, int dk, int dv, int qpg, const WindowExtra& ex) {
+  return (dtype == DT_BF16 || dtype == DT_F16) && dk % 8 == 0 && dk <= 256 && dv % 8 == 0 &&
+         dv <= 256 && qpg >= 3 && ex.pool == 0 && ex.vtab == nullptr;
+}
+
+template <typename T>
+static void decode_mfma_dispatch(T* out, const T* q, const T* kc, const T* vc, const int* ctx_lens,
+                                 const int* dbt, int bt_stride, int Tp, int D, int H, int G, int dk,
+                                 int dv, int krs, int vrs, int bs, int num_blocks, float scale,
+                                 int window, int keep_first, const float* gate, WindowExtra ex,
+                                 hipStream_t s) {
+  const dim3 grid(D, G, (H / G + 15) / 16);
+  const bool shared = kc == vc && krs == vrs && dv <= dk;
+  const bool small = (int64_t)grid.x * grid.y * grid.z >= 512;     // several workgroups per CU
+#define KGC_DM(K, D_, W)                                                                       \
+  window_decode_mfma_kernel<T, K, D_, W><<<grid, 64 * W, 0, s>>>(                              \
+      out, q, kc, vc, ctx_lens, dbt, bt_stride, Tp, H, G, dk, dv, krs, vrs, bs, num_blocks, scale, \
+      window, keep_first, gate, shared, ex)
+#define KGC_DM2(K, D_)                              \
+  do {                                              \
+    if (small) KGC_DM(K, D_, 4); else KGC_DM(K, D_, 8); \
+  } while (0)
+  if (dk <= 128 && dv <= 128) KGC_DM2(4, 8);
+  else if (dv <= 192) KGC_DM2(8, 12);
+  else KGC_DM(8, 16, 4);
+#undef KGC_DM2
+#undef KGC_DM
+}
+
+void launch_window_decode_mfma(int dtype, void* out, const void* q, const void* k_cache,
+                               const void* v_cache, const int* ctx_lens, const int* dbt,
+                               int bt_stride, int Tp, int D, int H, int G, int dk, int dv, int krs,
+                               int vrs, int bs, int num_blocks, float scale, int window,
+                               int keep_first, const float* gate, WindowExtra ex, hipStream_t s) {
+  if (D <= 0) return;
+  if (dtype == DT_BF16)
+    decode_mfma_dispatch<bf16>((bf16*)out, (const bf16*)q, (const bf16*)k_cache,
+                               (const bf16*)v_cache, ctx_lens, dbt, bt_stride, Tp, D, H, G, dk, dv,
+                               krs, vrs, bs, num_blocks, scale, window, keep_first, gate, ex, s);
+  else
+    decode_mfma_dispatch<f16>((f16*)out, (const f16*)q, (const f16*)k_cache, (const f16*)v_cache,
+                              ctx_lens, dbt, bt_stride, Tp, D, H, G, dk, dv, krs, vrs, bs,
+                              num_blocks, scale, window, keep_first, gate, ex, s);
 }
 
 size_t window_prefill_mfma_lds(int dk, int dv) {

@@ -323,6 +323,13 @@ void launch_window_decode(int dtype, void* out, const void* q, const void* k_cac
                           int bt_stride, int Tp, int D, int H, int G, int dk, int dv, int krs,
                           int vrs, int bs, int num_blocks, float scale, int window, int keep_first,
                           const float* gate, WindowExtra ex, hipStream_t s);
+// decode rows on the matrix cores (no pooled blocks, no rotated values)
+bool window_decode_mfma_ok(int dtype, int dk, int dv, int qpg, const WindowExtra& ex);
+void launch_window_decode_mfma(int dtype, void* out, const void* q, const void* k_cache,
+                               const void* v_cache, const int* ctx_lens, const int* dbt,
+                               int bt_stride, int Tp, int D, int H, int G, int dk, int dv, int krs,
+                               int vrs, int bs, int num_blocks, float scale, int window,
+                               int keep_first, const float* gate, WindowExtra ex, hipStream_t s);
 bool window_prefill_mfma_ok(int dtype, int dk, int dv);
 void launch_window_prefill_mfma(int dtype, void* out, const void* q, const void* k_cache,
                                 const void* v_cache, const int* qsl, const int* seq_lens,

@@ -13,6 +13,7 @@ graph capture bakes the chosen kernel into each decode bucket's graph.
 """
 from __future__ import annotations
 
+import functools
 import logging
 import os
 import time
@@ -94,6 +95,7 @@ def _packed_put(w: torch.Tensor, silu: bool, p: torch.Tensor) -> None:
 _PACK_FRACTION = float(os.environ.get("KGC_DGEMM_PACK_FRACTION", "0.25"))
 
 
+@functools.lru_cache(maxsize=None)
 def _dg_info(cfg: int):
     from . import _k
     bm, bn, pk = _k().dgemm_cfg_info(cfg)
@@ -179,7 +181,10 @@ def dgemm(x: torch.Tensor, w: torch.Tensor, cfg: int, S: int, epi: int = 1,
 def _dg_plan(x: torch.Tensor, w: torch.Tensor, kind: str):
     if not _plan_dg or not x.is_cuda or x.dim() != 2 or x.stride(1) != 1 or x.stride(0) % 8:
         return None
-    return _plan_dg.get((x.shape[0], w.shape[0], w.shape[1], kind))
+    p = _plan_dg.get((x.shape[0], w.shape[0], w.shape[1], kind))
+    if p is not None and cfg_packed(p[0]) and packed_weight(w, kind == "silu") is None:
+        return None             # tuned for another engine's packed weight of this shape
+    return p
 
 
 def linear_silu(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None) -> torch.Tensor:

@@ -22,6 +22,7 @@ import torch
 sys.path.insert(0, os.path.dirname(os.path.dirname(os.path.abspath(__file__))))
 from kubernetes_gpu_cluster_amd import ops
 from kubernetes_gpu_cluster_amd.ops import reference as ref
+from kubernetes_gpu_cluster_amd.ops import gemm
 from kubernetes_gpu_cluster_amd.ops.gemm import linear
 
 DEV = torch.device("cuda")
@@ -573,20 +574,20 @@ def ratizen(reps):
         emit("residual_norm", f"{T}x{W}", us, gbytes=T * W * 12 / 1e9)
         h = torch.randn(T, W, device=DEV, dtype=BF)
         router = torch.randn(8, W, device=DEV, dtype=BF)
-        us = timed(lambda: ops.gate_proj(h, router, None, ops.GATE_SIGMOID), reps)
-        emit("gate_proj (8 experts)", f"{T}x{W}", us, gbytes=T * W * 2 / 1e9)
-        sc = torch.rand(T, 8, device=DEV)
-        us = timed(lambda: ops.moe_route_sigmoid(sc, None, 2, 1.0, False), reps)
-        emit("moe_route_sigmoid (raw scores)", f"{T}x8", us, like="moe_route_sigmoid")
+        us = timed(lambda: ops.moe_gate_sigmoid(h, router, None, 2, 1.0, False), reps)
+        emit("moe_gate_sigmoid (8 experts)", f"{T}x{W}", us, gbytes=T * W * 2 / 1e9,
+             like="gate_proj + moe_route_sigmoid")
         corr = torch.zeros(8, device=DEV)
-        us = timed(lambda: ops.moe_route_sigmoid(sc, corr, 2, 1.0), reps)
-        emit("moe_route_sigmoid", f"{T}x8", us)
+        us = timed(lambda: ops.moe_route_sigmoid(ops.gate_proj(h, router, None, ops.GATE_SIGMOID), corr, 2, 1.0),
+                   reps)
+        emit("gate_proj + moe_route_sigmoid", f"{T}x{W}", us, gbytes=T * W * 2 / 1e9)
     # experts: 8 of 1792 (two per token) and a shared one of 1920
     E, I, Is, top = 8, 1792, 1920, 2
     w_in = torch.randn(2 * (E * I + Is), W, device=DEV, dtype=BF) * 0.02
     w_dn = torch.randn(W, E * I + Is, device=DEV, dtype=BF) * 0.02
     up, dn = w_in[: 2 * E * I].view(E, 2 * I, W), w_dn[:, : E * I].view(W, E, I).transpose(0, 1)
     dnc = dn.contiguous()
+    gemm.pack_decode_weights([w_in, w_dn], [])
     for T in (16384, 256, 64, 8):
         h = torch.randn(T, W, device=DEV, dtype=BF)
         tw, ti = ops.moe_route_sigmoid(torch.rand(T, E, device=DEV), None, top, 1.0, False)
@@ -597,12 +598,14 @@ def ratizen(reps):
         us = timed(lambda: ops.fused_moe(h, up, dnc, tw, ti), reps)
         emit("fused_moe (same shape)", f"{T}x{W}, 2 of 8 x {I}", us, tflop=fl, gbytes=gb)
         if T <= 256:
+            cfg = 5 if T <= 128 else 6               # packed K9m tiles of 128 / 256 rows
+
             def dense():
-                a = ops.expert_silu_all(torch.nn.functional.linear(h, w_in), tw, ti, E, I, Is)
-                return torch.nn.functional.linear(a, w_dn)
+                a = ops.expert_silu_all(gemm.dgemm(h, w_in, cfg, 1), tw, ti, E, I, Is)
+                return gemm.dgemm(a, w_dn, cfg, 16)
             us = timed(dense, reps)
-            emit("all experts and the shared one as one GEMM pair (untuned)", f"{T}x{W}", us,
-                 gbytes=(w_in.numel() + w_dn.numel()) * 2 / 1e9, like="fused_moe")
+            emit("all experts and the shared one as one GEMM pair", f"{T}x{W}", us,
+                 gbytes=(w_in.numel() + w_dn.numel()) * 2 / 1e9, like="fused_moe (without the shared expert)")
             g = torch.randn(T, 2 * (E * I + Is), device=DEV, dtype=BF)
             us = timed(lambda: ops.expert_silu_all(g, tw, ti, E, I, Is), reps)
             emit("expert_silu_all", f"{T}x{E * I + Is}", us,
